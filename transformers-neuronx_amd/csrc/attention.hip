@@ -541,7 +541,8 @@ struct PrefillTileLayout {
 // What changes the scores, the mask and the result of the staged kernel (SCORED): a cap c on the scores
 // (c tanh(s / c)), a bias by the distance between query and key (`[heads, far + 1]` float32, read at
 // min(i - j, far); staged in LDS behind the tiles where `bias_in_lds`), visibility inside chunks of the request,
-// a gate on the result (the first `value_size` elements of a head times sigmoid(gate)), a factor on the result,
+// a sink in the softmax's denominator, a gate on the result (the first `value_size` elements of a head times
+// sigmoid(gate)), a factor on the result,
 // and result rows that lie `out_ld` elements apart.
 struct ScoreMods {
   float softcap;
@@ -553,6 +554,7 @@ struct ScoreMods {
   float out_scale;
   int value_size, vector_store;
   int gate_head;            // the gate's numbers a head: value_size (one an element) or 1 (one for the whole head)
+  const float* sink;        // [heads] or null: the softmax's denominator also holds exp(sink) of the head
 };
 
 __device__ __forceinline__ int first_visible_key(int pos, int window, int chunk) {
@@ -566,8 +568,8 @@ __device__ __forceinline__ float tanh_by_exp(float x) {
   return 1.f - 2.f * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * (2.f * LOG2E)));
 }
 
-// MODS: 0, the plain kernel; 1, everything `ScoreMods` names; 2, what it names of the result alone (the gate, the
-// factor, rows that lie apart), the scores and the mask being the plain ones: the tiles' loop is then the plain
+// MODS: 0, the plain kernel; 1, everything `ScoreMods` names; 2, what it names of the result alone (the sink, the
+// gate, the factor, rows that lie apart), the scores and the mask being the plain ones: the tiles' loop is then the plain
 // kernel's, with its registers.
 template <int NDB, bool FAST, int GROUPS, int MODS = 0>
 __global__ void __launch_bounds__(256 * GROUPS, (NDB <= 8 && GROUPS == 1 ? 2 : 1))
@@ -936,6 +938,7 @@ attention_prefill_lds_kernel(const bf16_t* __restrict__ q, const bf16_t* __restr
         const float a0 = __builtin_amdgcn_exp2f((m[qb] - m_safe) * LOG2E);
         const float a1 = __builtin_amdgcn_exp2f((m1 - m_safe) * LOG2E);
         l[qb] = l[qb] * a0 + l1 * a1;
+        m[qb] = m_safe;
 #pragma unroll
         for (int db = 0; db < NDB; ++db)
 #pragma unroll
@@ -950,7 +953,7 @@ attention_prefill_lds_kernel(const bf16_t* __restrict__ q, const bf16_t* __restr
     const int qi = qw0 + 16 * qb + r;
     if (qi >= qlen) continue;
     if (RESULT) {
-      const float inv = sm.out_scale / l[qb];
+      const float inv = sm.sink ? sm.out_scale * softmax_finish(m[qb], l[qb], sm.sink + h, nullptr) : sm.out_scale / l[qb];
       bf16_t* orow = out + (size_t)(t0 + qi) * sm.out_ld + h * head_size;
       const float* gate = sm.gate ? sm.gate + (size_t)(t0 + qi) * sm.gate_ld + (size_t)h * sm.gate_head : nullptr;
 #pragma unroll
@@ -1496,6 +1499,7 @@ attention_prefill_pipelined_kernel(const bf16_t* __restrict__ q, const bf16_t* _
         const float a0 = __builtin_amdgcn_exp2f((m[qb] - m_safe) * LOG2E);
         const float a1 = __builtin_amdgcn_exp2f((m1 - m_safe) * LOG2E);
         l[qb] = l[qb] * a0 + l1 * a1;
+        m[qb] = m_safe;
 #pragma unroll
         for (int db = 0; db < NDB; ++db)
 #pragma unroll
@@ -1510,7 +1514,7 @@ attention_prefill_pipelined_kernel(const bf16_t* __restrict__ q, const bf16_t* _
     const int qi = qw0 + 16 * qb + r;
     if (qi >= qlen) continue;
     if (RESULT) {
-      const float inv = sm.out_scale / l[qb];
+      const float inv = sm.sink ? sm.out_scale * softmax_finish(m[qb], l[qb], sm.sink + h, nullptr) : sm.out_scale / l[qb];
       bf16_t* orow = out + (size_t)(t0 + qi) * sm.out_ld + h * DH;
       const float* gate = sm.gate ? sm.gate + (size_t)(t0 + qi) * sm.gate_ld + (size_t)h * sm.gate_head : nullptr;
 #pragma unroll
@@ -1655,7 +1659,7 @@ extern "C" int tnx_attention_prefill_scored(const void* q, const void* k_pages, 
                                             const float* gate, long long gate_ld, const float* bias, int far,
                                             float softcap, int window, int chunk, int num_heads, int num_kv,
                                             int head_size, int value_size, int sets, int page_pad, int gate_head,
-                                            hipStream_t stream) {
+                                            const float* sink, hipStream_t stream) {
   TNX_REQUIRE(page_pad >= 0 && page_pad % 8 == 0, "attention_prefill_scored: bad distance between pages");
   TNX_REQUIRE(query_tile == PREFILL_Q_TILE, "attention_prefill_scored: tiles of %d queries, the kernels take %d",
               query_tile, PREFILL_Q_TILE);
@@ -1677,7 +1681,7 @@ extern "C" int tnx_attention_prefill_scored(const void* q, const void* k_pages, 
   int page_shift = 0;
   while ((1 << page_shift) < page_size) ++page_shift;
   ScoreMods sm{softcap, bias, far, 0, chunk, gate, gate_ld, out_ld, out_scale, value_size,
-               out_ld % 4 == 0 && ((uintptr_t)out & 7) == 0, gate_head};
+               out_ld % 4 == 0 && ((uintptr_t)out & 7) == 0, gate_head, sink};
   int rc = -1;
 #define SCORED_ARGS                                                                                              \
   grid, stream, (const bf16_t*)q, (const bf16_t*)k_pages, (const bf16_t*)v_pages, run_start, cached_lens, table, \

@@ -270,3 +270,22 @@ extern "C" int tnx_epilogue(const void* y, const float* bias, int act, const flo
   TNX_CHECK_LAUNCH("epilogue");
   return 0;
 }
+
+// In place: x <- scale * x, and with a cap c > 0, c tanh(x / c).
+__global__ void __launch_bounds__(256) scale_and_cap_kernel(float* __restrict__ x, float scale, float cap, size_t n) {
+  size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  const size_t stride = (size_t)gridDim.x * 256;
+  for (; i < n; i += stride) {
+    const float y = scale * x[i];
+    x[i] = cap > 0.f ? cap * tanhf(y / cap) : y;
+  }
+}
+
+extern "C" int tnx_scale_and_cap(float* x, float scale, float cap, long long n, hipStream_t stream) {
+  TNX_REQUIRE(n >= 0 && cap >= 0.f, "scale_and_cap: bad arguments");
+  if (n == 0) return 0;
+  const long long blocks = (n + 255) / 256;
+  scale_and_cap_kernel<<<(unsigned)(blocks < 4096 ? blocks : 4096), 256, 0, stream>>>(x, scale, cap, (size_t)n);
+  TNX_CHECK_LAUNCH("scale_and_cap");
+  return 0;
+}

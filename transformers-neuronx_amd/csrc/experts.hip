@@ -33,11 +33,16 @@ __device__ __forceinline__ float gated(float g, float u, int act, float limit) {
 // A wave a token: `top` rounds of the largest logit (the lower number where two are equal), whose score sigmoid(z)
 // or softmax(z) is the weight. The ranking is by the logits, which both scores grow with: two large logits that
 // float32 still tells apart can have scores that it does not. With `correction` (a number an expert) the ranking is
-// by score + correction, and the weight is the score without it; `scale` multiplies every weight.
+// by score + correction, and the weight is the score without it; `scale` multiplies every weight. With `keep` < `groups`
+// the experts form that many equal groups of neighbours, a group ranks by its best expert, and only experts of the `keep`
+// best groups (the lower number where two are equal) take part.
+constexpr int MAX_GROUPS = 256;
 __global__ void __launch_bounds__(256) route_kernel(const float* __restrict__ z, int tokens, int experts, int top,
                                                     int softmax, int renormalize, int* __restrict__ chosen,
                                                     float* __restrict__ weights, const float* __restrict__ correction,
-                                                    float scale) {
+                                                    float scale, int groups, int keep) {
+  __shared__ float best_of[4][MAX_GROUPS];        // a wave's groups: the best rank, and whether the group is kept
+  __shared__ unsigned char kept_of[4][MAX_GROUPS];
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= tokens) return;
   const float* row = z + (size_t)t * experts;
@@ -50,7 +55,32 @@ __global__ void __launch_bounds__(256) route_kernel(const float* __restrict__ z,
     total = wave_sum(s);
   }
   auto score = [&](float z) { return softmax ? expf(z - peak) / total : 1.f / (1.f + expf(-z)); };
-  auto rank = [&](int e) { return correction ? score(row[e]) + correction[e] : row[e]; };
+  auto plain_rank = [&](int e) { return correction ? score(row[e]) + correction[e] : row[e]; };
+  const int per = experts / groups;
+  const bool grouped = keep < groups;
+  if (grouped) {      // (a wave's own rows of LDS; a wave's LDS operations keep their order)
+    float* best = best_of[threadIdx.x >> 6];
+    unsigned char* kept = kept_of[threadIdx.x >> 6];
+    for (int g = 0; g < groups; ++g) {
+      float b = -INFINITY;
+      for (int e = lane; e < per; e += 64) b = fmaxf(b, plain_rank(g * per + e));
+      b = wave_max(b);
+      if (lane == 0) best[g] = b, kept[g] = 0;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    for (int c = 0; c < keep; ++c) {
+      float b = -INFINITY;
+      int at = groups;
+      for (int g = lane; g < groups; g += 64)
+        if (!kept[g] && (best[g] > b || at == groups)) b = best[g], at = g;
+      const float high = wave_max(b);
+      const int first = -(int)wave_max((float)-((b == high && at < groups) ? at : groups));
+      if (lane == 0 && first < groups) kept[first] = 1;
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    }
+  }
+  const unsigned char* kept = kept_of[threadIdx.x >> 6];
+  auto rank = [&](int e) { return !grouped || kept[e / per] ? plain_rank(e) : -INFINITY; };
   float sum = 0.f;
   unsigned long long taken = 0;        // bit i: expert lane + 64 i is chosen already (a lane's own experts)
   for (int c = 0; c < top; ++c) {
@@ -142,6 +172,7 @@ struct ProductArgs {
   void* out;
   int experts, top, n, k, act, weight_on_input, pairs;
   float limit;              // of the clamped activation
+  int direct;               // not GATED: pair rows are the tokens' rows of the result, and take the residual
 };
 
 template <typename T, bool GATED>
@@ -213,10 +244,8 @@ __global__ void __launch_bounds__(256) expert_product_kernel(ProductArgs p) {
     } else {
       float y = acc[0][r];
       if (!p.weight_on_input) y *= w;
-      if (p.top == 1)
-        ((float*)p.out)[(size_t)pair * p.n + col] = y + (p.residual ? p.residual[(size_t)pair * p.n + col] : 0.f);
-      else
-        ((float*)p.out)[(size_t)pair * p.n + col] = y;
+      if (p.direct && p.residual) y += p.residual[(size_t)pair * p.n + col];
+      ((float*)p.out)[(size_t)pair * p.n + col] = y;
     }
   }
 }
@@ -300,16 +329,20 @@ __global__ void __launch_bounds__(256) expert_product_mfma_kernel(ProductArgs p)
     } else {
       float y = acc[i];
       if (!p.weight_on_input) y *= w;
-      if (p.top == 1 && p.residual) y += p.residual[(size_t)pair * p.n + col];
+      if (p.direct && p.residual) y += p.residual[(size_t)pair * p.n + col];
       ((float*)p.out)[(size_t)pair * p.n + col] = y;
     }
   }
 }
 
-// (`place`: the row of y that holds pair t * top + c, where the rows lie in another order; `scale`: a factor a pair)
+// (`place`: the row of y that holds pair t * top + c, where the rows lie in another order; `scale`: a factor a pair.
+// With `same` a choice of `experts` or more is an expert without tensors: its row is the token's row of `same`, times the
+// pair's weight.)
+template <typename T>
 __global__ void combine_kernel(const float* __restrict__ y, const float* __restrict__ residual, float* __restrict__ out,
                                int top, size_t n, size_t total, const int* __restrict__ place,
-                               const float* __restrict__ scale) {
+                               const float* __restrict__ scale, const T* __restrict__ same,
+                               const int* __restrict__ chosen, const float* __restrict__ weights, int experts) {
   size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   const size_t stride = (size_t)gridDim.x * blockDim.x;
   for (; i < total; i += stride) {
@@ -317,6 +350,10 @@ __global__ void combine_kernel(const float* __restrict__ y, const float* __restr
     float s = residual ? residual[i] : 0.f;
     for (int c = 0; c < top; ++c) {
       const size_t pair = t * top + c;
+      if (same && chosen[pair] >= experts) {
+        s += weights[pair] * to_f32(same[i]);
+        continue;
+      }
       const float v = y[(place ? (size_t)place[pair] : pair) * n + col];
       s += scale ? scale[pair] * v : v;
     }
@@ -346,11 +383,15 @@ int blocks_for(size_t total) {
 }  // namespace
 
 extern "C" int tnx_route(const float* z, int tokens, int experts, int top, int softmax, int renormalize, int* chosen,
-                         float* weights, const float* correction, float scale, hipStream_t stream) {
+                         float* weights, const float* correction, float scale, int groups, int keep, hipStream_t stream) {
   TNX_REQUIRE(tokens >= 0 && experts > 0 && top > 0 && top <= experts, "route: %d of %d experts", top, experts);
+  TNX_REQUIRE(experts <= 4096, "route: up to 4096 experts, got %d", experts);
+  TNX_REQUIRE(groups >= 1 && groups <= MAX_GROUPS && experts % groups == 0 && keep >= 1 && keep <= groups &&
+                  top <= keep * (experts / groups),
+              "route: %d of %d experts in %d groups (up to %d) of which %d are kept", top, experts, groups, MAX_GROUPS, keep);
   if (tokens == 0) return 0;
   route_kernel<<<(tokens + 3) / 4, 256, 0, stream>>>(z, tokens, experts, top, softmax, renormalize, chosen, weights,
-                                                     correction, scale);
+                                                     correction, scale, groups, keep);
   TNX_CHECK_LAUNCH("route");
   return 0;
 }
@@ -359,11 +400,13 @@ extern "C" int tnx_expert_mixture(const void* h, const int* chosen, const float*
                                   const void* w_down, int* first, int* order, void* inner, float* pair_rows,
                                   const float* residual, float* out, int dtype, int tokens, int experts, int top,
                                   int width, int f, int act, int weight_on_input, int plain, float limit,
-                                  hipStream_t stream) {
+                                  int identity, hipStream_t stream) {
   TNX_REQUIRE(tokens >= 0 && experts > 0 && top > 0 && width > 0 && f > 0, "expert_mixture: bad sizes");
   TNX_REQUIRE(experts <= 4096, "expert_mixture: up to 4096 experts, got %d", experts);
   TNX_REQUIRE(dtype == TNX_F32 || dtype == TNX_BF16, "expert_mixture: dtype %d", dtype);
-  TNX_REQUIRE(top == 1 || pair_rows != nullptr, "expert_mixture: several choices a token need room for their rows");
+  const bool direct = top == 1 && !identity;
+  TNX_REQUIRE(direct || pair_rows != nullptr, "expert_mixture: several choices a token need room for their rows");
+  TNX_REQUIRE(!identity || !weight_on_input, "expert_mixture: experts without tensors take their weight on the output");
   if (tokens == 0) return 0;
   const int pairs = tokens * top;
   order_kernel<<<1, 1024, 2 * experts * sizeof(int), stream>>>(chosen, pairs, experts, first, order, nullptr, nullptr,
@@ -371,9 +414,9 @@ extern "C" int tnx_expert_mixture(const void* h, const int* chosen, const float*
   TNX_CHECK_LAUNCH("expert order");
   const int tiles = pairs / 16 + experts;       // the most tiles of 16 pairs: every expert may end in a part of one
   ProductArgs up{h, w_gate_up, first, order, weights, nullptr, inner, experts, top, f, width, act, weight_on_input, pairs,
-                 limit};
-  ProductArgs down{inner, w_down, first, order, weights, residual, top == 1 ? out : pair_rows, experts, top, width, f,
-                   act, weight_on_input, pairs, limit};
+                 limit, 0};
+  ProductArgs down{inner, w_down, first, order, weights, residual, direct ? out : pair_rows, experts, top, width, f,
+                   act, weight_on_input, pairs, limit, direct ? 1 : 0};
   const dim3 grid_up((f + 63) / 64, tiles), grid_down((width + 63) / 64, tiles);
   if (dtype == TNX_F32) {
     expert_product_kernel<float, true><<<grid_up, 256, 0, stream>>>(up);
@@ -386,10 +429,16 @@ extern "C" int tnx_expert_mixture(const void* h, const int* chosen, const float*
     expert_product_kernel<bf16_t, false><<<grid_down, 256, 0, stream>>>(down);
   }
   TNX_CHECK_LAUNCH("expert products");
-  if (top > 1) {
+  if (!direct) {
     const size_t total = (size_t)tokens * width;
-    combine_kernel<<<blocks_for(total), 256, 0, stream>>>(pair_rows, residual, out, top, (size_t)width, total, nullptr,
-                                                          nullptr);
+    if (dtype == TNX_F32)
+      combine_kernel<float><<<blocks_for(total), 256, 0, stream>>>(pair_rows, residual, out, top, (size_t)width, total, nullptr,
+                                                                   nullptr, identity ? (const float*)h : nullptr, chosen,
+                                                                   weights, experts);
+    else
+      combine_kernel<bf16_t><<<blocks_for(total), 256, 0, stream>>>(pair_rows, residual, out, top, (size_t)width, total, nullptr,
+                                                                    nullptr, identity ? (const bf16_t*)h : nullptr, chosen,
+                                                                    weights, experts);
     TNX_CHECK_LAUNCH("expert combine");
   }
   return 0;
@@ -423,13 +472,17 @@ extern "C" int tnx_expert_order(const int* chosen, const float* weights, int tok
   return 0;
 }
 
-// out[t] = residual[t] + sum_c scale[t, c] y[place[t * top + c]]
+// out[t] = residual[t] + sum_c scale[t, c] y[place[t * top + c]]; with `same` (bfloat16 rows) a choice of `experts` or more
+// adds scale[t, c] same[t]
 extern "C" int tnx_expert_combine(const float* y, const int* place, const float* scale, const float* residual, float* out,
-                                  int tokens, int top, int width, hipStream_t stream) {
+                                  int tokens, int top, int width, const void* same, const int* chosen, int experts,
+                                  hipStream_t stream) {
   TNX_REQUIRE(tokens >= 0 && top > 0 && width > 0, "expert_combine: bad sizes");
   if (tokens == 0) return 0;
   const size_t total = (size_t)tokens * width;
-  combine_kernel<<<blocks_for(total), 256, 0, stream>>>(y, residual, out, top, (size_t)width, total, place, scale);
+  TNX_REQUIRE(!same || (scale && chosen), "expert_combine: experts without tensors need the choices and their weights");
+  combine_kernel<bf16_t><<<blocks_for(total), 256, 0, stream>>>(y, residual, out, top, (size_t)width, total, place, scale,
+                                                                (const bf16_t*)same, chosen, scale, experts);
   TNX_CHECK_LAUNCH("expert combine");
   return 0;
 }

@@ -1,0 +1,603 @@
+// Linear memories: a matrix S [n, v] a head that is carried from token to token,
+//     S <- e^g S,   S <- S + k w^T,   o = S^T q,      w = write * val,  or with DELTA  w = write * (val - S^T k),
+// and what stands before and after them in a mixer:
+//   memory_inputs   a short causal convolution over time with silu, unit vectors a head, decays and write weights
+//   memory_walk     the recurrence token by token (decoded tokens, short runs)
+//   gated_norm      skip, gate and norm, up to what the output product reads
+// Everything is float32. State lies by position: the token at position p reads place (p - 1) & 1 of S's two (nothing at
+// p = 0) and writes place p & 1; the convolution's input at position p lies at place p mod taps. A step of single tokens
+// that is run twice reads the same both times.
+#include "common.h"
+
+TNX_DEFINE_ERROR_API
+
+namespace {
+
+__device__ __forceinline__ float silu(float x) { return x / (1.f + expf(-x)); }
+__device__ __forceinline__ float softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+
+// ------------------------------------------------------------------------------------------ what a memory reads
+
+struct InputArgs {
+  const float* proj;        // [T, ld]
+  int ld, conv_at, channels;
+  const float* w;           // [taps, channels]
+  const float* bias;        // [channels] or null
+  float* state;             // [slots, taps, channels]
+  int taps;
+  const int* positions;
+  const int* token_request;
+  const int* run_start;
+  const int* slots;
+  int unit_size, unit_count, scaled;      // the first unit_count channels are heads of unit_size, made unit vectors
+  float scale;                            // on the first `scaled` channels
+  float* u;                 // [T, channels]
+  int heads, dt_at, write_at;             // write_at < 0: the write weight is dt
+  const float* rate;        // [H]
+  const float* dt_bias;     // [H]
+  float* log_decay;         // [T, H]
+  float* write;             // [T, H]
+  int tokens, write_state;  // write_state: every run of the step is one token, so the state is written here
+};
+
+// A wave takes a piece of the channels for `per` consecutive tokens of the step: LANES: 256 channels, four a lane, where
+// unit heads are 4 * LANES elements (the sum of squares is then one over LANES lanes); LANES = 0, any sizes: a unit head,
+// or 256 channels, element lane + 64 e a lane. The inputs of the last taps - 1 tokens stay in registers while the run
+// goes on. Behind the channels' pieces come those of the gates, 64 heads a wave. TAPS 0: any number, read again for
+// every token.
+template <int LANES, int TAPS>
+__global__ void __launch_bounds__(256) memory_inputs_kernel(InputArgs a, int pieces, int per) {
+  const int lane = threadIdx.x & 63;
+  const int piece = blockIdx.x * 4 + (threadIdx.x >> 6);
+  const int t0 = blockIdx.y * per, t1 = min(a.tokens, t0 + per);
+  if (piece >= pieces) {      // the gates
+    const int head = 64 * (piece - pieces) + lane;
+    if (head >= a.heads) return;
+    for (int t = t0; t < t1; ++t) {
+      const float* row = a.proj + (size_t)t * a.ld;
+      const float dt = softplus(row[a.dt_at + head] + a.dt_bias[head]);
+      a.log_decay[(size_t)t * a.heads + head] = a.rate[head] * dt;
+      a.write[(size_t)t * a.heads + head] = a.write_at >= 0 ? 1.f / (1.f + expf(-row[a.write_at + head])) : dt;
+    }
+    return;
+  }
+  // this lane's channels: at[e], in[e]
+  int at[4];
+  bool in[4];
+  bool unit = false;
+  if (LANES > 0) {
+    const int c = 256 * piece + 4 * lane;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) at[e] = c + e, in[e] = c + e < a.channels;
+    unit = c < a.unit_count;
+  } else {
+    const int unit_pieces = a.unit_size > 0 ? a.unit_count / a.unit_size : 0;
+    unit = piece < unit_pieces;
+    const int first = unit ? piece * a.unit_size : a.unit_count + 256 * (piece - unit_pieces);
+    const int end = unit ? first + a.unit_size : a.channels;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) at[e] = first + lane + 64 * e, in[e] = at[e] < end;
+  }
+  const bool whole = LANES > 0 && in[3] && (a.channels & 3) == 0;       // four neighbours, 16 bytes aligned
+  constexpr int BACK = TAPS > 1 ? TAPS - 1 : 1;
+  float taps_w[TAPS > 0 ? TAPS : 1][4], bias[4], scale[4], before[BACK][4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const int c = in[e] ? at[e] : 0;
+    bias[e] = a.bias && in[e] ? a.bias[c] : 0.f;
+    scale[e] = at[e] < a.scaled ? a.scale : 1.f;
+#pragma unroll
+    for (int j = 0; j < (TAPS > 0 ? TAPS : 0); ++j) taps_w[j][e] = in[e] ? a.w[(size_t)j * a.channels + c] : 0.f;
+#pragma unroll
+    for (int b = 0; b < BACK; ++b) before[b][e] = 0.f;
+  }
+  const float* x = a.proj + a.conv_at;
+  const bool vec = whole && ((a.ld | a.conv_at) & 3) == 0;
+  auto load_row = [&](int t, float (&v)[4]) {
+    const float* row = x + (size_t)t * a.ld;
+    if (vec) {
+      const f32x4 got = *(const f32x4*)(row + at[0]);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = got[e];
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = in[e] ? row[at[e]] : 0.f;
+    }
+  };
+  auto load_back = [&](int t, int i, int p, int back, const float* mine, float (&v)[4]) {      // the input `back` tokens ago
+    if (back <= i) {
+      load_row(t - back, v);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = back <= p && in[e] ? mine[(size_t)((p - back) % a.taps) * a.channels + at[e]] : 0.f;
+    }
+  };
+  float next[4];
+  if (t0 < t1) load_row(t0, next);
+  for (int t = t0; t < t1; ++t) {
+    float now[4], acc[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) now[e] = next[e], acc[e] = bias[e];
+    if (t + 1 < t1) load_row(t + 1, next);
+    const int r = a.token_request[t], i = t - a.run_start[r], p = a.positions[t];
+    float* mine = a.state ? a.state + (size_t)a.slots[r] * a.taps * a.channels : nullptr;
+    if (TAPS > 0) {
+      if (TAPS > 1 && (t == t0 || i == 0)) {
+#pragma unroll
+        for (int b = 1; b < TAPS; ++b) load_back(t, i, p, b, mine, before[b - 1]);
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+#pragma unroll
+        for (int b = TAPS - 1; b >= 1; --b) acc[e] = fmaf(taps_w[TAPS - 1 - b][e], before[b - 1][e], acc[e]);
+        acc[e] = fmaf(taps_w[TAPS > 0 ? TAPS - 1 : 0][e], now[e], acc[e]);
+#pragma unroll
+        for (int b = BACK - 1; b >= 1; --b) before[b][e] = before[b - 1][e];
+        before[0][e] = now[e];
+      }
+    } else {
+      for (int b = a.taps - 1; b >= 0; --b) {
+        float v[4];
+        load_back(t, i, p, b, mine, v);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          acc[e] = fmaf(in[e] ? a.w[(size_t)(a.taps - 1 - b) * a.channels + at[e]] : 0.f, v[e], acc[e]);
+      }
+    }
+    if (a.write_state && a.taps > 1) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (in[e]) mine[(size_t)(p % a.taps) * a.channels + at[e]] = now[e];
+    }
+    float sum = 0.f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      acc[e] = in[e] ? silu(acc[e]) : 0.f;
+      sum += acc[e] * acc[e];
+    }
+    if (LANES == 0) {
+      if (unit) sum = wave_sum(sum);
+    } else if (a.unit_count > 0) {
+      sum += lane_dpp<TNX_DPP_XOR1>(sum);
+      sum += lane_dpp<TNX_DPP_XOR2>(sum);
+      sum += lane_dpp<TNX_DPP_HALF_MIRROR>(sum);
+      sum += lane_dpp<TNX_DPP_MIRROR>(sum);
+      if (LANES >= 32) {
+        unsigned lo, hi;
+        swap_rows(__float_as_uint(sum), lo, hi);
+        sum = __uint_as_float(lo) + __uint_as_float(hi);
+      }
+      if (LANES >= 64) {
+        unsigned lo, hi;
+        swap_halves(__float_as_uint(sum), lo, hi);
+        sum = __uint_as_float(lo) + __uint_as_float(hi);
+      }
+    }
+    const float f = unit ? 1.f / sqrtf(sum + 1e-6f) : 1.f;
+    float* out = a.u + (size_t)t * a.channels;
+    if (whole) {
+      f32x4 o;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) o[e] = acc[e] * f * scale[e];
+      *(f32x4*)(out + at[0]) = o;
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (in[e]) out[at[e]] = acc[e] * f * scale[e];
+    }
+  }
+}
+
+// the last taps - 1 inputs of every run, after the launch that read the state
+__global__ void __launch_bounds__(256) memory_state_kernel(InputArgs a) {
+  const int r = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
+  const int first = a.run_start[r], n = a.run_start[r + 1] - first;
+  if (c >= a.channels || n <= 0) return;
+  float* mine = a.state + (size_t)a.slots[r] * a.taps * a.channels;
+  for (int i = max(0, n - (a.taps - 1)); i < n; ++i)
+    mine[(size_t)(a.positions[first + i] % a.taps) * a.channels + c] = a.proj[(size_t)(first + i) * a.ld + a.conv_at + c];
+}
+
+// ------------------------------------------------------------------------------------------ the memory, token by token
+
+struct WalkArgs {
+  const float* u;           // [T, ld]
+  int ld, q_at, k_at, v_at;
+  const float* log_decay;   // [T, H]
+  const float* write;       // [T, H]
+  const int* run_start;     // [R + 1]
+  const int* cached;        // [R]
+  const int* slots;         // [R]
+  float* memory;            // [slots, 2, H, v, n]
+  float* out;               // [T, H v]
+  int heads, groups, n, v;
+  int longest;              // runs of more tokens than this are another kernel's (0: none are)
+};
+
+template <bool ALIGNED>
+__device__ __forceinline__ f32x4 load4(const float* p, int valid) {      // the first `valid` of four elements, zeros behind
+  f32x4 r = {0.f, 0.f, 0.f, 0.f};
+  if (valid <= 0) return r;
+  if (ALIGNED) return *(const f32x4*)p;
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+    if (e < valid) r[e] = p[e];
+  return r;
+}
+
+// sums over the 16 lanes of a row of lanes
+__device__ __forceinline__ float sum16(float x) {
+  x += lane_dpp<TNX_DPP_XOR1>(x);
+  x += lane_dpp<TNX_DPP_XOR2>(x);
+  x += lane_dpp<TNX_DPP_HALF_MIRROR>(x);
+  x += lane_dpp<TNX_DPP_MIRROR>(x);
+  return x;
+}
+
+// grid: requests * heads * column blocks; a block is four waves and 16 columns of S. In a wave the 16 lanes of a row of
+// lanes share a column (column 16 b + 4 w + lane / 16): lane % 16 holds its rows NR (lane % 16) + j, j < NR. CH tokens a
+// chunk go through LDS, the next chunk's loads under way meanwhile, a token's operands read a token ahead.
+// With DELTA S^T k, S^T q and k . q are summed side by side from the S that came in, and S'^T q = S^T q + w (k . q).
+template <int NR, int CH, bool DELTA, bool ALIGNED>
+__global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column_blocks) {
+  constexpr int np = 16 * NR;                             // a token's queries (and keys) in LDS, zeros behind n
+  constexpr int PT = np / 4;                              // 16-byte pieces of a token's queries
+  constexpr int QN = (CH * PT + 255) / 256;               // pieces of queries (and keys) a thread and chunk
+  __shared__ __attribute__((aligned(16))) float qs[CH * np];
+  __shared__ __attribute__((aligned(16))) float ks[CH * np];
+  __shared__ __attribute__((aligned(16))) float vs[CH * 16];
+  __shared__ float kp[CH], wr[CH];                        // e^g, write
+  const int cb = blockIdx.x % column_blocks, rh = blockIdx.x / column_blocks;
+  const int r = rh / a.heads, head = rh - r * a.heads;
+  const int group = head / (a.heads / a.groups);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int grp = lane & 15;
+  const int start = a.run_start[r], count = a.run_start[r + 1] - start;
+  const int have = a.cached[r], slot = a.slots[r];
+  if (count <= 0 || (a.longest > 0 && count > a.longest)) return;
+  const int col = 16 * cb + 4 * wave + (lane >> 4);
+  const bool col_ok = col < a.v;
+  float S[NR];
+  const int from = (have - 1) & 1, to = (have + count - 1) & 1;
+  const size_t head_at = (size_t)slot * 2 * a.heads + head;        // + place * heads
+  const float* Sp = a.memory + ((head_at + (size_t)from * a.heads) * a.v + (col_ok ? col : 0)) * a.n;
+  const bool live = have > 0 && col_ok;
+  if (NR % 4 == 0) {
+#pragma unroll
+    for (int j = 0; j < NR; j += 4) {
+      const int d = grp * NR + j;
+      const f32x4 got = load4<ALIGNED>(Sp + d, live ? a.n - d : 0);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) S[j + (NR % 4 == 0 ? e : 0)] = got[e];
+    }
+  } else {
+#pragma unroll
+    for (int j = 0; j < NR; ++j) S[j] = live && grp * NR + j < a.n ? Sp[grp * NR + j] : 0.f;
+  }
+  f32x4 rq[QN], rk[QN], rv = {0.f, 0.f, 0.f, 0.f};
+  float rkeep = 1.f, rwrite = 0.f;
+  auto fetch = [&](int t0) {
+    const int len = min(CH, count - t0);
+#pragma unroll
+    for (int u = 0; u < QN; ++u) {
+      const int f = threadIdx.x + 256 * u, t = f / PT, d = 4 * (f - t * PT);
+      const bool in = f < CH * PT && t < len;
+      const float* row = a.u + (size_t)(start + t0 + (in ? t : 0)) * a.ld + group * a.n + d;
+      rq[u] = load4<ALIGNED>(row + a.q_at, in ? a.n - d : 0);
+      rk[u] = load4<ALIGNED>(row + a.k_at, in ? a.n - d : 0);
+    }
+    if (threadIdx.x < CH * 4) {                            // a token's 16 values: four pieces
+      const int t = threadIdx.x >> 2, c = 16 * cb + 4 * (threadIdx.x & 3);
+      const bool in = t < len;
+      rv = load4<ALIGNED>(a.u + (size_t)(start + t0 + (in ? t : 0)) * a.ld + a.v_at + head * a.v + c, in ? a.v - c : 0);
+    }
+    if (threadIdx.x < CH) {
+      const bool in = threadIdx.x < len;
+      const size_t at = (size_t)(start + t0 + (in ? threadIdx.x : 0)) * a.heads + head;
+      rkeep = in ? expf(a.log_decay[at]) : 1.f;
+      rwrite = in ? a.write[at] : 0.f;
+    }
+  };
+  auto stash = [&]() {
+#pragma unroll
+    for (int u = 0; u < QN; ++u) {
+      const int f = threadIdx.x + 256 * u;                // piece f of the chunk: token f / PT, elements 4 (f % PT) on
+      if (f < CH * PT) {
+        *(f32x4*)(qs + 4 * f) = rq[u];
+        *(f32x4*)(ks + 4 * f) = rk[u];
+      }
+    }
+    if (threadIdx.x < CH * 4) *(f32x4*)(vs + 4 * threadIdx.x) = rv;
+    if (threadIdx.x < CH) kp[threadIdx.x] = rkeep, wr[threadIdx.x] = rwrite;
+  };
+  fetch(0);
+  stash();
+  __syncthreads();
+  for (int t0 = 0; t0 < count; t0 += CH) {
+    const int len = min(CH, count - t0);
+    const bool more = t0 + CH < count;
+    if (more) fetch(t0 + CH);                             // under way while this chunk is worked on
+    float q_n[NR], k_n[NR], val_n, keep_n, write_n;
+    auto read = [&](int t) {
+      const float* q = qs + t * np + grp * NR;
+      const float* k = ks + t * np + grp * NR;
+#pragma unroll
+      for (int j = 0; j < NR; ++j) q_n[j] = q[j], k_n[j] = k[j];
+      val_n = vs[t * 16 + 4 * wave + (lane >> 4)];
+      keep_n = kp[t];
+      write_n = wr[t];
+    };
+    auto token = [&](int t, bool last) {
+      float q[NR], k[NR];
+#pragma unroll
+      for (int j = 0; j < NR; ++j) q[j] = q_n[j], k[j] = k_n[j];
+      const float val = val_n, keep = keep_n, write = write_n;
+      if (!last) read(t + 1);
+      float o = 0.f;
+      if (DELTA) {
+        float sk = 0.f, sq = 0.f, kq = 0.f;
+#pragma unroll
+        for (int j = 0; j < NR; ++j) {
+          S[j] *= keep;
+          sk += S[j] * k[j];
+          sq += S[j] * q[j];
+          kq += k[j] * q[j];
+        }
+        sk = sum16(sk), sq = sum16(sq), kq = sum16(kq);
+        const float w = write * (val - sk);
+#pragma unroll
+        for (int j = 0; j < NR; ++j) S[j] += k[j] * w;
+        o = sq + w * kq;
+      } else {
+        const float w = write * val;
+#pragma unroll
+        for (int j = 0; j < NR; ++j) {
+          S[j] = keep * S[j] + k[j] * w;
+          o += S[j] * q[j];
+        }
+        o = sum16(o);
+      }
+      if (grp == 0 && col_ok) a.out[((size_t)(start + t0 + t) * a.heads + head) * a.v + col] = o;
+    };
+    read(0);
+    if (len == CH) {        // a whole chunk: a count the compiler knows
+#pragma unroll 4
+      for (int t = 0; t < CH; ++t) token(t, t == CH - 1);
+    } else {
+      for (int t = 0; t < len; ++t) token(t, t == len - 1);
+    }
+    __syncthreads();        // before the next chunk takes the place of what this one read
+    if (more) {
+      stash();
+      __syncthreads();
+    }
+  }
+  if (!col_ok) return;
+  float* Sw = a.memory + ((head_at + (size_t)to * a.heads) * a.v + col) * a.n;
+#pragma unroll
+  for (int j = 0; j < NR; ++j)
+    if (grp * NR + j < a.n) Sw[grp * NR + j] = S[j];
+}
+
+template <int NR, bool DELTA>
+void launch_walk(const WalkArgs& a, int requests, bool singles, bool aligned, hipStream_t stream) {
+  constexpr int CH = NR == 16 ? 16 : 32;
+  const int column_blocks = (a.v + 15) / 16;
+  const dim3 grid(requests * a.heads * column_blocks);
+  if (singles) {
+    if (aligned)
+      memory_walk_kernel<NR, 1, DELTA, true><<<grid, 256, 0, stream>>>(a, column_blocks);
+    else
+      memory_walk_kernel<NR, 1, DELTA, false><<<grid, 256, 0, stream>>>(a, column_blocks);
+  } else {
+    if (aligned)
+      memory_walk_kernel<NR, CH, DELTA, true><<<grid, 256, 0, stream>>>(a, column_blocks);
+    else
+      memory_walk_kernel<NR, CH, DELTA, false><<<grid, 256, 0, stream>>>(a, column_blocks);
+  }
+}
+
+template <bool DELTA>
+void launch_walk_sized(const WalkArgs& a, int requests, bool singles, bool aligned, hipStream_t stream) {
+  const int rows16 = (a.n + 15) / 16;
+  if (rows16 <= 2)
+    launch_walk<2, DELTA>(a, requests, singles, aligned, stream);
+  else if (rows16 <= 4)
+    launch_walk<4, DELTA>(a, requests, singles, aligned, stream);
+  else if (rows16 <= 8)
+    launch_walk<8, DELTA>(a, requests, singles, aligned, stream);
+  else
+    launch_walk<16, DELTA>(a, requests, singles, aligned, stream);
+}
+
+// ------------------------------------------------------------------------------------------ after the memory
+
+struct FinishArgs {
+  const float* o;           // [T, width]
+  const float* gate;        // [T, gate_ld]
+  long long gate_ld;
+  const float* weight;      // [width]
+  float eps;
+  int parts, gate_first;
+  const float* skip;        // [heads] or null
+  const float* x;           // [T, x_ld]
+  long long x_ld;
+  int per_head;             // elements a head
+  void* out;                // [T, width]
+  int tokens, width;
+};
+
+// A row's `parts` equal parts at unit root mean square, times weight; (o + skip x) silu(gate) before the norm or
+// silu(gate) after it. A part is THREADS threads' work, element by element or (VEC) four neighbours a thread.
+template <typename T, int THREADS, int VEC>
+__global__ void __launch_bounds__(256) gated_norm_kernel(FinishArgs a) {
+  __shared__ float scratch[4];
+  constexpr int PER_BLOCK = 256 / THREADS;
+  const long long idx = (long long)blockIdx.x * PER_BLOCK + (THREADS == 256 ? 0 : threadIdx.x >> 6);
+  const bool active = idx < (long long)a.tokens * a.parts;
+  if (THREADS < 256 && !active) return;
+  const size_t t = active ? idx / a.parts : 0;
+  const int part = active ? (int)(idx - (long long)t * a.parts) : 0;
+  const int size = a.width / a.parts, first = part * size;
+  const int me = THREADS == 256 ? threadIdx.x : threadIdx.x & 63;
+  const float* o = a.o + t * a.width + first;
+  const float* gate = a.gate + t * a.gate_ld + first;
+  const float* x = a.skip ? a.x + t * a.x_ld + first : nullptr;
+  auto value = [&](int i) {
+    float y = o[i];
+    if (x) y += a.skip[(first + i) / a.per_head] * x[i];
+    if (a.gate_first) y *= silu(gate[i]);
+    return y;
+  };
+  constexpr int HELD = 4;              // so many pieces of a part stay in registers between the two passes
+  float held[HELD][VEC];
+  float s = 0.f;
+#pragma unroll
+  for (int c = 0; c < HELD; ++c) {
+    const int i = VEC * (me + THREADS * c);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      held[c][e] = i + e < size ? value(i + e) : 0.f;
+      s += held[c][e] * held[c][e];
+    }
+  }
+  for (int i = VEC * (me + THREADS * HELD); i < size; i += VEC * THREADS)
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      const float y = i + e < size ? value(i + e) : 0.f;
+      s += y * y;
+    }
+  s = THREADS == 256 ? block_sum<4>(s, scratch) : wave_sum(s);
+  const float r = 1.f / sqrtf(s / (float)size + a.eps);
+  T* out = (T*)a.out + t * a.width + first;
+  const float* w = a.weight + first;
+  auto put = [&](int i, float y) {
+    y *= r * w[i];
+    if (!a.gate_first) y *= silu(gate[i]);
+    out[i] = from_f32<T>(y);
+  };
+#pragma unroll
+  for (int c = 0; c < HELD; ++c) {
+    const int i = VEC * (me + THREADS * c);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e)
+      if (i + e < size) put(i + e, held[c][e]);
+  }
+  for (int i = VEC * (me + THREADS * HELD); i < size; i += VEC * THREADS)
+#pragma unroll
+    for (int e = 0; e < VEC; ++e)
+      if (i + e < size) put(i + e, value(i + e));
+}
+
+template <typename T>
+void launch_gated_norm(const FinishArgs& a, hipStream_t stream) {
+  const int size = a.width / a.parts;
+  const long long rows = (long long)a.tokens * a.parts;
+  if (size <= 64)
+    gated_norm_kernel<T, 64, 1><<<(unsigned)((rows + 3) / 4), 256, 0, stream>>>(a);
+  else if (size <= 256)
+    gated_norm_kernel<T, 64, 4><<<(unsigned)((rows + 3) / 4), 256, 0, stream>>>(a);
+  else
+    gated_norm_kernel<T, 256, 4><<<(unsigned)rows, 256, 0, stream>>>(a);
+}
+
+}  // namespace
+
+extern "C" int tnx_memory_inputs(const float* proj, int ld, int conv_at, int channels, const float* w, const float* bias,
+                                 float* state, int taps, const int* positions, const int* token_request,
+                                 const int* run_start, const int* slots, int unit_size, int unit_count, int scaled,
+                                 float scale, float* u, int heads, int dt_at, int write_at, const float* rate,
+                                 const float* dt_bias, float* log_decay, float* write, int tokens, int runs,
+                                 hipStream_t stream) {
+  TNX_REQUIRE(tokens >= 0 && runs >= 0 && channels > 0 && taps >= 1 && heads > 0, "memory_inputs: bad sizes");
+  TNX_REQUIRE(conv_at >= 0 && ld >= conv_at + channels && dt_at >= 0 && ld >= dt_at + heads && ld >= write_at + heads,
+              "memory_inputs: rows of %d elements do not hold what is read", ld);
+  TNX_REQUIRE(taps == 1 || state, "memory_inputs: %d taps need the requests' state", taps);
+  TNX_REQUIRE(unit_count >= 0 && unit_count <= channels && scaled <= channels &&
+                  (unit_count == 0 || (unit_size > 0 && unit_size <= 256 && unit_count % unit_size == 0)),
+              "memory_inputs: %d channels in unit heads of %d (up to 256 elements)", unit_count, unit_size);
+  TNX_REQUIRE(runs < 65536, "memory_inputs: too many runs");
+  if (tokens == 0 || runs == 0) return 0;
+  const bool singles = tokens == runs;
+  InputArgs a{proj, ld, conv_at, channels, w, bias, taps > 1 ? state : nullptr, taps, positions, token_request, run_start, slots,
+              unit_count ? unit_size : 0, unit_count, scaled, scale, u, heads, dt_at, write_at, rate, dt_bias, log_decay, write,
+              tokens, singles};
+  int lanes = 0;
+  if (unit_count == 0 || unit_size == 64)
+    lanes = 16;
+  else if (unit_size == 128)
+    lanes = 32;
+  else if (unit_size == 256)
+    lanes = 64;
+  const int pieces = lanes ? (channels + 255) / 256 : unit_count / unit_size + (channels - unit_count + 255) / 256;
+  const int gates = (heads + 63) / 64;
+  // tokens a wave: as many as leave the chip a few waves a compute unit, up to 16
+  int per = 1;
+  while (per < 16 && (long long)(pieces + gates) * (tokens / (2 * per)) >= 8 * tnx_compute_units()) per *= 2;
+  const long long rows = (tokens + per - 1) / per;
+  TNX_REQUIRE(rows < 65536, "memory_inputs: too many tokens");
+  const dim3 grid((pieces + gates + 3) / 4, (unsigned)rows);
+#define INPUTS_LAUNCH(L, N) memory_inputs_kernel<L, N><<<grid, 256, 0, stream>>>(a, pieces, per)
+#define INPUTS_TAPS(L)                        \
+  if (taps == 1) INPUTS_LAUNCH(L, 1);         \
+  else if (taps == 2) INPUTS_LAUNCH(L, 2);    \
+  else if (taps == 3) INPUTS_LAUNCH(L, 3);    \
+  else if (taps == 4) INPUTS_LAUNCH(L, 4);    \
+  else INPUTS_LAUNCH(L, 0)
+  if (lanes == 16) {
+    INPUTS_TAPS(16);
+  } else if (lanes == 32) {
+    INPUTS_TAPS(32);
+  } else if (lanes == 64) {
+    INPUTS_TAPS(64);
+  } else {
+    INPUTS_TAPS(0);
+  }
+#undef INPUTS_TAPS
+#undef INPUTS_LAUNCH
+  TNX_CHECK_LAUNCH("memory_inputs");
+  if (taps > 1 && !singles) {
+    memory_state_kernel<<<dim3((channels + 255) / 256, runs), 256, 0, stream>>>(a);
+    TNX_CHECK_LAUNCH("memory_state");
+  }
+  return 0;
+}
+
+extern "C" int tnx_memory_walk(const float* u, int ld, int q_at, int k_at, int v_at, const float* log_decay,
+                               const float* write, const int* run_start, const int* cached, const int* slots, float* memory,
+                               float* out, int tokens, int requests, int heads, int groups, int n, int v, int delta,
+                               int longest, hipStream_t stream) {
+  TNX_REQUIRE(tokens >= 0 && requests >= 0 && heads > 0 && groups > 0 && heads % groups == 0 && n > 0 && v > 0,
+              "memory_walk: bad sizes");
+  TNX_REQUIRE(n <= 256, "memory_walk: query/key heads of up to 256 elements, got %d", n);
+  TNX_REQUIRE(q_at >= 0 && k_at >= 0 && v_at >= 0 && ld >= q_at + groups * n && ld >= k_at + groups * n && ld >= v_at + heads * v,
+              "memory_walk: rows of %d elements do not hold what is read", ld);
+  if (tokens == 0 || requests == 0) return 0;
+  TNX_REQUIRE((long long)requests * heads * ((v + 15) / 16) < (1ll << 31), "memory_walk: too many blocks");
+  WalkArgs a{u, ld, q_at, k_at, v_at, log_decay, write, run_start, cached, slots, memory, out, heads, groups, n, v, longest};
+  // rows and heads that begin at multiples of 16 bytes are loaded 16 bytes at a time
+  const bool aligned = n % 4 == 0 && v % 4 == 0 && ((ld | q_at | k_at | v_at) & 3) == 0 && (uintptr_t)u % 16 == 0;
+  if (delta)
+    launch_walk_sized<true>(a, requests, tokens == requests, aligned, stream);
+  else
+    launch_walk_sized<false>(a, requests, tokens == requests, aligned, stream);
+  TNX_CHECK_LAUNCH("memory_walk");
+  return 0;
+}
+
+extern "C" int tnx_gated_norm(const float* o, const float* gate, long long gate_ld, const float* weight, float eps, int parts,
+                              int gate_first, const float* skip, int skip_heads, const float* x, long long x_ld, void* out,
+                              int dtype, int tokens, int width, hipStream_t stream) {
+  TNX_REQUIRE(tokens >= 0 && width > 0 && parts > 0 && width % parts == 0 && gate_ld >= width, "gated_norm: bad sizes");
+  TNX_REQUIRE(!skip || (skip_heads > 0 && width % skip_heads == 0 && x && x_ld >= width), "gated_norm: bad skip");
+  TNX_REQUIRE(dtype == TNX_F32 || dtype == TNX_BF16, "gated_norm: dtype %d", dtype);
+  TNX_REQUIRE((long long)tokens * parts < (1ll << 31), "gated_norm: too many rows");
+  if (tokens == 0) return 0;
+  FinishArgs a{o, gate, gate_ld, weight, eps, parts, gate_first, skip, x, x_ld, skip ? width / skip_heads : 1, out, tokens, width};
+  if (dtype == TNX_F32)
+    launch_gated_norm<float>(a, stream);
+  else
+    launch_gated_norm<bf16_t>(a, stream);
+  TNX_CHECK_LAUNCH("gated_norm");
+  return 0;
+}

@@ -33,7 +33,15 @@ struct PrepareArgs {
   int per_head;             // every head is normed by itself (the weights, if any, still one a projection element)
   int values_at;            // the column of a row where the values begin (behind the keys, or the keys' own)
   const float* head_scale;  // [H] or null: a query head's elements times its number, beside `scale`
+  float temp_coef;          // the queries of position p times 1 + temp_coef ln(floor((p + 1) / temp_every) + 1)
+  int temp_every;           // 0: not
 };
+
+// what the token's queries are multiplied by, beside a head's own number
+__device__ __forceinline__ float query_scale(const PrepareArgs& a, int t) {
+  if (a.temp_every <= 0) return a.scale;
+  return a.scale * (1.f + a.temp_coef * logf((float)((a.positions[t] + 1) / a.temp_every + 1)));
+}
 
 // Element `e` of head `head` of a normed projection, turned by the token's position. `x` points at the
 // projection's first head, `w` at its norm weight (or null), `r` is the factor of the norm.
@@ -87,6 +95,7 @@ __global__ void __launch_bounds__(256) qkv_prepare_kernel(PrepareArgs a) {
     }
     return;
   }
+  const float scale = part == 0 ? query_scale(a, t) : 1.f;
   if (a.freqs != nullptr) {
     const float pos = (float)a.positions[t];
     for (int i = threadIdx.x; i < a.half; i += 256) sincosf(pos * a.freqs[i], &sines[i], &cosines[i]);
@@ -108,7 +117,7 @@ __global__ void __launch_bounds__(256) qkv_prepare_kernel(PrepareArgs a) {
       for (int e = lane; e < a.d; e += 64) {
         const float val = e < a.n ? turned(x, w, r, head, e, a, cosines, sines) : 0.f;
         if (part == 0)
-          q_out[head * a.d + e] = from_f32<T>(val * (a.head_scale ? a.scale * a.head_scale[head] : a.scale));
+          q_out[head * a.d + e] = from_f32<T>(val * (a.head_scale ? scale * a.head_scale[head] : scale));
         else
           kp[((size_t)head * a.page_size + off) * a.d + e] = from_f32<T>(val);
       }
@@ -128,7 +137,7 @@ __global__ void __launch_bounds__(256) qkv_prepare_kernel(PrepareArgs a) {
     for (int i = threadIdx.x; i < heads * a.d; i += 256) {
       const int head = i / a.d, e = i - head * a.d;
       q_out[i] = from_f32<T>(e < a.n ? turned(x, w, norm, head, e, a, cosines, sines) *
-                                           (a.head_scale ? a.scale * a.head_scale[head] : a.scale)
+                                           (a.head_scale ? scale * a.head_scale[head] : scale)
                                      : 0.f);
     }
   } else {
@@ -147,7 +156,8 @@ extern "C" int tnx_qkv_prepare(const float* proj, int ld, const float* q_weight,
                                const float* mix_weight, const float* first, long long first_ld, const int* token_page,
                                const int* token_offset, void* q_out, void* k_pages, void* v_pages, long long page_stride,
                                int num_pages, int page_size, int dtype, int tokens, int heads, int groups, int n, int v,
-                               int d, int per_head, int values_at, const float* head_scale, hipStream_t stream) {
+                               int d, int per_head, int values_at, const float* head_scale, float temp_coef, int temp_every,
+                               hipStream_t stream) {
   TNX_REQUIRE(tokens >= 0 && heads > 0 && groups > 0 && n > 0 && v > 0, "qkv_prepare: bad sizes");
   TNX_REQUIRE(d >= n && d >= v, "qkv_prepare: cached heads of %d elements do not hold %d and %d", d, n, v);
   if (values_at < 0) values_at = heads * n + groups * n;
@@ -161,7 +171,7 @@ extern "C" int tnx_qkv_prepare(const float* proj, int ld, const float* q_weight,
   if (tokens == 0) return 0;
   PrepareArgs a{proj, ld, q_weight, k_weight, eps, freqs, half, interleaved, positions, scale, mix_weight, first, first_ld,
                 token_page, token_offset, q_out, k_pages, v_pages, page_stride, num_pages, page_size, heads, groups, n, v, d,
-                per_head, values_at, head_scale};
+                per_head, values_at, head_scale, temp_coef, temp_every};
   if (dtype == TNX_F32)
     qkv_prepare_kernel<float><<<dim3(tokens, 3), 256, 0, stream>>>(a);
   else

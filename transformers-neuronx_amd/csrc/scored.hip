@@ -1,5 +1,6 @@
 // Attention whose scores or mask are not the plain ones: a cap on the scores (c tanh(s / c)), a learned bias by
-// the distance between query and key, visibility inside chunks of the sequence, and a gate on the result.
+// the distance between query and key, visibility inside chunks of the sequence, a sink in the softmax's denominator, and
+// a gate on the result.
 //   attention_scored_any   one wave per (token, head), any dtype, any head size in steps of 16: the float32 path
 //                          and whatever the matrix-unit kernels do not take
 //   attention_scored_tiles bfloat16 on MFMA 16x16x32: a block takes 128 queries of a run of several tokens for
@@ -33,7 +34,13 @@ struct ScoredArgs {
   float softcap;            // 0: none
   int window, chunk;        // 0: none
   int tokens, num_heads, num_kv, head_size, value_size, page_pad;
+  const float* sink;        // [H] or null: the softmax's denominator also holds exp(sink) of the head
 };
+
+// What a head's maximum and sum make of its weighted values: the factor on the result, with the sink in the denominator.
+__device__ __forceinline__ float finish(const ScoredArgs& a, float m, float l, int head) {
+  return a.sink ? a.out_scale * softmax_finish(m, l, a.sink + head, nullptr) : a.out_scale / l;
+}
 
 __device__ __forceinline__ float exp_for(float x, float) { return expf(x); }
 __device__ __forceinline__ float exp_for(float x, bf16_t) { return __expf(x); }
@@ -118,7 +125,7 @@ __global__ void __launch_bounds__(256) attention_scored_any_kernel(ScoredArgs a)
       }
     }
   }
-  const float inv = a.out_scale / l;
+  const float inv = finish(a, m, l, h);
   T* out = (T*)a.out + (size_t)t * a.out_ld + (size_t)h * head_size;
   const float* gate = a.gate ? a.gate + (size_t)t * a.gate_ld + (size_t)h * a.gate_head : nullptr;
 #pragma unroll
@@ -380,7 +387,7 @@ attention_scored_tiles_kernel(ScoredArgs a, const int* __restrict__ run_start, c
   for (int qb = 0; qb < 2; ++qb) {
     const int qi = qw0 + 16 * qb + r;
     if (qi >= qlen) continue;
-    const float inv = a.out_scale / l[qb];
+    const float inv = finish(a, m[qb], l[qb], h);
 #pragma unroll
     for (int db = 0; db < NDB; ++db) {
       if (db >= ndb) continue;
@@ -491,7 +498,7 @@ attention_scored_single_kernel(ScoredArgs a, const int* __restrict__ run_start, 
       if (db < ndb) *(f32x4*)(mine + 4 + 16 * db + 4 * g) = o[db][0];
     return;
   }
-  const float inv = a.out_scale / l[0];
+  const float inv = finish(a, m[0], l[0], head);
 #pragma unroll
   for (int db = 0; db < NDB; ++db) {
     if (db >= ndb) continue;
@@ -515,6 +522,7 @@ attention_scored_join_kernel(ScoredArgs a, const int* __restrict__ run_start, co
     const float ms = mine[s * stride];
     ll += ms == -INFINITY ? 0.f : mine[s * stride + 1] * __expf(ms - mm);
   }
+  const float inv = finish(a, mm, ll, head);
   bf16_t* orow = (bf16_t*)a.out + (size_t)token * a.out_ld + (size_t)head * a.head_size;
   const float* gate = a.gate ? a.gate + (size_t)token * a.gate_ld + (size_t)head * a.gate_head : nullptr;
   for (int d = threadIdx.x; d < a.head_size; d += 64) {
@@ -523,7 +531,7 @@ attention_scored_join_kernel(ScoredArgs a, const int* __restrict__ run_start, co
       const float ms = mine[s * stride];
       if (ms != -INFINITY) oo += mine[s * stride + 4 + d] * __expf(ms - mm);
     }
-    float x = oo * a.out_scale / ll;
+    float x = oo * inv;
     if (gate && d < a.value_size) x *= 1.f / (1.f + __expf(-gate[a.gate_head == 1 ? 0 : d]));
     orow[d] = (bf16_t)x;
   }
@@ -536,7 +544,7 @@ extern "C" int tnx_attention_scored(const void* q, int dtype, const void* k_page
                                     int page_size, int num_pages, void* out, long long out_ld, float out_scale,
                                     const float* gate, long long gate_ld, const float* bias, int far, float softcap,
                                     int window, int chunk, int tokens, int num_heads, int num_kv, int head_size,
-                                    int value_size, int page_pad, int gate_head, hipStream_t stream) {
+                                    int value_size, int page_pad, int gate_head, const float* sink, hipStream_t stream) {
   TNX_REQUIRE(tokens >= 0 && num_heads > 0 && num_kv > 0 && num_heads % num_kv == 0, "attention_scored: bad head counts");
   TNX_REQUIRE(page_pad >= 0 && page_pad % 8 == 0, "attention_scored: bad distance between pages");
   TNX_REQUIRE(head_size % 16 == 0 && head_size >= 16 && head_size <= 256,
@@ -555,7 +563,7 @@ extern "C" int tnx_attention_scored(const void* q, int dtype, const void* k_page
   TNX_REQUIRE(blocks < (1ll << 31), "attention_scored: too many (token, head) pairs");
   ScoredArgs a{q, k_pages, v_pages, positions, token_request, table, table_width, page_size, num_pages, out, out_ld,
                out_scale, gate, gate_ld, gate_head, bias, far, softcap, window, chunk, tokens, num_heads, num_kv, head_size,
-               value_size, page_pad};
+               value_size, page_pad, sink};
   if (dtype == TNX_F32)
     attention_scored_any_kernel<float><<<(unsigned)blocks, 256, 0, stream>>>(a);
   else
@@ -573,7 +581,8 @@ extern "C" int tnx_attention_scored_mfma(const void* q, const void* k_pages, con
                                          long long out_ld, float out_scale, const float* gate, long long gate_ld,
                                          const float* bias, int far, float softcap, int window, int chunk,
                                          int num_heads, int num_kv, int head_size, int value_size, int page_pad,
-                                         int splits, float* partial, int gate_head, hipStream_t stream) {
+                                         int splits, float* partial, int gate_head, const float* sink,
+                                         hipStream_t stream) {
   TNX_REQUIRE(num_heads > 0 && num_kv > 0 && num_heads % num_kv == 0, "attention_scored_mfma: bad head counts");
   TNX_REQUIRE(splits >= 1 && splits <= 64 && (splits == 1 || partial),
               "attention_scored_mfma: %d blocks a decoded token need a workspace", splits);
@@ -592,7 +601,7 @@ extern "C" int tnx_attention_scored_mfma(const void* q, const void* k_pages, con
   TNX_REQUIRE(num_single < 65536 * 1024 && num_kv < 65536, "attention_scored_mfma: too many runs or heads");
   ScoredArgs a{q, k_pages, v_pages, nullptr, nullptr, table, table_width, page_size, num_pages, out, out_ld,
                out_scale, gate, gate_ld, gate_head, bias, far, softcap, window, chunk, 0, num_heads, num_kv, head_size,
-               value_size, page_pad};
+               value_size, page_pad, sink};
   const int vector_store = out_ld % 4 == 0 && ((uintptr_t)out & 7) == 0;
   const int pack = num_heads / num_kv;
   const size_t budget = 64 * 1024;

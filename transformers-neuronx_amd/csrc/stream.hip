@@ -394,6 +394,146 @@ extern "C" int tnx_norm_add(const float* y, const float* weight, const float* bi
   return 0;
 }
 
+// ------------------------------------------------------------------------------------------------ a sum, then the norm
+
+// The norm that follows a sum: out = r / sqrt(mean(r^2) + eps) * weight, r = alpha x + fa za + fb zb, where z is the row
+// y itself or, with a norm weight w, y / sqrt(mean(y^2) + part_eps) * w; the second row may be missing. A float32 result
+// and, if asked for, a copy in another dtype.
+struct JoinArgs {
+  const float* x;
+  float alpha;
+  const float* ya;
+  const float* wa;
+  float fa;
+  const float* yb;          // null: one row
+  const float* wb;
+  float fb, part_eps;
+  const float* weight;
+  float eps;
+  float* out;
+  void* copy;
+  int copy_dtype, width;
+};
+
+// Sums of two numbers over a block of four waves.
+__device__ __forceinline__ void block_sum_two(float& a, float& b, float* scratch) {      // scratch: 8 floats
+  a = wave_sum(a);
+  b = wave_sum(b);
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  if (lane == 0) scratch[w] = a, scratch[4 + w] = b;
+  __syncthreads();
+  a = (scratch[0] + scratch[1]) + (scratch[2] + scratch[3]);
+  b = (scratch[4] + scratch[5]) + (scratch[6] + scratch[7]);
+}
+
+template <int PER, bool TWO>
+__global__ void __launch_bounds__(256) join_norm_rows_kernel(JoinArgs a) {
+  __shared__ float scratch[12];
+  const int w4 = a.width >> 2;
+  const size_t base = (size_t)blockIdx.x * a.width;
+  rf4 r[PER], ya[PER], yb[TWO ? PER : 1], wa[PER], wb[TWO ? PER : 1], g[PER];
+  row_load<PER>(a.x + base, w4, r);
+  row_load<PER>(a.ya + base, w4, ya);
+  if (TWO) row_load<TWO ? PER : 1>(a.yb + base, w4, yb);
+  vector_load<PER>(a.wa, w4, 1.f, wa);
+  if (TWO) vector_load<TWO ? PER : 1>(a.wb, w4, 1.f, wb);
+  vector_load<PER>(a.weight, w4, 0.f, g);
+  float fa = a.fa, fb = a.fb;
+  if (a.wa || (TWO && a.wb)) {
+    float sa = 0.f, sb = 0.f;
+#pragma unroll
+    for (int c = 0; c < PER; ++c) {
+      sa += (ya[c].x * ya[c].x + ya[c].y * ya[c].y) + (ya[c].z * ya[c].z + ya[c].w * ya[c].w);
+      if (TWO) sb += (yb[c].x * yb[c].x + yb[c].y * yb[c].y) + (yb[c].z * yb[c].z + yb[c].w * yb[c].w);
+    }
+    block_sum_two(sa, sb, scratch);
+    if (a.wa) fa *= 1.f / sqrtf(sa / (float)a.width + a.part_eps);
+    if (TWO && a.wb) fb *= 1.f / sqrtf(sb / (float)a.width + a.part_eps);
+  }
+  float s = 0.f;
+#pragma unroll
+  for (int c = 0; c < PER; ++c) {
+    r[c] = a.alpha * r[c] + fa * ya[c] * wa[c];
+    if (TWO) r[c] = r[c] + fb * yb[c] * wb[c];
+    s += (r[c].x * r[c].x + r[c].y * r[c].y) + (r[c].z * r[c].z + r[c].w * r[c].w);      // (zeros beyond the row)
+  }
+  const float rstd = 1.f / sqrtf(block_sum<4>(s, scratch + 8) / (float)a.width + a.eps);
+#pragma unroll
+  for (int c = 0; c < PER; ++c) {
+    const int i = threadIdx.x + 256 * c;
+    if (i < w4) {
+      const rf4 h = r[c] * rstd * g[c];
+      ((rf4*)(a.out + base))[i] = h;
+      if (a.copy) store_chunk(a.copy, a.copy_dtype, (base >> 2) + i, h);
+    }
+  }
+}
+
+// Any width: the rows are read from memory (from cache, after the first time) in every pass.
+__global__ void __launch_bounds__(256) join_norm_kernel(JoinArgs a) {
+  __shared__ float scratch[12];
+  const size_t base = (size_t)blockIdx.x * a.width;
+  float fa = a.fa, fb = a.yb ? a.fb : 0.f;
+  float sa = 0.f, sb = 0.f;
+  if (a.wa || (a.yb && a.wb)) {
+    for (int i = threadIdx.x; i < a.width; i += 256) {
+      const float u = a.ya[base + i], v = a.yb ? a.yb[base + i] : 0.f;
+      sa += u * u;
+      sb += v * v;
+    }
+    block_sum_two(sa, sb, scratch);
+    if (a.wa) fa *= 1.f / sqrtf(sa / (float)a.width + a.part_eps);
+    if (a.yb && a.wb) fb *= 1.f / sqrtf(sb / (float)a.width + a.part_eps);
+  }
+  auto sum_at = [&](int i) {
+    float r = a.alpha * a.x[base + i] + fa * a.ya[base + i] * (a.wa ? a.wa[i] : 1.f);
+    if (a.yb) r += fb * a.yb[base + i] * (a.wb ? a.wb[i] : 1.f);
+    return r;
+  };
+  float s = 0.f;
+  for (int i = threadIdx.x; i < a.width; i += 256) {
+    const float r = sum_at(i);
+    s += r * r;
+  }
+  const float rstd = 1.f / sqrtf(block_sum<4>(s, scratch + 8) / (float)a.width + a.eps);
+  for (int i = threadIdx.x; i < a.width; i += 256) {
+    const float h = sum_at(i) * rstd * a.weight[i];
+    a.out[base + i] = h;
+    if (a.copy) store_any(a.copy, a.copy_dtype, base + i, h);
+  }
+}
+
+extern "C" int tnx_join_norm(const float* x, float alpha, const float* ya, const float* wa, float fa, const float* yb,
+                             const float* wb, float fb, float part_eps, const float* weight, float eps, float* out,
+                             void* copy, int copy_dtype, int tokens, int width, hipStream_t stream) {
+  TNX_REQUIRE(tokens >= 0 && width > 0 && eps > 0.f && part_eps > 0.f, "join_norm: bad sizes tokens=%d width=%d", tokens, width);
+  TNX_REQUIRE(x && ya && weight && out && out != x && out != ya && out != yb, "join_norm: the result lies where a row is read");
+  TNX_REQUIRE(copy_dtype == TNX_F32 || copy_dtype == TNX_BF16, "join_norm: dtype %d", copy_dtype);
+  if (tokens == 0) return 0;
+  const JoinArgs a{x, alpha, ya, wa, fa, yb, wb, fb, part_eps, weight, eps, out, copy, copy_dtype, width};
+  if (rows_fit(width) && width <= 8192) {
+#define JOIN_LAUNCH(PER)                                                   \
+  if (yb)                                                                  \
+    join_norm_rows_kernel<PER, true><<<tokens, 256, 0, stream>>>(a);       \
+  else                                                                     \
+    join_norm_rows_kernel<PER, false><<<tokens, 256, 0, stream>>>(a)
+    if (width <= 1024) {
+      JOIN_LAUNCH(1);
+    } else if (width <= 2048) {
+      JOIN_LAUNCH(2);
+    } else if (width <= 4096) {
+      JOIN_LAUNCH(4);
+    } else {
+      JOIN_LAUNCH(8);
+    }
+#undef JOIN_LAUNCH
+  } else {
+    join_norm_kernel<<<tokens, 256, 0, stream>>>(a);
+  }
+  TNX_CHECK_LAUNCH("join_norm");
+  return 0;
+}
+
 // See `join_norm_conv_kernel`. `h_keep` `[tokens, width]` floats is needed unless every run is one token
 // (`single_runs`); widths that `tnx_rows_fit` takes only.
 extern "C" int tnx_rows_fit(int width) { return rows_fit(width) ? 1 : 0; }

@@ -31,6 +31,7 @@ _SIGNATURES = {
                               _c_int, _c_int, _c_int, _c_float, _c_void_p],
         "tnx_cast": [_c_void_p, _c_int, _c_void_p, _c_int, _c_ll, _c_void_p],
         "tnx_epilogue": [_c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
+        "tnx_scale_and_cap": [_c_void_p, _c_float, _c_float, _c_ll, _c_void_p],
         "tnx_layernorm": [_c_void_p, _c_void_p, _c_void_p, _c_float, _c_void_p, _c_void_p, _c_int, _c_int, _c_int,
                           _c_int, _c_void_p],
     },
@@ -64,7 +65,7 @@ _SIGNATURES = {
         "tnx_attention_prefill_scored": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int,
                                          _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p, _c_ll, _c_float,
                                          _c_void_p, _c_ll, _c_void_p, _c_int, _c_float, _c_int, _c_int, _c_int, _c_int,
-                                         _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+                                         _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p],
         "tnx_attention_prefill": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int,
                                   _c_int, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int,
                                   _c_int, _c_int, _c_int, _c_void_p],
@@ -91,6 +92,8 @@ _SIGNATURES = {
         "tnx_norm_add": [_c_void_p, _c_void_p, _c_void_p, _c_float, _c_int, _c_void_p, _c_float, _c_void_p, _c_void_p,
                          _c_int, _c_int, _c_int, _c_void_p],
         "tnx_rows_fit": [_c_int],
+        "tnx_join_norm": [_c_void_p, _c_float, _c_void_p, _c_void_p, _c_float, _c_void_p, _c_void_p, _c_float, _c_float,
+                          _c_void_p, _c_float, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
         "tnx_join_norm_conv": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_float, _c_void_p, _c_void_p,
                                _c_void_p, _c_int, _c_float, _c_void_p, _c_void_p, _c_ll, _c_int, _c_void_p, _c_void_p,
                                _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int,
@@ -126,7 +129,7 @@ _SIGNATURES = {
         "tnx_qkv_prepare": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_float, _c_void_p, _c_int, _c_int, _c_void_p,
                             _c_float, _c_void_p, _c_void_p, _c_ll, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                             _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                            _c_int, _c_void_p, _c_void_p],
+                            _c_int, _c_void_p, _c_float, _c_int, _c_void_p],
     },
     "memory": {
         "tnx_matrix_memory": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
@@ -135,14 +138,15 @@ _SIGNATURES = {
     },
     "experts": {
         "tnx_route": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_float,
-                      _c_void_p],
+                      _c_int, _c_int, _c_void_p],
         "tnx_expert_mixture": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                                _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                               _c_int, _c_int, _c_float, _c_void_p],
+                               _c_int, _c_int, _c_float, _c_int, _c_void_p],
         "tnx_gated_activation": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_float, _c_void_p],
         "tnx_expert_order": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                              _c_void_p, _c_void_p],
-        "tnx_expert_combine": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
+        "tnx_expert_combine": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p,
+                               _c_void_p, _c_int, _c_void_p],
     },
     "hyper": {
         "tnx_add_sinusoid": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int,
@@ -163,10 +167,20 @@ _SIGNATURES = {
         "tnx_attention_scored_mfma": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int,
                                       _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p, _c_int, _c_void_p, _c_ll,
                                       _c_float, _c_void_p, _c_ll, _c_void_p, _c_int, _c_float, _c_int, _c_int, _c_int,
-                                      _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_int, _c_void_p],
+                                      _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p],
         "tnx_attention_scored": [_c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int,
                                  _c_int, _c_void_p, _c_ll, _c_float, _c_void_p, _c_ll, _c_void_p, _c_int, _c_float,
-                                 _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+                                 _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p,
+                                 _c_void_p],
+    },
+    "linear_memory": {
+        "tnx_memory_inputs": [_c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p,
+                              _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_float, _c_void_p, _c_int, _c_int,
+                              _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p],
+        "tnx_memory_walk": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
+                            _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+        "tnx_gated_norm": [_c_void_p, _c_void_p, _c_ll, _c_void_p, _c_float, _c_int, _c_int, _c_void_p, _c_int, _c_void_p,
+                           _c_ll, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
     },
     "probe": {
         "tnx_probe_stream_read": [_c_void_p, ctypes.c_size_t, _c_void_p, _c_int, _c_void_p],
@@ -1116,6 +1130,29 @@ class HipOps:
             return out
         return out, (copy if copy is not None else self.cast(out, self.dtype))
 
+    def join_norm(self, x, alpha, results, weight, eps, dtype):
+        """See `ReferenceOps.join_norm`."""
+        _want(x, "x", torch.float32)
+        t, width = x.shape
+        _want(weight, "norm weight", torch.float32, (width,))
+        if not 1 <= len(results) <= 2:
+            raise ValueError(f"join_norm takes one or two results, got {len(results)}")
+        part_eps = {float(e) for _, w, e, _ in results if w is not None}
+        if len(part_eps) > 1:
+            raise ValueError("join_norm: the two results' norms have one eps")
+        for y, w, _, _ in results:
+            _want(y, "a part's result", torch.float32, (t, width))
+            if w is not None:
+                _want(w, "a result's norm weight", torch.float32, (width,))
+        (ya, wa, _, fa), (yb, wb, _, fb) = results[0], results[1] if len(results) > 1 else (None, None, None, 0.0)
+        out = torch.empty_like(x)
+        copy = torch.empty(t, width, dtype=dtype, device=x.device) if dtype != torch.float32 else None
+        self._call("stream", "tnx_join_norm", _ptr(x), float(alpha), _ptr(ya), _ptr(wa), float(fa), _ptr(yb), _ptr(wb),
+                   float(fb), part_eps.pop() if part_eps else 1.0, _ptr(weight), float(eps), _ptr(out), _ptr(copy), _code(dtype),
+                   t, width, _stream(),
+                   work=(f"{t}x{width}x{len(results)}", t * width * (8.0 + 4.0 * len(results) + (2 if copy is not None else 0)), 0.0))
+        return out, (copy if copy is not None else out)
+
     fuse_rows = 64       # up to this many rows the join, the norm and the convolution are one launch
 
     @staticmethod
@@ -1424,7 +1461,7 @@ class HipOps:
 
     def qkv_prepare(self, proj, num_heads, num_kv, head_size, value_size, cache_head, q_weight, k_weight, eps, freqs,
                     interleaved, scale, mix_weight, first_values, ctx, view, k_pages, v_pages, per_head=False,
-                    values_at=None, head_scale=None):
+                    values_at=None, head_scale=None, temperature=None):
         """See `ReferenceOps.qkv_prepare`. The rows of `proj` may hold more behind the values."""
         t = ctx.num_tokens
         need = num_heads * head_size + num_kv * head_size
@@ -1458,7 +1495,8 @@ class HipOps:
                    _ptr(view.token_page), _ptr(view.token_offset), _ptr(q), _ptr(k_pages), _ptr(v_pages),
                    k_pages.stride(0), num_pages, view.page_size, _code(self.dtype), t, num_heads, num_kv, head_size,
                    value_size, cache_head, int(bool(per_head)), -1 if values_at is None else int(values_at),
-                   _ptr(head_scale), _stream(),
+                   _ptr(head_scale), float(temperature[0]) if temperature else 0.0, int(temperature[1]) if temperature else 0,
+                   _stream(),
                    work=(f"{t}x{total}", t * (total * 4 + (num_heads + 2 * num_kv) * cache_head * q.element_size()), 0.0))
         return q
 
@@ -1522,9 +1560,11 @@ class HipOps:
 
     def attention_scored(self, q, num_heads, num_kv_heads, head_size, ctx, view, k_pages, v_pages, window=None,
                          chunk=None, softcap=None, distance_bias=None, gate=None, value_size=None, out=None,
-                         out_scale=1.0, gate_per_head=False):
+                         out_scale=1.0, gate_per_head=False, sink=None):
         """See `ReferenceOps.attention_scored`."""
         t = ctx.num_tokens
+        if sink is not None:
+            _want(sink, "sinks", torch.float32, (num_heads,))
         value_size = head_size if value_size is None else value_size
         _want(q, "q", self.dtype, (t, num_heads * head_size))
         num_pages = self._check_pages(k_pages, v_pages, num_kv_heads, head_size, view.page_size)
@@ -1557,7 +1597,7 @@ class HipOps:
                            num_pages, _ptr(tiles), _ptr(ctx.plan["tile_start"]), tiles.numel(), QUERY_TILE, _ptr(out), out_ld,
                            float(out_scale), _ptr(gate), gate_ld, _ptr(distance_bias), far, float(softcap or 0.0),
                            int(window or 0), int(chunk or 0), num_heads, num_kv_heads, head_size, value_size, sets, pad,
-                           gate_head, _stream(), work=work)
+                           gate_head, _ptr(sink), _stream(), work=work)
             if not staged or single.numel():
                 splits, partial = self._scored_splits(ctx, single.numel(), num_heads, num_kv_heads, head_size, window, chunk)
                 self._call("scored", "tnx_attention_scored_mfma", _ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(ctx.run_start),
@@ -1565,13 +1605,13 @@ class HipOps:
                            _ptr(ctx.plan["tile_start"]), 0 if staged else tiles.numel(), QUERY_TILE, _ptr(single),
                            single.numel(), _ptr(out), out_ld, float(out_scale), _ptr(gate), gate_ld, _ptr(distance_bias), far,
                            float(softcap or 0.0), int(window or 0), int(chunk or 0), num_heads, num_kv_heads, head_size,
-                           value_size, pad, splits, _ptr(partial), gate_head, _stream(), work=None if staged else work)
+                           value_size, pad, splits, _ptr(partial), gate_head, _ptr(sink), _stream(), work=None if staged else work)
             return out
         self._call("scored", "tnx_attention_scored", _ptr(q), _code(self.dtype), _ptr(k_pages), _ptr(v_pages),
                    _ptr(ctx.positions), _ptr(ctx.token_request), _ptr(view.block_table), view.width, view.page_size,
                    num_pages, _ptr(out), out_ld, float(out_scale), _ptr(gate), gate_ld, _ptr(distance_bias), far,
                    float(softcap or 0.0), int(window or 0), int(chunk or 0), t, num_heads, num_kv_heads, head_size,
-                   value_size, pad, gate_head, _stream(), work=work)
+                   value_size, pad, gate_head, _ptr(sink), _stream(), work=work)
         return out
 
     scored_decode_splits = None       # tests set it: the blocks that share a decoded token's keys
@@ -1690,9 +1730,72 @@ class HipOps:
                    work=(f"{t} tokens {ctx.num_requests} runs", state + t * total * 4.0, 4.0 * t * h * n * v))
         return out
 
+    # ---------------------------------------------------------------- linear memories
+
+    def memory_inputs(self, proj, conv_at, weight, bias, ctx, state, heads, dt_at, rate, dt_bias, write_at=None, unit=None):
+        """See `ReferenceOps.memory_inputs`."""
+        t = ctx.num_tokens
+        _want(proj, "projections", torch.float32)
+        channels, taps = weight.shape
+        if proj.dim() != 2 or proj.shape[0] != t:
+            raise ValueError(f"projections must be [{t}, columns], got {tuple(proj.shape)}")
+        _want(weight, "convolution weights", torch.float32)
+        if bias is not None:
+            _want(bias, "convolution bias", torch.float32, (channels,))
+        if taps > 1:
+            _want(state, "convolution state", torch.float32, (state.shape[0], taps, channels))
+        _want(rate, "rates", torch.float32, (heads,))
+        _want(dt_bias, "dt bias", torch.float32, (heads,))
+        size, count, scaled, scale = unit if unit is not None else (0, 0, 0, 1.0)
+        u = torch.empty(t, channels, dtype=torch.float32, device=proj.device)
+        gates = torch.empty(2, t, heads, dtype=torch.float32, device=proj.device)
+        self._call("linear_memory", "tnx_memory_inputs", _ptr(proj), proj.shape[1], int(conv_at), channels,
+                   _ptr(self._taps_first(weight)), _ptr(bias), _ptr(state) if taps > 1 else None, taps, _ptr(ctx.positions),
+                   _ptr(ctx.token_request), _ptr(ctx.run_start), _ptr(ctx.slots), int(size), int(count), int(scaled),
+                   float(scale), _ptr(u), heads, int(dt_at), -1 if write_at is None else int(write_at), _ptr(rate),
+                   _ptr(dt_bias), _ptr(gates[0]), _ptr(gates[1]), t, ctx.num_requests, _stream(),
+                   work=(f"{t}x{channels}", t * channels * 8.0 + ctx.num_requests * (taps - 1) * channels * 8.0, 0.0))
+        return u, gates[0], gates[1]
+
+    def linear_memory(self, u, q_at, k_at, v_at, heads, groups, n, v, log_decay, write, ctx, memory, delta):
+        """See `ReferenceOps.linear_memory`."""
+        t = ctx.num_tokens
+        _want(u, "queries, keys and values", torch.float32)
+        if u.dim() != 2 or u.shape[0] != t:
+            raise ValueError(f"queries, keys and values must be [{t}, columns], got {tuple(u.shape)}")
+        _want(log_decay, "decays", torch.float32, (t, heads))
+        _want(write, "write weights", torch.float32, (t, heads))
+        _want(memory, "memory", torch.float32, (memory.shape[0], 2, heads, v, n))
+        out = torch.empty(t, heads * v, dtype=torch.float32, device=u.device)
+        state = float(ctx.num_requests) * heads * n * v * 8
+        work = (f"{t} tokens {ctx.num_requests} runs", state + t * (u.shape[1] + heads * v) * 4.0,
+                (6.0 if delta else 4.0) * t * heads * n * v)
+        self._call("linear_memory", "tnx_memory_walk", _ptr(u), u.shape[1], int(q_at), int(k_at), int(v_at), _ptr(log_decay),
+                   _ptr(write), _ptr(ctx.run_start), _ptr(ctx.cached_lens), _ptr(ctx.slots), _ptr(memory), _ptr(out), t,
+                   ctx.num_requests, heads, groups, n, v, int(bool(delta)), 0, _stream(), work=work)
+        return out
+
+    def gated_norm(self, o, gate, weight, eps, parts, gate_first, skip=None):
+        """See `ReferenceOps.gated_norm`."""
+        _want(o, "the memory's result", torch.float32)
+        t, width = o.shape
+        gate_ld = self._rows_apart(gate, "the gate", torch.float32, t, width)
+        _want(weight, "norm weight", torch.float32, (width,))
+        factors, x, x_ld = None, None, 0
+        if skip is not None:
+            factors, x = skip
+            _want(factors, "skip factors", torch.float32)
+            x_ld = self._rows_apart(x, "the skipped input", torch.float32, t, width)
+        out = torch.empty(t, width, dtype=self.dtype, device=o.device)
+        self._call("linear_memory", "tnx_gated_norm", _ptr(o), _ptr(gate), gate_ld, _ptr(weight), float(eps), int(parts),
+                   int(bool(gate_first)), _ptr(factors), factors.numel() if factors is not None else 0, _ptr(x), x_ld, _ptr(out),
+                   _code(self.dtype), t, width, _stream(),
+                   work=(f"{t}x{width}", t * width * (8.0 + (4 if skip is not None else 0) + out.element_size()), 0.0))
+        return out
+
     # ---------------------------------------------------------------- experts
 
-    def route(self, z, top, score="sigmoid", renormalize=False, correction=None, scale=1.0):
+    def route(self, z, top, score="sigmoid", renormalize=False, correction=None, scale=1.0, groups=None):
         """See `ReferenceOps.route`."""
         _want(z, "router logits", torch.float32)
         t, experts = z.shape
@@ -1702,8 +1805,9 @@ class HipOps:
         weights = torch.empty(t, top, dtype=torch.float32, device=z.device)
         if correction is not None:
             _want(correction, "the choice's correction", torch.float32, (experts,))
+        count, keep = groups if groups is not None else (1, 1)
         self._call("experts", "tnx_route", _ptr(z), t, experts, top, int(score == "softmax"), int(bool(renormalize)),
-                   _ptr(chosen), _ptr(weights), _ptr(correction), float(scale), _stream())
+                   _ptr(chosen), _ptr(weights), _ptr(correction), float(scale), int(count), int(keep), _stream())
         return chosen, weights
 
     def gated_activation(self, gate_up, activation, row_weights=None, limit=None):
@@ -1729,13 +1833,14 @@ class HipOps:
     expert_plain_products = False      # tests set it: the kernel without the matrix unit in bfloat16 too
 
     def expert_mixture(self, h, chosen, weights, w_gate_up, w_down, activation, weight_on, residual=None, may_wait=False,
-                       limit=None):
+                       limit=None, identity=0):
         """See `ReferenceOps.expert_mixture`. `may_wait`: the step is not being recorded, so the host may read
-        what the device has made."""
+        what the device has made. `identity`: how many experts without tensors the numbers behind the experts' stand
+        for."""
         t, top = chosen.shape
         experts, two_f, width = w_gate_up.shape
         f = two_f // 2
-        if activation not in _GATE_ACT or weight_on not in ("input", "output"):
+        if activation not in _GATE_ACT or weight_on not in ("input", "output") or (identity and weight_on == "input"):
             raise ValueError(f"expert_mixture: activation {activation!r}, weight_on {weight_on!r}")
         _want(h, "h", w_gate_up.dtype, (t, width))
         _want(chosen, "chosen experts", torch.int32)
@@ -1775,23 +1880,29 @@ class HipOps:
                 inner = self.gated_activation(gu, activation, scale[a:b] if on_input else None, limit=limit)
                 self.linear(inner, w_down[e], None, out_f32=True, f32_by_library=True, into=y[a:b])
             self._call("experts", "tnx_expert_combine", _ptr(y), _ptr(place), None if on_input else _ptr(weights),
-                       _ptr(residual), _ptr(out), t, top, width, _stream(),
+                       _ptr(residual), _ptr(out), t, top, width, _ptr(h) if identity else None, _ptr(chosen), experts, _stream(),
                        work=(f"{t}x{top}x{width}", (pairs + 2.0 * t) * width * 4, 0.0))
             return out
         ints = torch.empty(experts + 1 + pairs, dtype=torch.int32, device=dev)
         inner = torch.empty(pairs, f, dtype=h.dtype, device=dev)
-        rows = torch.empty(pairs, width, dtype=torch.float32, device=dev) if top > 1 else None
+        rows = torch.empty(pairs, width, dtype=torch.float32, device=dev) if top > 1 or identity else None
         item = h.element_size()
         used = min(experts, pairs)
         self._call("experts", "tnx_expert_mixture", _ptr(h), _ptr(chosen), _ptr(weights), _ptr(w_gate_up), _ptr(w_down),
                    _ptr(ints[:experts + 1]), _ptr(ints[experts + 1:]), _ptr(inner), _ptr(rows), _ptr(residual), _ptr(out),
                    _code(h.dtype), t, experts, top, width, f, _GATE_ACT[activation], int(weight_on == "input"),
-                   int(bool(self.expert_plain_products)), float(limit or 0.0), _stream(),
+                   int(bool(self.expert_plain_products)), float(limit or 0.0), int(identity), _stream(),
                    work=(f"{t}x{top} of {experts}", used * 3.0 * f * width * item + t * width * (item + 8.0),
                          6.0 * t * top * f * width))
         return out
 
     # ---------------------------------------------------------------- output end
+
+    def scale_and_cap(self, logits, scale, cap):
+        """See `ReferenceOps.scale_and_cap`."""
+        _want(logits, "logits", torch.float32)
+        self._call("elementwise", "tnx_scale_and_cap", _ptr(logits), float(scale), float(cap or 0.0), logits.numel(), _stream())
+        return logits
 
     def ban_tokens(self, logits, tokens):
         """In place: `logits[i, tokens[i]] = -inf` where `tokens[i] >= 0`."""

@@ -255,6 +255,17 @@ class ReferenceOps:
             result = out
         return (result, result.to(self.dtype)) if want_compute else result
 
+    def join_norm(self, x, alpha, results, weight, eps, dtype):
+        """The norm that follows a sum, `h = r / sqrt(mean(r^2) + eps) * weight` with
+        `r = alpha x + sum_k factor_k z_k`, `results` = [(y, norm weight, norm eps, factor), ...] (one or two of them):
+        z = y, or, where a norm weight is given, y / sqrt(mean(y^2) + norm eps) * norm weight. All float32. Returns
+        (h in float32, h in `dtype`)."""
+        r = alpha * x.float()
+        for y, w, e, factor in results:
+            z = y.float() if w is None else self.layernorm(y, w, None, e, torch.float32, True, False, center=False)[0]
+            r = r + factor * z
+        return self.layernorm(r, weight, None, eps, dtype, True, True, center=False)
+
     def join_norm_conv(self, x, join, pre, conv_w, state, which, ctx, dtype):
         """What a part reads: `h = pre_norm(x')`, the result `h + conv(h)` as `input_conv` makes it, with `x' = x`,
         or for `join` = (y, weight, bias, center, mult), `x' = x + mult * post_norm(y)`. `pre` = (weight, bias,
@@ -446,7 +457,7 @@ class ReferenceOps:
 
     def qkv_prepare(self, proj, num_heads, num_kv, head_size, value_size, cache_head, q_weight, k_weight, eps, freqs,
                     interleaved, scale, mix_weight, first_values, ctx, view, k_pages, v_pages, per_head=False,
-                    values_at=None, head_scale=None):
+                    values_at=None, head_scale=None, temperature=None):
         """From the float32 projections `proj` `[T, H n + G n + G v]` (bias added) to the queries and the cache:
         the queries and the keys are each scaled to unit root mean square over their whole width and weighted
         (`q_weight`, `k_weight`; None: not), the first `2 len(freqs)` elements of every head are turned by
@@ -456,7 +467,8 @@ class ReferenceOps:
         tokens' places in the pages, heads filled up with zeros to `cache_head` elements; the queries come back
         `[T, H cache_head]`, filled up alike, in the compute dtype. `values_at`: the column of a row where the
         values begin, if not behind the keys (the keys' own first column: the values are the keys as projected).
-        `head_scale` (float32 `[H]`): a query head's elements are multiplied by its number as well."""
+        `head_scale` (float32 `[H]`): a query head's elements are multiplied by its number as well. `temperature` =
+        (coef, every): the queries of the token at position p are multiplied by 1 + coef ln(floor((p + 1) / every) + 1)."""
         t = proj.shape[0]
         nq, nk, nv = num_heads * head_size, num_kv * head_size, num_kv * value_size
         x = proj.float()
@@ -502,17 +514,22 @@ class ReferenceOps:
         out = torch.zeros(t, num_heads, cache_head, dtype=self.dtype, device=proj.device)
         if head_scale is not None:
             q = q * head_scale.float()[None, :, None]
+        if temperature is not None:
+            coef, every = temperature
+            ages = torch.div(ctx.positions.long() + 1, int(every), rounding_mode="floor") + 1
+            q = q * (1.0 + float(coef) * torch.log(ages.float()))[:, None, None]
         out[:, :, :head_size] = (q * scale).to(self.dtype)
         return out.reshape(t, num_heads * cache_head)
 
     def attention_scored(self, q, num_heads, num_kv_heads, head_size, ctx, view, k_pages, v_pages, window=None,
                          chunk=None, softcap=None, distance_bias=None, gate=None, value_size=None, out=None,
-                         out_scale=1.0, gate_per_head=False):
+                         out_scale=1.0, gate_per_head=False, sink=None):
         """Attention whose scores or mask are not the plain ones. For a query at position i and a key at j <= i of
         its request: s = q . k (the query comes scaled); with `softcap` c, s <- c tanh(s / c); with
         `distance_bias` (float32 `[heads, D + 1]`), s <- s + distance_bias[head, min(i - j, D)]. Visible are the
         keys with i - j < window (if given) and floor(j / chunk) = floor(i / chunk) (if given). Softmax over the
-        visible keys, times the values. `gate` (float32 `[T, heads * value_size]`, rows may lie apart): the first
+        visible keys, times the values; `sink` (float32 `[heads]`): the softmax's denominator also holds exp(sink) of the
+        head, once. `gate` (float32 `[T, heads * value_size]`, rows may lie apart): the first
         `value_size` elements of every head are multiplied by sigmoid(gate) (`gate_per_head`: `[T, heads]`, one
         number for all elements of a head). The result times `out_scale` goes to
         `out` (`[T, heads * head_size]` in the compute dtype, rows may lie apart) or to a new tensor."""
@@ -549,8 +566,7 @@ class ReferenceOps:
                 allowed &= j > pos - window
             if chunk is not None:
                 allowed &= (j // chunk) == (pos // chunk)
-            scores = scores.masked_fill(~allowed.unsqueeze(0), float("-inf"))
-            p = torch.softmax(scores, dim=-1)
+            p = self._with_sink(scores, allowed, sink)
             res[s:e] = (p @ vals.transpose(1, 2)).permute(1, 0, 2)
         if gate is not None:
             res[:, :, :value_size] *= torch.sigmoid(gate.float()).reshape(t, num_heads, 1 if gate_per_head else value_size)
@@ -694,17 +710,97 @@ class ReferenceOps:
         y = out.reshape(t, h * v) * norm_weight.float() * torch.sigmoid(gate)
         return y.to(self.dtype)
 
+    # ---------------------------------------------------------------- linear memories
+
+    def memory_inputs(self, proj, conv_at, weight, bias, ctx, state, heads, dt_at, rate, dt_bias, write_at=None, unit=None):
+        """What a linear memory reads of a step's tokens, from the float32 projections `proj` `[T, columns]`.
+
+        u = silu(conv(x)) over the columns x from `conv_at` on, one a channel of `weight` `[channels, taps]`: a causal
+        convolution over the tokens of a request (`bias` `[channels]` or None, zeros before its start; `state`
+        `[slots, taps, channels]` as in `channel_conv`). `unit` = (size, count, scaled, scale): the first `count`
+        channels are heads of `size` elements, each made a unit vector, x / sqrt(sum(x^2) + 1e-6), and the first
+        `scaled` channels are multiplied by `scale`.
+        dt = softplus(columns from `dt_at` on + dt_bias), one a head; the decay's logarithm is rate * dt (`rate` `[H]`,
+        negative); the write weight is dt, or sigmoid of the columns from `write_at` on.
+        Returns (u float32 `[T, channels]`, log decays `[T, H]`, write weights `[T, H]`)."""
+        channels = weight.shape[0]
+        none = torch.zeros(channels, dtype=torch.float32, device=proj.device)
+        u, _ = self.channel_conv(proj[:, conv_at:conv_at + channels], weight, none if bias is None else bias, ctx, state)
+        u = u * torch.sigmoid(u)
+        if unit is not None:
+            size, count, scaled, scale = unit
+            heads_of = u[:, :count].reshape(u.shape[0], -1, size)
+            heads_of = heads_of / torch.sqrt((heads_of * heads_of).sum(-1, keepdim=True) + 1e-6)
+            u[:, :count] = heads_of.reshape(u.shape[0], count)
+            u[:, :scaled] *= scale
+        dt = torch.nn.functional.softplus(proj[:, dt_at:dt_at + heads].float() + dt_bias.float(), threshold=1e9)
+        write = dt if write_at is None else torch.sigmoid(proj[:, write_at:write_at + heads].float())
+        return u, dt * rate.float(), write
+
+    def linear_memory(self, u, q_at, k_at, v_at, heads, groups, n, v, log_decay, write, ctx, memory, delta):
+        """A matrix S `[n, v]` a head that is carried from token to token: S <- e^log_decay S, S <- S + k w^T with
+        w = write * val, or, with `delta`, w = write * (val - S^T k), and o = S^T q. Queries, keys and values are
+        columns of `u` float32 `[T, columns]` from `q_at`, `k_at`, `v_at` on; queries and keys come in `groups` heads,
+        head h takes number h // (heads / groups). `memory` float32 `[slots, 2, heads, v, n]` (a column's rows side by
+        side): the token at position p reads place (p - 1) & 1 (zeros at p = 0) and writes place p & 1. Returns
+        float32 `[T, heads * v]`."""
+        t = u.shape[0]
+        share = torch.arange(heads, device=u.device) // (heads // groups)
+        q = u[:, q_at:q_at + groups * n].reshape(t, groups, n)[:, share]
+        k = u[:, k_at:k_at + groups * n].reshape(t, groups, n)[:, share]
+        val = u[:, v_at:v_at + heads * v].reshape(t, heads, v)
+        decay = torch.exp(log_decay)
+        out = torch.empty(t, heads, v, dtype=torch.float32, device=u.device)
+        start = 0
+        for r in range(ctx.num_requests):
+            count, slot, have = int(ctx.run_lens_host[r]), int(ctx.slots_host[r]), int(ctx.cached_lens_host[r])
+            s = memory[slot, (have - 1) & 1].clone() if have > 0 else torch.zeros_like(memory[slot, 0])       # [H, v, n]
+            for i in range(start, start + count):
+                s = s * decay[i][:, None, None]
+                w = val[i]
+                if delta:
+                    w = w - torch.einsum("hvn,hn->hv", s, k[i])
+                s = s + (write[i][:, None] * w)[:, :, None] * k[i][:, None, :]
+                out[i] = torch.einsum("hvn,hn->hv", s, q[i])
+            if count:
+                memory[slot, (have + count - 1) & 1] = s
+            start += count
+        return out.reshape(t, heads * v)
+
+    def gated_norm(self, o, gate, weight, eps, parts, gate_first, skip=None):
+        """What follows a memory up to the output product: rows `o` float32 `[T, width]` in `parts` equal parts, each
+        scaled to unit root mean square, times `weight` `[width]`; times silu(`gate`) (float32 `[T, width]`, rows may lie
+        apart) after the norm, or before it with `gate_first`. `skip` = (factors `[heads]`, x float32 `[T, width]`, rows
+        may lie apart): o + factor x first, head by head. In the compute dtype."""
+        t, width = o.shape
+        o = o.float()
+        if skip is not None:
+            factors, x = skip
+            o = o + factors.float().repeat_interleave(width // factors.numel())[None, :] * x.float()
+        g = gate.float() * torch.sigmoid(gate.float())
+        if gate_first:
+            o = o * g
+        p = o.reshape(t, parts, width // parts)
+        o = (p * torch.rsqrt((p * p).mean(-1, keepdim=True) + eps)).reshape(t, width) * weight.float()
+        return (o if gate_first else o * g).to(self.dtype)
+
     # ---------------------------------------------------------------- experts
 
-    def route(self, z, top, score="sigmoid", renormalize=False, correction=None, scale=1.0):
+    def route(self, z, top, score="sigmoid", renormalize=False, correction=None, scale=1.0, groups=None):
         """float32 router logits `[T, E]` -> (int32 `[T, top]` the experts with the largest scores, the lower
         number first where two are equal; float32 `[T, top]` their scores, sigmoid(z) or softmax(z), divided by
         their sum with `renormalize`). The ranking is by the logits, which both scores grow with: two large
         logits that float32 still tells apart can have scores that it does not. With `correction` (float32 `[E]`)
         the ranking is by score + correction, and the weights are the scores without it; `scale` multiplies the
-        weights."""
+        weights. `groups` = (count, keep): the experts form `count` equal groups of neighbours, a group ranks by its best
+        expert, and only experts of the `keep` best groups (the lower number where two are equal) can be chosen."""
         s = torch.sigmoid(z.float()) if score == "sigmoid" else torch.softmax(z.float(), dim=-1)
         ranked = z.float() if correction is None else s + correction.float()
+        if groups is not None and groups[1] < groups[0]:
+            best = ranked.reshape(z.shape[0], groups[0], -1).max(-1).values
+            kept = torch.sort(best, dim=-1, descending=True, stable=True).indices[:, :groups[1]]
+            seen = torch.zeros_like(best, dtype=torch.bool).scatter_(1, kept, True)
+            ranked = ranked.masked_fill(~seen.repeat_interleave(z.shape[1] // groups[0], dim=1), float("-inf"))
         order = torch.sort(ranked, dim=-1, descending=True, stable=True).indices[:, :top]
         w = torch.gather(s, 1, order)
         if renormalize:
@@ -734,23 +830,28 @@ class ReferenceOps:
         return self._gated(g, u, activation, limit).to(self.dtype)
 
     def expert_mixture(self, h, chosen, weights, w_gate_up, w_down, activation, weight_on, residual=None, may_wait=False,
-                       limit=None):
+                       limit=None, identity=0):
         """float32 `residual + sum_c expert_(chosen[t, c])(h[t])` with the weights `weights[t, c]` on the expert's
         input (`weight_on="input"`: act(w g) * (w u), the float32 sums of the first product times w) or on its
-        output. `w_gate_up` `[E, 2 F, D]` (gate rows, then up rows), `w_down` `[E, D, F]`."""
+        output. `w_gate_up` `[E, 2 F, D]` (gate rows, then up rows), `w_down` `[E, D, F]`. A number of E or more in
+        `chosen` is an expert without tensors, whose output is its input (weight_on "output")."""
         t, top = chosen.shape
         f = w_down.shape[2]
         out = residual.float().clone() if residual is not None else torch.zeros(t, w_down.shape[1], dtype=torch.float32,
                                                                                 device=h.device)
         x = h.to(w_gate_up.dtype).float()
+        experts = w_gate_up.shape[0]
         for c in range(top):
             e = chosen[:, c].long()
+            same = e >= experts
+            e = e.clamp(max=experts - 1)
             gu = torch.einsum("tk,tnk->tn", x, w_gate_up[e].float())
             w = weights[:, c].float()[:, None]
             if weight_on == "input":
                 gu = gu * w
             inner = self._gated(gu[:, :f], gu[:, f:], activation, limit).to(self.dtype)
             y = torch.einsum("tf,tdf->td", inner.to(w_down.dtype).float(), w_down[e].float())
+            y = torch.where(same[:, None], h.float(), y)
             out = out + (y if weight_on == "input" else y * w)
         return out
 
@@ -761,6 +862,11 @@ class ReferenceOps:
 
     def cast(self, x, dtype):
         return x.to(dtype)
+
+    def scale_and_cap(self, logits, scale, cap):
+        """In place: y = scale * x, and with a cap c (0: none) c tanh(y / c)."""
+        logits.mul_(scale)
+        return logits.copy_(cap * torch.tanh(logits / cap)) if cap else logits
 
     def ban_tokens(self, logits, tokens):
         rows = torch.nonzero(tokens >= 0).flatten()

@@ -110,6 +110,13 @@ class Mixer(Part):
     def forward(self, h, ctx, cache, residual):
         raise NotImplementedError
 
+    def results(self, h, ctx, cache) -> list:
+        """mix(h) as a sum for an arrangement that adds and norms in a launch of its own: a list of
+        (y, norm weight, norm eps, factor), float32 `[T, hidden]` each, sum of factor * y, or, where a norm weight is
+        given, of factor * y / sqrt(mean(y^2) + norm eps) * weight. One entry without a norm if not said otherwise
+        (`forward` then takes `residual` None)."""
+        return [(self.forward(h, ctx, cache, None), None, None, 1.0)]
+
     def first_weight(self):
         """The matrix that `h` is multiplied by, if that product is all this part does with `h` and it goes
         through `ops.linear` or `ops.qkv_project`; None otherwise. A block may then hand `h` over as

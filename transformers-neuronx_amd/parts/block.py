@@ -34,14 +34,38 @@ class PreNormBlock(Block):
 
 @register_block("post_norm")
 class PostNormBlock(Block):
-    """`x = norm(x + mixer(x))`, `x = norm(x + feed_forward(x))`: the norm follows
-    each sum, and its output is the stream."""
+    """`x = norm(alpha x + mixer(x))`, `x = norm(alpha x + feed_forward(x))`: the norm follows
+    each sum, and its output is the stream. Without `alpha` (None) it is 1, and the sums are made by the last
+    product of each part. With it the part's result comes alone and one launch makes the sum and the norm (a norm
+    that only scales); a mixer whose result is a sum of normed results (`Mixer.results`) has them normed and summed
+    in the same launch."""
 
     recordable = True
 
     reads_compute_copy = True      # the mixer reads the stream itself, in the compute dtype
 
+    def __init__(self, mixer, feed_forward, mixer_norm, feed_forward_norm, *, alpha=None):
+        super().__init__(mixer, feed_forward, mixer_norm, feed_forward_norm)
+        self.alpha = None if alpha is None else float(alpha)
+        self.has_ff = not getattr(feed_forward, "absent", False)
+        if self.alpha is not None:
+            for norm in (mixer_norm,) + ((feed_forward_norm,) if self.has_ff else ()):
+                if not hasattr(norm, "fused_form") or norm.fused_form()[2]:
+                    raise ValueError("the norm behind a sum with a factor is one that only scales (rms_norm)")
+
+    def _join(self, norm, x, results):
+        weight, _, _, eps = norm.fused_form()
+        return self.ops.join_norm(x, self.alpha, results, weight, eps, self.dtype)
+
     def forward(self, stream: Stream, ctx, cache) -> Stream:
+        if self.alpha is not None:
+            x = stream.x
+            h = stream.compute if stream.compute is not None else self.ops.cast(x, self.dtype)
+            x, h = self._join(self.mixer_norm, x, self.mixer.results(h, ctx, cache))
+            debug.tap("after_mixer", x)
+            if self.has_ff:
+                x, h = self._join(self.feed_forward_norm, x, [(self.feed_forward.forward(h, ctx, None), None, None, 1.0)])
+            return Stream(x, h)
         h = stream.compute if stream.compute is not None else self.mixer_norm.ops.cast(stream.x, self.mixer_norm.dtype)
         t = self.mixer.forward(h, ctx, cache, stream.x)
         x, h = self.mixer_norm.forward(t, True, True)

@@ -17,18 +17,23 @@ class TokenEmbedding(Part):
     recordable = True
 
     def __init__(self, vocab: int, embed_width: int, width: int, position: PartSpec,
-                 table_name: str, projection_name: Optional[str], position_name: str, scale: float = 1.0):
-        """`scale`: the token's row times this number (in float32, where the row joins the stream)."""
+                 table_name: str, projection_name: Optional[str], position_name: str, scale: float = 1.0,
+                 norm: Optional[PartSpec] = None, norm_name: str = ""):
+        """`scale`: the token's row times this number (in float32, where the row joins the stream). `norm`: a norm of
+        what has been embedded, whose output is the stream (its tensors under `norm_name`)."""
         self.vocab, self.embed_width, self.width = vocab, embed_width, width
         self.scale = float(scale)
         self.table_name, self.projection_name, self.position_name = table_name, projection_name, position_name
         self.position = POSITIONS.build(position)
         self.projects = embed_width != width
+        self.norm, self.norm_name = NORMS.build(norm) if norm is not None else None, norm_name
 
     def param_decls(self, prefix: str = "") -> List[ParamDecl]:
         d = [ParamDecl(self.table_name, (self.vocab, self.embed_width), "table")]
         if self.projects:
             d.append(ParamDecl(self.projection_name, (self.width, self.embed_width)))
+        if self.norm is not None:
+            d += self.norm.param_decls(self.norm_name)
         return d + self.position.param_decls(self.position_name)
 
     def load(self, tensors: Dict, prefix: str, ops, dtype) -> None:
@@ -36,8 +41,11 @@ class TokenEmbedding(Part):
         self.table = tensors[self.table_name]
         self.projection = ops.prepare_weight(tensors[self.projection_name]) if self.projects else None
         self.position.load(tensors, self.position_name, ops, dtype)
+        if self.norm is not None:
+            self.norm.load(tensors, self.norm_name, ops, dtype)
 
     def forward(self, ctx, want_compute: bool) -> Stream:
+        normed, want_compute = want_compute, want_compute and self.norm is None
         x = self.ops.embed(ctx.token_ids, self.table, self.dtype, ctx.kept_tokens)
         if self.projects:
             x = self.ops.linear(x, self.projection, None)
@@ -45,6 +53,8 @@ class TokenEmbedding(Part):
             xf, xc = self.position.at_input(x, ctx.positions, want_compute, scale=self.scale)
         else:
             xf, xc = self.position.at_input(x, ctx.positions, want_compute)
+        if self.norm is not None:
+            xf, xc = self.norm.forward(xf, True, normed)
         return Stream(xf, xc)
 
 
@@ -98,10 +108,10 @@ class VocabHead(Part):
 
     def __init__(self, vocab: int, embed_width: int, width: int, norm: Optional[PartSpec],
                  weight_name: str, tied_to: Optional[str], projection_name: Optional[str], norm_name: str,
-                 logit_scale: float = 1.0):
+                 logit_scale: float = 1.0, softcap: Optional[float] = None):
         """`logit_scale`: the logits are the product times this number (folded into the matrix's float32
-        result, not into the matrix)."""
-        self.logit_scale = float(logit_scale)
+        result, not into the matrix). `softcap` c: then c tanh(logits / c)."""
+        self.logit_scale, self.softcap = float(logit_scale), float(softcap or 0.0)
         self.vocab, self.embed_width, self.width = vocab, embed_width, width
         self.norm = NORMS.build(norm) if norm is not None else None
         self.weight_name, self.tied_to = weight_name, tied_to
@@ -134,4 +144,6 @@ class VocabHead(Part):
         if self.projects:
             h = self.ops.linear(h, self.projection, None)
         logits = self.ops.linear(h, self.weight, None, out_f32=True)
+        if self.softcap:
+            return self.ops.scale_and_cap(logits, self.logit_scale, self.softcap)
         return logits if self.logit_scale == 1.0 else logits.mul_(self.logit_scale)

@@ -65,11 +65,14 @@ class GatedFeedForward(FeedForward):
 
     recordable = True
 
-    def __init__(self, width: int, inner: int, activation: str, names, weight_suffix: str = ""):
+    def __init__(self, width: int, inner: int, activation: str, names, weight_suffix: str = "", limit: float = None):
         """`names`: the checkpoint's names of the gate, up and down matrices; `activation`: "gelu_new" (the tanh
-        form) or "silu"."""
-        if activation not in ("gelu_new", "silu"):
-            raise ValueError(f"a gated feed-forward's activation is gelu_new or silu, got {activation!r}")
+        form), "silu", or "clamped_swiglu" with its `limit` (as in `mixture`)."""
+        if activation not in ("gelu_new", "silu", "clamped_swiglu"):
+            raise ValueError(f"a gated feed-forward's activation is gelu_new, silu or clamped_swiglu, got {activation!r}")
+        if (activation == "clamped_swiglu") != (limit is not None) or (limit is not None and not float(limit) > 0):
+            raise ValueError("a gated feed-forward: activation 'clamped_swiglu' and no other takes a positive `limit`")
+        self.limit = dict(limit=float(limit)) if limit is not None else {}
         self.width, self.inner, self.activation = width, inner, activation
         self.names, self.weight_suffix = tuple(names), weight_suffix
 
@@ -87,7 +90,7 @@ class GatedFeedForward(FeedForward):
 
     def forward(self, h, ctx, residual):
         inner = self.ops.gated_activation(self.ops.linear(h, self.w_in, None, out_f32=True, f32_by_library=True),
-                                          self.activation)
+                                          self.activation, **self.limit)
         return self.ops.linear(inner, self.w_down, None, residual=residual, out_f32=True,
                                f32_by_library=residual is None)
 
@@ -120,18 +123,32 @@ class ExpertMixture(FeedForward):
     `correction_name`: a tensor of one number an expert that is added to the scores where the experts are chosen
     and nowhere else (the weights are the scores without it). `route_scale`: the weights times this number.
     `activation="clamped_swiglu"` with `limit` (`shared_limit` for the shared expert): g = min(W_gate x, limit),
-    u = clamp(W_up x, -limit, limit), and the expert is W_down (g sigmoid(1.702 g) (u + 1))."""
+    u = clamp(W_up x, -limit, limit), and the expert is W_down (g sigmoid(1.702 g) (u + 1)).
+
+    `identity`: so many router outputs behind the experts' stand for experts that have no tensors: their output is
+    their input. They are scored, corrected, grouped and chosen like the others. `groups` = {count, keep}: experts and
+    identity experts together form `count` equal groups of neighbours, a group's score is the largest score (with
+    the correction) in it, and only experts of the `keep` best groups can be chosen."""
 
     recordable = True
 
     def __init__(self, width: int, experts: int, top: int, inner: int, router_name: str, expert_name: str, names,
                  shared_inner: int = 0, shared_name: str = "shared.", score: str = "sigmoid", renormalize: bool = False,
                  weight_on: str = "output", activation: str = "silu", weight_suffix: str = "",
-                 correction_name: str = None, route_scale: float = 1.0, limit: float = None, shared_limit: float = None):
+                 correction_name: str = None, route_scale: float = 1.0, limit: float = None, shared_limit: float = None,
+                 identity: int = 0, groups=None):
         """`expert_name`: a format string that takes the expert's number ("e{}."); `names`: the names of an
         expert's gate, up and down matrices."""
-        if not 1 <= top <= experts:
-            raise ValueError(f"a token takes {top} of {experts} experts")
+        self.routed, self.identity = experts + identity, identity
+        self.groups = (int(groups["count"]), int(groups["keep"])) if groups else None
+        if not 1 <= top <= self.routed or experts < 1 or identity < 0:
+            raise ValueError(f"a token takes {top} of {experts} experts and {identity} without tensors")
+        if self.groups is not None:
+            count, keep = self.groups
+            if count < 1 or self.routed % count or not 1 <= keep <= count or top > keep * (self.routed // count):
+                raise ValueError(f"{self.routed} experts in {count} groups of which {keep} are kept, {top} a token")
+        if identity and (weight_on != "output" or renormalize):
+            raise ValueError("mixture: experts without tensors take their weight on the output, not renormalized")
         if score not in ("sigmoid", "softmax") or weight_on not in ("input", "output") \
                 or activation not in ("silu", "gelu_new", "clamped_swiglu"):
             raise ValueError(f"mixture: score {score!r}, weight_on {weight_on!r}, activation {activation!r}")
@@ -140,8 +157,8 @@ class ExpertMixture(FeedForward):
                 raise ValueError("mixture: activation 'clamped_swiglu' needs a positive `limit` (and `shared_limit`)")
             if weight_on != "output":
                 raise ValueError("mixture: a clamped expert takes its weight on the output")
-        if correction_name and (score != "sigmoid" or renormalize):
-            raise ValueError("mixture: a correction of the choice goes with sigmoid scores that are not renormalized")
+        if correction_name and renormalize:
+            raise ValueError("mixture: a correction of the choice goes with scores that are not renormalized")
         self.correction_name, self.route_scale = correction_name, float(route_scale)
         self.limit = float(limit) if limit is not None else None
         self.shared_limit = float(shared_limit) if shared_limit is not None else None
@@ -160,9 +177,9 @@ class ExpertMixture(FeedForward):
         d = []
         for e in range(self.experts):
             d += self._expert_decls(prefix + self.expert_name.format(e), self.inner)
-        d.append(ParamDecl(f"{prefix}{self.router_name}{self.weight_suffix}", (self.experts, self.width)))
+        d.append(ParamDecl(f"{prefix}{self.router_name}{self.weight_suffix}", (self.routed, self.width)))
         if self.correction_name:
-            d.append(ParamDecl(f"{prefix}{self.correction_name}", (self.experts,), "vector"))
+            d.append(ParamDecl(f"{prefix}{self.correction_name}", (self.routed,), "vector"))
         if self.shared_inner:
             d += self._expert_decls(prefix + self.shared_name, self.shared_inner)
         return d
@@ -184,7 +201,7 @@ class ExpertMixture(FeedForward):
             self.w_shared_down = ops.prepare_weight(tensors[f"{p}{d}{s}"])
 
     def flops_per_token(self, keys: float = 0.0) -> float:
-        return 2.0 * self.width * (self.experts + 3 * self.top * self.inner + 3 * self.shared_inner)
+        return 2.0 * self.width * (self.routed + 3 * self.top * self.inner * self.experts / self.routed + 3 * self.shared_inner)
 
     def forward(self, h, ctx, residual):
         ops = self.ops
@@ -192,8 +209,12 @@ class ExpertMixture(FeedForward):
         more = {}
         if self.correction is not None or self.route_scale != 1.0:
             more = dict(correction=self.correction, scale=self.route_scale)
+        if self.groups is not None:
+            more["groups"] = self.groups
         chosen, weights = ops.route(z, self.top, self.score, self.renormalize, **more)
         limit = dict(limit=self.limit) if self.limit is not None else {}
+        if self.identity:
+            limit["identity"] = self.identity
         # (a step that is being recorded is sized by `length_bound`; any other may let the host read)
         x = ops.expert_mixture(h, chosen, weights, self.w_gate_up, self.w_down, self.activation, self.weight_on, residual,
                                may_wait=ctx is not None and ctx.length_bound is None, **limit)

@@ -58,7 +58,7 @@ class Attention(Mixer):
                  qk_norm=None, value_mix=None, weight_suffix: str = ".weight", bias_suffix: str = ".bias",
                  softcap: Optional[float] = None, distance_bias=None, chunk: Optional[int] = None,
                  out_gate: Optional[str] = None, out_gate_per_head: bool = False, values_from_keys: bool = False,
-                 head_scale: Optional[str] = None):
+                 head_scale: Optional[str] = None, temperature=None, sink: Optional[str] = None):
         """`names`: the checkpoint's names of the query, key, value and output projections, relative to
         the mixer's prefix (the architecture's spec gives them); a matrix's name adds `weight_suffix`, a bias's
         `bias_suffix`. `out_bias`: whether the output projection has a bias (as the others, if not said).
@@ -91,7 +91,9 @@ class Attention(Mixer):
 
         `values_from_keys`: there is no value projection (its name in `names` is not read): a token's values are
         its keys as projected, before their norm and turn. `head_scale`: the name of a tensor of one number a query
-        head that multiplies the head's scores (beside `scale`). With `shared` in `qk_norm` (which implies
+        head that multiplies the head's scores (beside `scale`). `temperature` = {coef, every}: the queries of the token
+        at position p are multiplied by 1 + coef ln(floor((p + 1) / every) + 1). `sink`: the name of a tensor of one
+        number a query head; the softmax's denominator also holds exp(sink), once, a term that stands for no token. With `shared` in `qk_norm` (which implies
         `per_head`) the two weight tensors hold one head's `head_size` elements, the same for every head."""
         self.width, self.num_heads, self.head_size = width, num_heads, head_size
         self.num_kv_heads = num_kv_heads if num_kv_heads is not None else num_heads
@@ -107,6 +109,10 @@ class Attention(Mixer):
         self.chunk = int(chunk) if chunk else None
         self.out_gate, self.out_gate_per_head = out_gate, bool(out_gate_per_head) and bool(out_gate)
         self.values_from_keys, self.head_scale = bool(values_from_keys), head_scale
+        self.temperature = (float(temperature["coef"]), int(temperature["every"])) if temperature else None
+        if self.temperature and self.temperature[1] < 1:
+            raise ValueError(f"a temperature that grows every {self.temperature[1]} tokens")
+        self.sink = sink
         if self.qk_norm and self.qk_norm.get("shared"):
             self.qk_norm["per_head"] = True
         if self.values_from_keys and self.value_size != head_size:
@@ -115,9 +121,9 @@ class Attention(Mixer):
             raise ValueError("values that are the keys are not blended")
         if self.chunk is not None and window is not None:
             raise ValueError("an attention mixer masks by a window or by chunks, not both")
-        self.scored = bool(self.softcap or self.distance_bias or self.chunk or out_gate)
+        self.scored = bool(self.softcap or self.distance_bias or self.chunk or out_gate or sink)
         self.prepared = bool(self.qk_norm or self.value_mix or halves or self.value_size != head_size or self.scored
-                             or self.values_from_keys or head_scale)
+                             or self.values_from_keys or head_scale or self.temperature)
         self.defer_out = False      # set by a mixer that runs this one beside another and owns the output product
         if self.prepared:
             if not own_kv:
@@ -163,6 +169,8 @@ class Attention(Mixer):
                   ParamDecl(f"{prefix}{kn}{self.qk_norm['suffix']}", (self.head_size if shared else kv_out,), "vector", "around_one")]
         if self.head_scale:
             d.append(ParamDecl(f"{prefix}{self.head_scale}", (self.num_heads,), "vector", "around_one"))
+        if self.sink:
+            d.append(ParamDecl(f"{prefix}{self.sink}", (self.num_heads,), "vector"))
         if self.distance_bias:
             d.append(ParamDecl(f"{prefix}{self.distance_bias['name']}", (self.distance_bias.get("rows"), self.num_heads),
                                "vector"))
@@ -216,6 +224,7 @@ class Attention(Mixer):
                 self.q_norm = self.q_norm.repeat(self.num_heads).contiguous()
                 self.k_norm = self.k_norm.repeat(self.num_kv_heads).contiguous()
         self.head_scales = tensors[f"{prefix}{self.head_scale}"] if self.head_scale else None
+        self.sinks = tensors[f"{prefix}{self.sink}"] if self.sink else None
         if self.value_mix and not self.value_mix["first"]:
             self.mix_weight = tensors[f"{prefix}{self.value_mix['name']}"].reshape(1)
 
@@ -257,7 +266,7 @@ class Attention(Mixer):
         attention over heads of the cache's size, the output projection."""
         ops = self.ops
         c = self._inner_prepared(h, ctx, cache, view, None, 1.0)
-        return ops.linear(c, self.w_out, self.b_out, residual=residual, out_f32=True)
+        return ops.linear(c, self.w_out, self.b_out, residual=residual, out_f32=True, f32_by_library=residual is None)
 
     def _inner_prepared(self, h, ctx, cache, view, out, out_scale):
         ops = self.ops
@@ -279,6 +288,8 @@ class Attention(Mixer):
             more["values_at"] = self.num_heads * self.head_size        # the keys' columns are read a second time
         if self.head_scales is not None:
             more["head_scale"] = self.head_scales
+        if self.temperature is not None:
+            more["temperature"] = self.temperature
         q = ops.qkv_prepare(proj, self.num_heads, self.num_kv_heads, self.head_size, self.value_size, self.cache_head,
                             self.q_norm, self.k_norm, self.qk_norm["eps"] if self.qk_norm else 0.0, self.freqs,
                             bool(rot.interleaved) if rot is not None else False, self.scale, self.mix_weight, first,
@@ -287,6 +298,8 @@ class Attention(Mixer):
             return ops.attention(q, self.num_heads, self.num_kv_heads, self.cache_head, ctx, view, cache.k_pages,
                                  cache.v_pages, self.window)
         gate, more = None, {}
+        if self.sinks is not None:
+            more["sink"] = self.sinks
         if self.out_gate:
             at = self.num_heads * self.head_size + self.num_kv_heads * (
                 self.head_size + (0 if self.values_from_keys else self.value_size))

@@ -160,6 +160,156 @@ class GatedLinearRecurrence(_BesideAnother, Mixer):
         return self.ops.linear(y, self.w_out, None, residual=residual, out_f32=True, f32_by_library=residual is None)
 
 
+class _LinearMemory(Mixer):
+    """What the mixers around a linear memory share: a matrix S `[n, v]` a head that is carried from token to token,
+
+        S <- e^g S,   S <- S + k w^T,   o = S^T q,        w = write * val   or   w = write * (val - S^T k)  (`delta`),
+
+    whose queries, keys and values come out of a short causal convolution over time (`taps` a channel) and silu. Queries
+    and keys have `groups` heads, head h takes number floor(h / (heads / groups)). One product makes everything that is
+    read of a token, one kernel the convolution, its activation, unit norms, decays and write weights, one walks the
+    memory, one makes what the output product reads. Everything between the two products is float32; the state is S and
+    the convolution's last `taps - 1` inputs."""
+
+    recordable = True
+    delta = False
+
+    def _sizes(self, width, heads, groups, head_size, value_size, taps, eps):
+        if heads % groups or taps < 1:
+            raise ValueError(f"a linear memory of {heads} heads over {groups} query/key heads with {taps} taps")
+        if head_size > 256:
+            raise ValueError(f"a linear memory's queries and keys have up to 256 elements a head, got {head_size}")
+        self.width, self.heads, self.groups, self.taps, self.eps = width, heads, groups, taps, float(eps)
+        self.n, self.v = head_size, value_size
+        self.inner = heads * value_size
+        self.channels = 2 * groups * head_size + self.inner
+
+    def cache_need(self) -> Optional[CacheNeed]:
+        # (a column's rows side by side: what a lane of the kernel holds are neighbours in memory)
+        shapes = (("memory", (2, self.heads, self.v, self.n)),)
+        if self.taps > 1:
+            shapes += (("inputs", (self.taps, self.channels)),)
+        return CacheNeed("state", state_shapes=shapes)
+
+    def _load_in(self, tensors, names, ops):
+        """The rows of the input matrices one under the other, filled up with zero rows to a multiple of 16."""
+        w = torch.cat([tensors[n] for n in names], dim=0)
+        return ops.prepare_weight(torch.nn.functional.pad(w, (0, 0, 0, -w.shape[0] % 16)).contiguous())
+
+    def flops_per_token(self, keys: float = 0.0) -> float:
+        # the memory's update and its product with the query, a head (with `delta` its product with the key too)
+        return (super().flops_per_token(keys) + 2.0 * self.channels * self.taps
+                + (6.0 if self.delta else 4.0) * self.heads * self.n * self.v)
+
+    def forward(self, h, ctx, cache, residual):
+        y = self._inner(self.ops.linear(h, self.w_in, None, out_f32=True, f32_by_library=True), ctx, cache.state)
+        return self.ops.linear(y, self.w_out, None, residual=residual, out_f32=True, f32_by_library=residual is None)
+
+
+@register_mixer("gated_delta")
+class GatedDeltaRule(_LinearMemory):
+    """The gated delta rule (gated DeltaNet). With q, k of `groups` heads of n elements and val of `heads` heads of v,
+    each through a convolution over time and silu, q and k made unit vectors a head and q times n^(-1/2):
+
+        beta = sigmoid(W_b h),   g = -exp(A_log) softplus(W_a h + dt_bias)                     (a number a head each)
+        S <- e^g S;   u = beta (val - S^T k);   S <- S + k u^T;   o = S^T q
+
+    A head's o at unit root mean square, times `norm` (v elements, the same for all heads), times silu(W_g h);
+    W_o on the heads side by side."""
+
+    delta = True
+
+    def __init__(self, width: int, heads: int, groups: int, head_size: int, value_size: int, taps: int, eps: float, names,
+                 conv_suffix: str = ".conv", weight_suffix: str = ""):
+        """`names`: the checkpoint's names of W_q, W_k, W_v, W_g, W_a, W_b, W_o, A_log, dt_bias and the norm's weight; a
+        convolution's weight `[channels, taps]` is its projection's name with `conv_suffix`."""
+        self._sizes(width, heads, groups, head_size, value_size, taps, eps)
+        self.names, self.conv_suffix, self.weight_suffix = tuple(names), conv_suffix, weight_suffix
+        if len(self.names) != 10:
+            raise ValueError("names: W_q, W_k, W_v, W_g, W_a, W_b, W_o, A_log, dt_bias and the norm, ten names")
+
+    def param_decls(self, prefix: str) -> List[ParamDecl]:
+        q, k, v, g, a, b, o, a_log, dt_bias, norm = (prefix + n for n in self.names)
+        ws, cs, h = self.weight_suffix, self.conv_suffix, self.heads
+        qk = self.groups * self.n
+        return [ParamDecl(q + ws, (qk, self.width)), ParamDecl(q + cs, (qk, self.taps), "vector"),
+                ParamDecl(k + ws, (qk, self.width)), ParamDecl(k + cs, (qk, self.taps), "vector"),
+                ParamDecl(v + ws, (self.inner, self.width)), ParamDecl(v + cs, (self.inner, self.taps), "vector"),
+                ParamDecl(g + ws, (self.inner, self.width)), ParamDecl(a + ws, (h, self.width)),
+                ParamDecl(b + ws, (h, self.width)), ParamDecl(o + ws, (self.width, self.inner)),
+                ParamDecl(a_log, (h,), "vector"), ParamDecl(dt_bias, (h,), "vector"),
+                ParamDecl(norm, (self.v,), "vector", "around_one")]
+
+    def load(self, tensors: Dict, prefix: str, ops, dtype) -> None:
+        super().load(tensors, prefix, ops, dtype)
+        q, k, v, g, a, b, o, a_log, dt_bias, norm = (prefix + n for n in self.names)
+        ws, cs = self.weight_suffix, self.conv_suffix
+        self.w_in = self._load_in(tensors, [n + ws for n in (q, k, v, g, a, b)], ops)
+        self.conv_w = torch.cat([tensors[n + cs] for n in (q, k, v)], dim=0).contiguous()
+        self.rate = (-torch.exp(tensors[a_log].float())).contiguous()
+        self.dt_bias = tensors[dt_bias]
+        self.norm_weight = tensors[norm].repeat(self.heads).contiguous()
+        self.w_out = ops.prepare_weight(tensors[o + ws])
+
+    def _inner(self, proj, ctx, state):
+        ops, qk, c, h = self.ops, self.groups * self.n, self.channels, self.heads
+        at = c + self.inner                                     # the columns: q | k | v | gate | a | b
+        u, decay, write = ops.memory_inputs(proj, 0, self.conv_w, None, ctx, state.get("inputs"), h, at, self.rate,
+                                            self.dt_bias, write_at=at + h, unit=(self.n, 2 * qk, qk, self.n ** -0.5))
+        o = ops.linear_memory(u, 0, qk, 2 * qk, h, self.groups, self.n, self.v, decay, write, ctx, state["memory"], True)
+        return ops.gated_norm(o, proj[:, c:c + self.inner], self.norm_weight, self.eps, h, False)
+
+
+@register_mixer("state_space")
+class StateSpace(_LinearMemory):
+    """A selective state space with one decay a head (Mamba-2). W_in h is laid out [z | x | B | C | dt]: z and x of
+    `heads` heads of v elements, B and C of `groups` heads of n, dt a number a head. x, B and C together pass a convolution
+    over time with a bias, and silu; dt <- softplus(dt + dt_bias):
+
+        S <- exp(-exp(A_log) dt) S + dt B x^T,   y = S^T C + D x
+
+    The heads' y side by side times silu(z), in `norm_groups` equal parts at unit root mean square, times `norm`; W_o."""
+
+    def __init__(self, width: int, heads: int, groups: int, head_size: int, value_size: int, taps: int, norm_groups: int,
+                 eps: float, names, bias_suffix: str = ".b", weight_suffix: str = ""):
+        """`head_size`: n, the size of B and C. `names`: the checkpoint's names of W_in, the convolution (its bias: with
+        `bias_suffix`), dt_bias, A_log, D, the norm's weight and W_o."""
+        self._sizes(width, heads, groups, head_size, value_size, taps, eps)
+        if self.inner % norm_groups:
+            raise ValueError(f"{self.inner} elements do not divide into {norm_groups} equal parts")
+        self.norm_groups, self.names = norm_groups, tuple(names)
+        self.bias_suffix, self.weight_suffix = bias_suffix, weight_suffix
+        if len(self.names) != 7:
+            raise ValueError("names: W_in, the convolution, dt_bias, A_log, D, the norm and W_o, seven names")
+
+    def param_decls(self, prefix: str) -> List[ParamDecl]:
+        w_in, conv, dt_bias, a_log, d, norm, o = (prefix + n for n in self.names)
+        ws = self.weight_suffix
+        return [ParamDecl(w_in + ws, (self.inner + self.channels + self.heads, self.width)),
+                ParamDecl(conv, (self.channels, self.taps), "vector"),
+                ParamDecl(conv + self.bias_suffix, (self.channels,), "vector"),
+                ParamDecl(dt_bias, (self.heads,), "vector"), ParamDecl(a_log, (self.heads,), "vector"),
+                ParamDecl(d, (self.heads,), "vector", "around_one"), ParamDecl(norm, (self.inner,), "vector", "around_one"),
+                ParamDecl(o + ws, (self.width, self.inner))]
+
+    def load(self, tensors: Dict, prefix: str, ops, dtype) -> None:
+        super().load(tensors, prefix, ops, dtype)
+        w_in, conv, dt_bias, a_log, d, norm, o = (prefix + n for n in self.names)
+        self.w_in = self._load_in(tensors, [w_in + self.weight_suffix], ops)
+        self.conv_w, self.conv_b = tensors[conv], tensors[conv + self.bias_suffix]
+        self.rate = (-torch.exp(tensors[a_log].float())).contiguous()
+        self.dt_bias, self.skip, self.norm_weight = tensors[dt_bias], tensors[d], tensors[norm]
+        self.w_out = ops.prepare_weight(tensors[o + self.weight_suffix])
+
+    def _inner(self, proj, ctx, state):
+        ops, i, gn = self.ops, self.inner, self.groups * self.n
+        u, decay, write = ops.memory_inputs(proj, i, self.conv_w, self.conv_b, ctx, state.get("inputs"), self.heads,
+                                            i + self.channels, self.rate, self.dt_bias)
+        o = ops.linear_memory(u, i + gn, i, 0, self.heads, self.groups, self.n, self.v, decay, write, ctx, state["memory"],
+                              False)
+        return ops.gated_norm(o, proj[:, :i], self.norm_weight, self.eps, self.norm_groups, True, skip=(self.skip, u[:, :i]))
+
+
 class _SubCache:
     """The part of a call's cache that one of two mixers side by side sees: the pages as they are, and of the
     state the tensors under its own prefix, named as the mixer names them."""
@@ -179,12 +329,17 @@ class SideBySide(Mixer):
     Both end in an output product; the two are made one: each mixer writes what its output matrix reads, times
     its factor, into its own columns of one buffer (`inner_into`), and the product of that buffer with the two
     output matrices side by side is the weighted sum, added up in float32. At most one of the two keeps pages;
-    the state of both lives in the one cache of the call, under the prefixes `left.` and `right.`."""
+    the state of both lives in the one cache of the call, under the prefixes `left.` and `right.`.
+
+    With `out_norms` = {eps, left, right} each of the two results is first scaled to unit root mean square over the
+    width and weighted (the tensors `left` and `right`, names under the mixer's prefix): each mixer then keeps its own
+    output product, and the norms and the sum are the arrangement's (`results`) or, in `forward`, a launch a norm."""
 
     def __init__(self, left: PartSpec, right: PartSpec, left_name: str = "left.", right_name: str = "right.",
-                 left_scale: float = 1.0, right_scale: float = 1.0):
+                 left_scale: float = 1.0, right_scale: float = 1.0, out_norms=None):
         self.left, self.right = MIXERS.build(left), MIXERS.build(right)
-        for m in (self.left, self.right):
+        self.out_norms = dict(out_norms) if out_norms else None
+        for m in (self.left, self.right) if self.out_norms is None else ():
             if not hasattr(m, "inner_into"):
                 raise ValueError(f"mixer {m.kind!r} cannot run beside another: it has no `inner_into`")
             m.defer_out = True
@@ -205,12 +360,19 @@ class SideBySide(Mixer):
         return CacheNeed("state", state_shapes=state) if state else None
 
     def param_decls(self, prefix: str) -> List[ParamDecl]:
-        return self.left.param_decls(prefix + self.left_name) + self.right.param_decls(prefix + self.right_name)
+        d = self.left.param_decls(prefix + self.left_name) + self.right.param_decls(prefix + self.right_name)
+        if self.out_norms:
+            d += [ParamDecl(prefix + self.out_norms[side], (self.left.width,), "vector", "around_one")
+                  for side in ("left", "right")]
+        return d
 
     def load(self, tensors: Dict, prefix: str, ops, dtype) -> None:
         super().load(tensors, prefix, ops, dtype)
         self.left.load(tensors, prefix + self.left_name, ops, dtype)
         self.right.load(tensors, prefix + self.right_name, ops, dtype)
+        if self.out_norms:
+            self.norm_weights = [tensors[prefix + self.out_norms[side]] for side in ("left", "right")]
+            return
         self.split = self.left.inner_width()
         self.w_out = ops.prepare_weight(torch.cat([self.left.out_matrix(), self.right.out_matrix()], dim=1).contiguous())
 
@@ -223,10 +385,26 @@ class SideBySide(Mixer):
     def flops_per_token(self, keys: float = 0.0) -> float:
         return self.left.flops_per_token(keys) + self.right.flops_per_token(keys)
 
-    def forward(self, h, ctx, cache, residual):
+    def _parts(self, cache):
         subs = self._subs.get(id(cache))
         if subs is None or subs[0] is not cache:
             subs = self._subs[id(cache)] = (cache, _SubCache(cache, "left."), _SubCache(cache, "right."))
+        return subs
+
+    def results(self, h, ctx, cache):
+        if not self.out_norms:
+            return super().results(h, ctx, cache)
+        subs, eps = self._parts(cache), float(self.out_norms["eps"])
+        return [(m.forward(h, ctx, sub, None), w, eps, scale) for m, sub, w, scale in
+                zip((self.left, self.right), subs[1:], self.norm_weights, (self.left_scale, self.right_scale))]
+
+    def forward(self, h, ctx, cache, residual):
+        if self.out_norms:
+            x = residual
+            for y, w, eps, scale in self.results(h, ctx, cache):
+                x = self.ops.norm_add(y, w, None, eps, False, torch.zeros_like(y) if x is None else x, scale)
+            return x
+        subs = self._parts(cache)
         both = torch.empty(h.shape[0], self.split + self.right.inner_width(), dtype=self.dtype, device=self.ops.device)
         self.left.inner_into(h, ctx, subs[1], both[:, :self.split], self.left_scale)
         self.right.inner_into(h, ctx, subs[2], both[:, self.split:], self.right_scale)
