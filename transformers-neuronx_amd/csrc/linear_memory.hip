@@ -3,6 +3,7 @@
 // and what stands before and after them in a mixer:
 //   memory_inputs   a short causal convolution over time with silu, unit vectors a head, decays and write weights
 //   memory_walk     the recurrence token by token (decoded tokens, short runs)
+//   memory_pairs, memory_scan   the same for long runs, 64 tokens at a time on the matrix unit
 //   gated_norm      skip, gate and norm, up to what the output product reads
 // Everything is float32. State lies by position: the token at position p reads place (p - 1) & 1 of S's two (nothing at
 // p = 0) and writes place p & 1; the convolution's input at position p lies at place p mod taps. A step of single tokens
@@ -211,7 +212,7 @@ struct WalkArgs {
   float* memory;            // [slots, 2, H, v, n]
   float* out;               // [T, H v]
   int heads, groups, n, v;
-  int longest;              // runs of more tokens than this are another kernel's (0: none are)
+  int longest;              // runs of more tokens than this are other kernels' (0: none are)
 };
 
 template <bool ALIGNED>
@@ -410,6 +411,332 @@ void launch_walk_sized(const WalkArgs& a, int requests, bool singles, bool align
     launch_walk<16, DELTA>(a, requests, singles, aligned, stream);
 }
 
+// ------------------------------------------------------------------------------------------ the memory, chunk by chunk
+
+// 64 tokens at a time, with c_i = g_1 + ... + g_i the sum of the chunk's log decays up to token i and S the state the
+// chunk begins with. Token i's write w_i and result o_i follow from S and the tokens before it in the chunk:
+//     DELTA:  w_i = write_i (val_i - e^c_i S^T k_i - sum_{j<i} e^(c_i - c_j) (k_i . k_j) w_j),   otherwise write_i val_i
+//     o_i = e^c_i S^T q_i + sum_{j<=i} e^(c_i - c_j) (q_i . k_j) w_j
+//     the state after the chunk: e^c_64 S + sum_j e^(c_64 - c_j) k_j w_j^T
+// With DELTA the w are the solution of a unit lower triangular system; S enters its right side linearly, so what needs no
+// S is made for all chunks side by side (`memory_pairs`): the decays, the weights e^(c_i - c_j) (q_i . k_j), and the
+// system solved for write_i val_i (`u0`) and for write_i e^c_i k_i (`w`), so that w = u0 - w S. What is left goes from
+// chunk to chunk (`memory_scan`): three products with S or of 64 tokens for 16 columns of S at a time. All products are
+// float32 on the matrix unit (16x16x4: float32 operands, float32 sums). The sums c are taken in float64: their
+// differences decide what a token far back in the chunk still weighs.
+//
+// The matrix unit's operands: lane l holds row (or column) l % 16 and k = l / 16; four instructions take k = 16 kk +
+// 4 (l / 16) + j for j = 0 .. 3, so that a lane reads 16 bytes for four of them. The accumulator: column l % 16, rows
+// 4 (l / 16) + i.
+constexpr int CHUNK = 64;
+
+struct ChunkArgs {
+  const float* u;           // [T, ld]
+  int ld, q_at, k_at, v_at;
+  const float* log_decay;   // [T, H]
+  const float* write;       // [T, H]
+  const int* run_start;
+  const int* cached;
+  const int* slots;
+  const int* chunk_run;     // [chunks]
+  const int* chunk_begin;   // [chunks]
+  int chunks;
+  const int* long_run;      // [num_long]
+  const int* long_first;    // [num_long]
+  int num_long;
+  float* memory;            // [slots, 2, H, v, n]
+  float* out;               // [T, H v]
+  float* ahead;             // [T, H]: e^c_i
+  float* behind;            // [T, H]: e^(c_64 - c_i)
+  float* pairs;             // [chunks, H, 64, 64]: e^(c_i - c_j) (q_i . k_j), j <= i; blocks above the diagonal unwritten
+  float* w;                 // [T, H, n]
+  float* u0;                // [T, H, v]
+  int heads, groups, n, v;
+};
+
+// grid: chunks * groups * parts of a group's heads, `per` heads a block. Wave w makes rows 16 w .. 16 w + 15 of q . k
+// (and k . k) once for the group, then every head's weights; with DELTA a thread then solves the system for a column.
+template <int NB, bool DELTA, bool ALIGNED>
+__global__ void __launch_bounds__(256) memory_pairs_kernel(ChunkArgs a, int parts, int per) {
+  constexpr int MLD = CHUNK + 4;
+  __shared__ double cs[CHUNK];
+  __shared__ float beta[CHUNK], up[CHUNK];
+  __shared__ __attribute__((aligned(16))) float mt[DELTA ? CHUNK * MLD : 4];      // the system, column by column
+  const int part = blockIdx.x % parts, rest = blockIdx.x / parts;
+  const int group = rest % a.groups, chunk = rest / a.groups;
+  const int run = a.chunk_run[chunk], begin = a.chunk_begin[chunk];
+  const int t0 = a.run_start[run] + begin, len = min(CHUNK, a.run_start[run + 1] - t0);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
+  const float* q = a.u + a.q_at + group * a.n;
+  const float* k = a.u + a.k_at + group * a.n;
+  f32x4 qk[4], kk[4];
+#pragma unroll
+  for (int cb = 0; cb < 4; ++cb) qk[cb] = kk[cb] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  {
+    const int i = 16 * wave + r;
+    const size_t row = (size_t)(t0 + min(i, len - 1)) * a.ld;
+#pragma unroll 2
+    for (int s = 0; s < NB; ++s) {
+      const int d = 16 * s + 4 * g, valid = i < len ? a.n - d : 0;
+      const f32x4 qa = load4<ALIGNED>(q + row + d, valid);
+      f32x4 ka = {0.f, 0.f, 0.f, 0.f};
+      if (DELTA) ka = load4<ALIGNED>(k + row + d, valid);
+#pragma unroll
+      for (int cb = 0; cb < 4; ++cb) {
+        if (cb > wave) continue;
+        const int j = 16 * cb + r;
+        const f32x4 kb = load4<ALIGNED>(k + (size_t)(t0 + min(j, len - 1)) * a.ld + d, j < len ? a.n - d : 0);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          qk[cb] = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[e], kb[e], qk[cb], 0, 0, 0);
+          if (DELTA) kk[cb] = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[e], kb[e], kk[cb], 0, 0, 0);
+        }
+      }
+    }
+  }
+  const int per_group = a.heads / a.groups;
+  for (int hh = part * per; hh < min(per_group, (part + 1) * per); ++hh) {
+    const int head = group * per_group + hh;
+    if (wave == 0) {
+      const size_t at = (size_t)(t0 + min(lane, len - 1)) * a.heads + head;
+      double c = lane < len ? (double)a.log_decay[at] : 0.0;
+#pragma unroll
+      for (int d = 1; d < 64; d *= 2) {
+        const double before = __shfl_up(c, d, 64);
+        if (lane >= d) c += before;
+      }
+      const double all = __shfl(c, 63, 64);
+      const float e = expf((float)c);
+      cs[lane] = c;
+      up[lane] = e;
+      beta[lane] = lane < len ? a.write[at] : 0.f;
+      if (lane < len) {
+        a.ahead[at] = e;
+        a.behind[at] = expf((float)(all - c));
+      }
+    }
+    __syncthreads();
+    float* pairs = a.pairs + ((size_t)chunk * a.heads + head) * CHUNK * CHUNK;
+#pragma unroll
+    for (int cb = 0; cb < 4; ++cb) {
+      if (cb > wave) continue;
+      const int j = 16 * cb + r;
+      f32x4 m;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int i = 16 * wave + 4 * g + e;
+        const float d = j <= i ? expf((float)(cs[i] - cs[j])) : 0.f;
+        pairs[i * CHUNK + j] = qk[cb][e] * d;
+        if (DELTA) m[e] = j < i ? beta[i] * d * kk[cb][e] : 0.f;
+      }
+      if (DELTA) *(f32x4*)(mt + j * MLD + 16 * wave + 4 * g) = m;
+    }
+    if (DELTA) {
+      __syncthreads();
+      for (int c = threadIdx.x; c < a.v + a.n; c += 256) {
+        const bool value = c < a.v;
+        const float* src = a.u + (size_t)t0 * a.ld + (value ? a.v_at + head * a.v + c : a.k_at + group * a.n + c - a.v);
+        float x[CHUNK];
+#pragma unroll
+        for (int i = 0; i < CHUNK; ++i) x[i] = i < len ? src[(size_t)i * a.ld] : 0.f;
+#pragma unroll
+        for (int i = 0; i < CHUNK; ++i) x[i] *= value ? beta[i] : beta[i] * up[i];
+#pragma unroll
+        for (int j = 0; j < CHUNK - 1; ++j) {
+#pragma unroll
+          for (int i4 = j / 4; i4 < CHUNK / 4; ++i4) {
+            const f32x4 m = *(const f32x4*)(mt + j * MLD + 4 * i4);
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              if (4 * i4 + e > j) x[4 * i4 + e] -= m[e] * x[j];
+          }
+        }
+        float* dst = value ? a.u0 + ((size_t)t0 * a.heads + head) * a.v + c
+                           : a.w + ((size_t)t0 * a.heads + head) * a.n + c - a.v;
+        const size_t step = (size_t)a.heads * (value ? a.v : a.n);
+#pragma unroll
+        for (int i = 0; i < CHUNK; ++i)
+          if (i < len) dst[(size_t)i * step] = x[i];
+      }
+    }
+    __syncthreads();      // before the next head's decays
+  }
+}
+
+// grid: (run, head) pairs in eights * column blocks: the blocks of a (run, head) come eight apart, so that they share an
+// XCD's cache. A block walks a run's chunks for 16 columns of S; wave w has the chunk's tokens 16 w .. 16 w + 15, and of S
+// the blocks of 16 rows w, w + 4, ..., in the accumulators from chunk to chunk. What a chunk's products read of memory is
+// asked for during the products before them.
+template <int NB, bool DELTA, bool ALIGNED>
+__global__ void __launch_bounds__(256) memory_scan_kernel(ChunkArgs a, int column_blocks) {
+  constexpr int RB = (NB + 3) / 4;               // blocks of rows of S a wave
+  constexpr int SLD = 16 * NB + 4, ULD = CHUNK + 4;
+  __shared__ __attribute__((aligned(16))) float s_l[16 * SLD];        // [column][row]
+  __shared__ __attribute__((aligned(16))) float u_l[16 * ULD];        // [column][token]: the writes
+  __shared__ __attribute__((aligned(16))) float b_l[16 * ULD];        // the same times e^(c_64 - c_j)
+  const int rh = (blockIdx.x & 7) + 8 * (blockIdx.x / (8 * column_blocks));
+  const int cb = (blockIdx.x >> 3) % column_blocks;
+  if (rh >= a.num_long * a.heads) return;
+  const int li = rh / a.heads, head = rh - li * a.heads, group = head / (a.heads / a.groups);
+  const int run = a.long_run[li], first = a.long_first[li];
+  const int start = a.run_start[run], count = a.run_start[run + 1] - start, have = a.cached[run], slot = a.slots[run];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
+  const int col = 16 * cb + r;
+  const bool col_ok = col < a.v;
+  const int from = (have - 1) & 1, to = (have + count - 1) & 1;
+  const size_t head_at = (size_t)slot * 2 * a.heads + head;
+  const f32x4 zero4 = {0.f, 0.f, 0.f, 0.f};
+  f32x4 S[RB];
+#pragma unroll
+  for (int x = 0; x < RB; ++x) {
+    const int row = 16 * (wave + 4 * x) + 4 * g;
+    const float* p = a.memory + ((head_at + (size_t)from * a.heads) * a.v + (col_ok ? col : 0)) * a.n + row;
+    S[x] = load4<ALIGNED>(p, have > 0 && col_ok ? a.n - row : 0);
+    if (wave + 4 * x < NB) *(f32x4*)(s_l + r * SLD + row) = S[x];
+  }
+  f32x4 wa[DELTA ? NB : 1], qa[NB], pa[4];
+  float kt[RB][4][4], u0[4], up[4], down[4], decay = 0.f;
+  const float* q = a.u + a.q_at + group * a.n;
+  const float* k = a.u + a.k_at + group * a.n;
+  auto fetch_state_side = [&](int c) {          // what meets S: this wave's tokens' queries and rows of w, their u0
+    const int t0 = start + CHUNK * c, len = min(CHUNK, count - CHUNK * c);
+    const int i = 16 * wave + r;
+    const size_t t = t0 + min(i, len - 1);
+#pragma unroll
+    for (int s = 0; s < NB; ++s) {
+      const int d = 16 * s + 4 * g, valid = i < len ? a.n - d : 0;
+      qa[s] = load4<ALIGNED>(q + t * a.ld + d, valid);
+      if (DELTA) wa[DELTA ? s : 0] = load4<ALIGNED>(a.w + (t * a.heads + head) * a.n + d, valid);
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int it = 16 * wave + 4 * g + e;
+      const size_t tt = t0 + min(it, len - 1);
+      const bool in = it < len && col_ok;
+      if (DELTA)
+        u0[e] = in ? a.u0[(tt * a.heads + head) * a.v + col] : 0.f;
+      else
+        u0[e] = in ? a.write[tt * a.heads + head] * a.u[tt * a.ld + a.v_at + head * a.v + col] : 0.f;
+      up[e] = a.ahead[tt * a.heads + head];
+      down[e] = a.behind[tt * a.heads + head];
+    }
+    decay = a.ahead[(size_t)(t0 + len - 1) * a.heads + head];
+  };
+  auto fetch_token_side = [&](int c) {          // what meets the writes: the weights among the tokens, the keys
+    const int t0 = start + CHUNK * c, len = min(CHUNK, count - CHUNK * c);
+    const float* pairs = a.pairs + ((size_t)(first + c) * a.heads + head) * CHUNK * CHUNK + (16 * wave + r) * CHUNK;
+#pragma unroll
+    for (int s = 0; s < 4; ++s) pa[s] = s <= wave ? *(const f32x4*)(pairs + 16 * s + 4 * g) : zero4;
+#pragma unroll
+    for (int x = 0; x < RB; ++x) {
+      const int row = 16 * (wave + 4 * x) + r;
+#pragma unroll
+      for (int s = 0; s < 4; ++s)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int j = 16 * s + 4 * g + e;
+          kt[x][s][e] = j < len && row < a.n ? k[(size_t)(t0 + j) * a.ld + row] : 0.f;
+        }
+    }
+  };
+  fetch_state_side(0);
+  fetch_token_side(0);
+  __syncthreads();
+  const int chunks = (count + CHUNK - 1) / CHUNK;
+  for (int c = 0; c < chunks; ++c) {
+    const int t0 = start + CHUNK * c, len = min(CHUNK, count - CHUNK * c);
+    f32x4 o = zero4, m = zero4;
+#pragma unroll
+    for (int s = 0; s < NB; ++s) {
+      const f32x4 s4 = *(const f32x4*)(s_l + r * SLD + 16 * s + 4 * g);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        o = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[s][e], s4[e], o, 0, 0, 0);
+        if (DELTA) m = __builtin_amdgcn_mfma_f32_16x16x4f32(wa[DELTA ? s : 0][e], s4[e], m, 0, 0, 0);
+      }
+    }
+    f32x4 u4, b4;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      u4[e] = u0[e] - m[e];
+      b4[e] = u4[e] * down[e];
+      o[e] *= up[e];
+    }
+    *(f32x4*)(u_l + r * ULD + 16 * wave + 4 * g) = u4;
+    *(f32x4*)(b_l + r * ULD + 16 * wave + 4 * g) = b4;
+    const float keep = decay;
+    if (c + 1 < chunks) fetch_state_side(c + 1);
+    __syncthreads();
+#pragma unroll
+    for (int x = 0; x < RB; ++x) S[x] = S[x] * keep;
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+      const f32x4 us = *(const f32x4*)(u_l + r * ULD + 16 * s + 4 * g);
+      const f32x4 bs = *(const f32x4*)(b_l + r * ULD + 16 * s + 4 * g);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        if (s <= wave) o = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[s][e], us[e], o, 0, 0, 0);
+#pragma unroll
+        for (int x = 0; x < RB; ++x) S[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[x][s][e], bs[e], S[x], 0, 0, 0);
+      }
+    }
+    if (c + 1 < chunks) fetch_token_side(c + 1);
+#pragma unroll
+    for (int x = 0; x < RB; ++x)
+      if (wave + 4 * x < NB) *(f32x4*)(s_l + r * SLD + 16 * (wave + 4 * x) + 4 * g) = S[x];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = 16 * wave + 4 * g + e;
+      if (i < len && col_ok) a.out[((size_t)(t0 + i) * a.heads + head) * a.v + col] = o[e];
+    }
+    __syncthreads();
+  }
+  if (!col_ok) return;
+#pragma unroll
+  for (int x = 0; x < RB; ++x) {
+    const int row = 16 * (wave + 4 * x) + 4 * g;
+    float* p = a.memory + ((head_at + (size_t)to * a.heads) * a.v + col) * a.n + row;
+    if (ALIGNED) {
+      if (row < a.n) *(f32x4*)p = S[x];
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (row + e < a.n) p[e] = S[x][e];
+    }
+  }
+}
+
+template <int NB, bool DELTA>
+void launch_chunks(const ChunkArgs& a, bool aligned, hipStream_t stream) {
+  const int per_group = a.heads / a.groups;
+  int per = 1;                                   // heads of a group a block of the first kernel
+  while (!DELTA && per < per_group && (long long)a.chunks * a.groups * ((per_group + 2 * per - 1) / (2 * per)) >= 2 * tnx_compute_units())
+    per *= 2;
+  const int parts = (per_group + per - 1) / per;
+  const dim3 pair_grid((unsigned)((size_t)a.chunks * a.groups * parts));
+  const int column_blocks = (a.v + 15) / 16;
+  const dim3 scan_grid((unsigned)((a.num_long * a.heads + 7) / 8 * 8 * column_blocks));
+  if (aligned) {
+    memory_pairs_kernel<NB, DELTA, true><<<pair_grid, 256, 0, stream>>>(a, parts, per);
+    memory_scan_kernel<NB, DELTA, true><<<scan_grid, 256, 0, stream>>>(a, column_blocks);
+  } else {
+    memory_pairs_kernel<NB, DELTA, false><<<pair_grid, 256, 0, stream>>>(a, parts, per);
+    memory_scan_kernel<NB, DELTA, false><<<scan_grid, 256, 0, stream>>>(a, column_blocks);
+  }
+}
+
+template <bool DELTA>
+void launch_chunks_sized(const ChunkArgs& a, bool aligned, hipStream_t stream) {
+  if (a.n <= 32)
+    launch_chunks<2, DELTA>(a, aligned, stream);
+  else if (a.n <= 64)
+    launch_chunks<4, DELTA>(a, aligned, stream);
+  else if (a.n <= 128)
+    launch_chunks<8, DELTA>(a, aligned, stream);
+  else
+    launch_chunks<16, DELTA>(a, aligned, stream);
+}
+
 // ------------------------------------------------------------------------------------------ after the memory
 
 struct FinishArgs {
@@ -582,6 +909,34 @@ extern "C" int tnx_memory_walk(const float* u, int ld, int q_at, int k_at, int v
   else
     launch_walk_sized<false>(a, requests, tokens == requests, aligned, stream);
   TNX_CHECK_LAUNCH("memory_walk");
+  return 0;
+}
+
+// The runs of several tokens that `long_run` names, chunk by chunk: `chunk_run` and `chunk_begin` name the chunks of 64
+// tokens, a run's chunks one behind the other from `long_first` on. `ahead`, `behind` [T, H], `pairs` [chunks, H, 64, 64],
+// and with `delta` `w` [T, H, n] and `u0` [T, H, v] are room for what the first kernel leaves for the second.
+extern "C" int tnx_memory_chunks(const float* u, int ld, int q_at, int k_at, int v_at, const float* log_decay,
+                                 const float* write, const int* run_start, const int* cached, const int* slots,
+                                 const int* chunk_run, const int* chunk_begin, int chunks, int chunk_size, const int* long_run,
+                                 const int* long_first, int num_long, float* memory, float* out, float* ahead, float* behind,
+                                 float* pairs, float* w, float* u0, int heads, int groups, int n, int v, int delta,
+                                 hipStream_t stream) {
+  TNX_REQUIRE(heads > 0 && groups > 0 && heads % groups == 0 && n > 0 && v > 0 && n <= 256, "memory_chunks: bad sizes");
+  TNX_REQUIRE(chunk_size == CHUNK, "memory_chunks: chunks of %d tokens, the kernels take %d", chunk_size, CHUNK);
+  TNX_REQUIRE(q_at >= 0 && k_at >= 0 && v_at >= 0 && ld >= q_at + groups * n && ld >= k_at + groups * n && ld >= v_at + heads * v,
+              "memory_chunks: rows of %d elements do not hold what is read", ld);
+  TNX_REQUIRE(ahead && behind && pairs && (!delta || (w && u0)), "memory_chunks: no room for what is made ahead");
+  if (chunks <= 0 || num_long <= 0) return 0;
+  TNX_REQUIRE((long long)chunks * heads < (1ll << 30) && ((long long)num_long * heads + 7) * ((v + 15) / 16) < (1ll << 31),
+              "memory_chunks: too many blocks");
+  ChunkArgs a{u, ld, q_at, k_at, v_at, log_decay, write, run_start, cached, slots, chunk_run, chunk_begin, chunks, long_run,
+              long_first, num_long, memory, out, ahead, behind, pairs, w, u0, heads, groups, n, v};
+  const bool aligned = n % 4 == 0 && ((ld | q_at | k_at) & 3) == 0 && (uintptr_t)u % 16 == 0;
+  if (delta)
+    launch_chunks_sized<true>(a, aligned, stream);
+  else
+    launch_chunks_sized<false>(a, aligned, stream);
+  TNX_CHECK_LAUNCH("memory_chunks");
   return 0;
 }
 

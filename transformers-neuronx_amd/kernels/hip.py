@@ -13,6 +13,7 @@ import torch
 
 from . import build
 from .attention_plan import QUERY_TILE
+from .memory_plan import MEMORY_CHUNK, MEMORY_LONG
 from .. import debug
 
 _F32, _BF16 = 0, 1
@@ -179,6 +180,10 @@ _SIGNATURES = {
                               _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p],
         "tnx_memory_walk": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                             _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+        "tnx_memory_chunks": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
+                              _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_int, _c_void_p,
+                              _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int,
+                              _c_int, _c_void_p],
         "tnx_gated_norm": [_c_void_p, _c_void_p, _c_ll, _c_void_p, _c_float, _c_int, _c_int, _c_void_p, _c_int, _c_void_p,
                            _c_ll, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
     },
@@ -1770,10 +1775,31 @@ class HipOps:
         state = float(ctx.num_requests) * heads * n * v * 8
         work = (f"{t} tokens {ctx.num_requests} runs", state + t * (u.shape[1] + heads * v) * 4.0,
                 (6.0 if delta else 4.0) * t * heads * n * v)
+        by_chunks = ctx.plan.get("memory_long_run")
+        longest = 0
+        if by_chunks is not None and by_chunks.numel() and self.memory_by_chunks:
+            # the long runs, chunk by chunk
+            longest = MEMORY_LONG - 1
+            chunk_run, first = ctx.plan["memory_chunk_run"], ctx.plan["memory_long_first"]
+            chunks = chunk_run.numel()
+            ahead, behind, w, u0, pairs = (
+                torch.empty(size, dtype=torch.float32, device=u.device)
+                for size in (t * heads, t * heads, t * heads * n if delta else 0, t * heads * v if delta else 0,
+                             chunks * heads * MEMORY_CHUNK * MEMORY_CHUNK))
+            self._call("linear_memory", "tnx_memory_chunks", _ptr(u), u.shape[1], int(q_at), int(k_at), int(v_at),
+                       _ptr(log_decay), _ptr(write), _ptr(ctx.run_start), _ptr(ctx.cached_lens), _ptr(ctx.slots),
+                       _ptr(chunk_run), _ptr(ctx.plan["memory_chunk_begin"]), chunks, MEMORY_CHUNK, _ptr(by_chunks), _ptr(first),
+                       by_chunks.numel(), _ptr(memory), _ptr(out), _ptr(ahead), _ptr(behind), _ptr(pairs),
+                       _ptr(w) if delta else None, _ptr(u0) if delta else None, heads, groups, n, v, int(bool(delta)), _stream(),
+                       work=work)
+            if by_chunks.numel() == ctx.num_requests:
+                return out
         self._call("linear_memory", "tnx_memory_walk", _ptr(u), u.shape[1], int(q_at), int(k_at), int(v_at), _ptr(log_decay),
                    _ptr(write), _ptr(ctx.run_start), _ptr(ctx.cached_lens), _ptr(ctx.slots), _ptr(memory), _ptr(out), t,
-                   ctx.num_requests, heads, groups, n, v, int(bool(delta)), 0, _stream(), work=work)
+                   ctx.num_requests, heads, groups, n, v, int(bool(delta)), longest, _stream(), work=None if longest else work)
         return out
+
+    memory_by_chunks = True            # tests clear it: every run token by token
 
     def gated_norm(self, o, gate, weight, eps, parts, gate_first, skip=None):
         """See `ReferenceOps.gated_norm`."""

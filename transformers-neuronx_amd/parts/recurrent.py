@@ -191,6 +191,10 @@ class _LinearMemory(Mixer):
             shapes += (("inputs", (self.taps, self.channels)),)
         return CacheNeed("state", state_shapes=shapes)
 
+    def step_planners(self):
+        from ..kernels.memory_plan import memory_plan
+        return {"memory": memory_plan}
+
     def _load_in(self, tensors, names, ops):
         """The rows of the input matrices one under the other, filled up with zero rows to a multiple of 16."""
         w = torch.cat([tensors[n] for n in names], dim=0)
