@@ -113,6 +113,24 @@ def zotunex_config(width, heads, head, ff, vocab, layers):
                         for i in range(layers)])
 
 
+def gubulorn_config(width, heads, head, ff, vocab, layers):
+    """config.json contents of a Gubulorn model at the sizes of a published layer: by turns attention (a quarter as many
+    key/value heads as query heads) beside a state space of the model's width (heads of 64 over a state of 128 in eight
+    groups), and a gated delta rule of the model's width (heads of 128, two to a query/key head), convolutions of four
+    taps; the feed-forward by turns dense of `ff` and eight experts of ff / 4 beside four without tensors in four groups,
+    of which a token takes four out of two groups."""
+    pair = dict(left=dict(heads=heads, kv_heads=max(1, heads // 4), dim=head, vdim=head, scale=head ** -0.5,
+                          q_temp=dict(coef=0.1, every=1024)),
+                right=dict(heads=width // 64, vdim=64, state=128, groups=8, conv=4, norm_groups=8))
+    delta = dict(heads=width // 128, kv_heads=width // 256, dim=128, vdim=128, conv=4)
+    dense = dict(kind="dense", ff=ff, limit=7.0)
+    moe = dict(kind="moe", router=dict(experts=8, identity=4, top=4, groups=dict(count=4, keep=2)), expert=dict(ff=ff // 4))
+    return dict(architecture="Gubulorn", vocab=vocab, width=width, norm=dict(eps=1e-6), postln_alpha=2.0, logit_scale=1.0,
+                logit_softcap=30.0, init_std=0.02, max_positions=4096,
+                layers=[dict(type="delta" if i % 2 else "parallel", mixer=delta if i % 2 else pair,
+                             mlp=dense if i % 4 in (0, 3) else moe) for i in range(layers)])
+
+
 # a new design beside the closest one the engine had, at equal sizes: {design: {size: (its config, the other's)}};
 # the other's is the name of an OPT preset, or (design, its config)
 BESIDE = {"ratesun": {
@@ -130,6 +148,11 @@ BESIDE = {"ratesun": {
     "2048 wide": (lambda n: zotunex_config(2048, 32, 64, 8192, 50272, n),
                   ("sunatar", lambda n: sunatar_config(2048, 32, 64, 8192, 50272, n))),
     "4096 wide": (lambda n: zotunex_config(4096, 32, 128, 16384, 50272, n),
+                  ("sunatar", lambda n: sunatar_config(4096, 32, 128, 16384, 50272, n))),
+}, "gubulorn": {
+    "2048 wide": (lambda n: gubulorn_config(2048, 32, 64, 8192, 50272, n),
+                  ("sunatar", lambda n: sunatar_config(2048, 32, 64, 8192, 50272, n))),
+    "4096 wide": (lambda n: gubulorn_config(4096, 32, 128, 16384, 50272, n),
                   ("sunatar", lambda n: sunatar_config(4096, 32, 128, 16384, 50272, n))),
 }}
 PREFILL_TOKENS = 2048

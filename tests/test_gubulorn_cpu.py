@@ -382,9 +382,12 @@ def test_the_plan_of_a_step_names_the_chunks_of_its_long_runs():
     import numpy as np
     from transformers_neuronx_amd.kernels.memory_plan import MEMORY_CHUNK, MEMORY_LONG, memory_plan
     lens = np.array([1, MEMORY_LONG - 1, MEMORY_LONG, 2 * MEMORY_CHUNK, 1, 2 * MEMORY_CHUNK + 1])
-    plan, _ = memory_plan(lens, np.zeros(6, dtype=np.int64), 16)
-    assert plan["memory_long_run"].tolist() == [2, 3, 5] and plan["memory_long_first"].tolist() == [0, 1, 3]
-    assert plan["memory_chunk_run"].tolist() == [2, 3, 3, 5, 5, 5]
-    assert plan["memory_chunk_begin"].tolist() == [0, 0, MEMORY_CHUNK, 0, MEMORY_CHUNK, 2 * MEMORY_CHUNK]
+    plan, host = memory_plan(lens, np.zeros(6, dtype=np.int64), 16)
+    assert host == {"memory_walk_most": MEMORY_LONG - 1} and MEMORY_CHUNK < MEMORY_LONG <= 2 * MEMORY_CHUNK
+    assert plan["memory_long_run"].tolist() == [2, 3, 5] and plan["memory_long_first"].tolist() == [0, 2, 4]
+    assert plan["memory_chunk_run"].tolist() == [2, 2, 3, 3, 5, 5, 5]
+    assert plan["memory_chunk_begin"].tolist() == [0, MEMORY_CHUNK] * 2 + [0, MEMORY_CHUNK, 2 * MEMORY_CHUNK]
+    few, _ = memory_plan(lens, np.zeros(6, dtype=np.int64), 16, least=2)
+    assert few["memory_long_run"].tolist() == [1, 2, 3, 5]
     none, _ = memory_plan(np.array([1, 2]), np.zeros(2), 16)
     assert all(v.size == 0 and v.dtype == np.int32 for v in none.values())

@@ -48,7 +48,7 @@ def _close(got, want, tol, scale=None):
 
 
 # steps of a request in slot 2 and, from the third step on, of another in slot 0: (request, from, to, slot). Runs of one
-# token, of a few, just under and at the length from which they go by chunks, at and around whole chunks, and long ones.
+# token, of a few, just under and at the length from which they go by chunks here, at and around whole chunks, and long ones.
 CUTS0 = (0, 1, 2, 4, 5, 6, 29, 53, 54, 118, 181, 246, 247, 439, 440, 611)
 CUTS1 = (None, None, 0, 1, 2, 9, 11, 12, 76, 78, 141, 142, 143, None, None, None)
 
@@ -61,6 +61,12 @@ def _steps():
         yield step
 
 
+def _plan(run_lens, cached, page_size):
+    from transformers_neuronx_amd.kernels.memory_plan import memory_plan
+    return memory_plan(run_lens, cached, page_size, least=24)
+
+
+BY_CHUNKS = {"memory": _plan}
 LENGTHS = {0: CUTS0[-1], 1: 143}
 
 
@@ -76,10 +82,7 @@ def test_memories_across_steps_cut_anywhere(sizes, delta, by_chunks):
     """Convolution, unit vectors, decays, write weights and the recurrence over steps of 1, 2 and more tokens, two
     requests side by side in slots that former holders left full, every step of single tokens run twice (a recorded
     step is), against the whole sequence token by token. Decays from almost none to at once."""
-    from transformers_neuronx_amd.kernels.memory_plan import memory_plan
     heads, groups, n, v, taps = sizes
-    if not by_chunks and sizes[2] in (100, 33):
-        pytest.skip("the chunks' case covers these sizes' walk too")
     ops = _ops(torch.float32)
     ops.memory_by_chunks = by_chunks
     g = torch.Generator().manual_seed(4)
@@ -113,7 +116,7 @@ def test_memories_across_steps_cut_anywhere(sizes, delta, by_chunks):
     for step in _steps():
         rows = torch.cat([proj[r][a:b] for r, a, b, _ in step]).to(DEV)
         ctx = _ctx([b - a for _, a, b, _ in step], [a for _, a, _, _ in step], [slot for _, _, _, slot in step],
-                   planners={"memory": memory_plan})
+                   planners=BY_CHUNKS)
         single = all(b - a == 1 for _, a, b, _ in step)
         for _ in range(2 if single else 1):
             u, decay, write = ops.memory_inputs(rows, before, conv.to(DEV), None if bias is None else bias.to(DEV), ctx, inputs,
@@ -134,7 +137,6 @@ def test_memories_across_steps_cut_anywhere(sizes, delta, by_chunks):
 def test_a_memory_that_remembers_hundreds_of_tokens_and_forgets_at_once(delta):
     """Head 0 hardly forgets: what the last token reads is what one token far back wrote, the keys between having
     nothing along it. Head 1 forgets everything at every token. Whole, by chunks and token by token, and decoded."""
-    from transformers_neuronx_amd.kernels.memory_plan import memory_plan
     n, v, t = 64, 16, 400
     g = torch.Generator().manual_seed(2)
     k = torch.randn(t, n, generator=g)
@@ -159,7 +161,7 @@ def test_a_memory_that_remembers_hundreds_of_tokens_and_forgets_at_once(delta):
         memory = torch.full((1, 2, 2, v, n), 9.0, device=DEV)
         out = []
         for a, b in zip(cuts[:-1], cuts[1:]):
-            ctx = _ctx([b - a], [a], [0], planners={"memory": memory_plan})
+            ctx = _ctx([b - a], [a], [0], planners=BY_CHUNKS)
             out.append(ops.linear_memory(u[a:b], 0, n, 2 * n, 2, 1, n, v, log_decay[a:b].to(DEV), write[a:b].to(DEV), ctx, memory, delta))
         got = torch.cat(out)
         _close(got, want, 1e-5)
@@ -364,7 +366,7 @@ def test_experts_chosen_inside_groups_and_experts_without_tensors(name, dtype, t
     free, _ = P.route(z, wide["p.correction"], top, 1, 1)
     assert tokens < 30 or keep == count or chosen.tolist() != free.tolist()             # the groups matter here
     assert tokens < 100 or not identity or bool((chosen >= experts).any())
-    got_chosen, got_weight = ops.route(ops.linear(h.to(DEV), part.w_router, None, out_f32=True), top, "softmax", False,
+    got_chosen, got_weight = ops.route(ops.linear(h.to(DEV), part.w_router, None, out_f32=True)[:, :part.routed], top, "softmax", False,
                                        correction=part.correction, groups=(count, keep))
     assert got_chosen.cpu()[clear].tolist() == chosen[clear].tolist()
     _close(got_weight.cpu()[clear], weight[clear], 1e-5 if dtype == torch.float32 else 1e-2)

@@ -37,7 +37,7 @@ __device__ __forceinline__ float gated(float g, float u, int act, float limit) {
 // the experts form that many equal groups of neighbours, a group ranks by its best expert, and only experts of the `keep`
 // best groups (the lower number where two are equal) take part.
 constexpr int MAX_GROUPS = 256;
-__global__ void __launch_bounds__(256) route_kernel(const float* __restrict__ z, int tokens, int experts, int top,
+__global__ void __launch_bounds__(256) route_kernel(const float* __restrict__ z, int ld, int tokens, int experts, int top,
                                                     int softmax, int renormalize, int* __restrict__ chosen,
                                                     float* __restrict__ weights, const float* __restrict__ correction,
                                                     float scale, int groups, int keep) {
@@ -45,7 +45,7 @@ __global__ void __launch_bounds__(256) route_kernel(const float* __restrict__ z,
   __shared__ unsigned char kept_of[4][MAX_GROUPS];
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= tokens) return;
-  const float* row = z + (size_t)t * experts;
+  const float* row = z + (size_t)t * ld;
   float peak = -INFINITY, total = 1.f;
   if (softmax) {
     for (int e = lane; e < experts; e += 64) peak = fmaxf(peak, row[e]);
@@ -382,15 +382,16 @@ int blocks_for(size_t total) {
 
 }  // namespace
 
-extern "C" int tnx_route(const float* z, int tokens, int experts, int top, int softmax, int renormalize, int* chosen,
+extern "C" int tnx_route(const float* z, int ld, int tokens, int experts, int top, int softmax, int renormalize, int* chosen,
                          float* weights, const float* correction, float scale, int groups, int keep, hipStream_t stream) {
   TNX_REQUIRE(tokens >= 0 && experts > 0 && top > 0 && top <= experts, "route: %d of %d experts", top, experts);
+  TNX_REQUIRE(ld >= experts, "route: rows of %d logits, %d experts", ld, experts);
   TNX_REQUIRE(experts <= 4096, "route: up to 4096 experts, got %d", experts);
   TNX_REQUIRE(groups >= 1 && groups <= MAX_GROUPS && experts % groups == 0 && keep >= 1 && keep <= groups &&
                   top <= keep * (experts / groups),
               "route: %d of %d experts in %d groups (up to %d) of which %d are kept", top, experts, groups, MAX_GROUPS, keep);
   if (tokens == 0) return 0;
-  route_kernel<<<(tokens + 3) / 4, 256, 0, stream>>>(z, tokens, experts, top, softmax, renormalize, chosen, weights,
+  route_kernel<<<(tokens + 3) / 4, 256, 0, stream>>>(z, ld, tokens, experts, top, softmax, renormalize, chosen, weights,
                                                      correction, scale, groups, keep);
   TNX_CHECK_LAUNCH("route");
   return 0;

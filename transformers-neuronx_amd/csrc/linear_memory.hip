@@ -32,7 +32,8 @@ struct InputArgs {
   const int* slots;
   int unit_size, unit_count, scaled;      // the first unit_count channels are heads of unit_size, made unit vectors
   float scale;                            // on the first `scaled` channels
-  float* u;                 // [T, channels]
+  float* u;                 // [T, u_ld]
+  int u_ld;
   int heads, dt_at, write_at;             // write_at < 0: the write weight is dt
   const float* rate;        // [H]
   const float* dt_bias;     // [H]
@@ -79,7 +80,7 @@ __global__ void __launch_bounds__(256) memory_inputs_kernel(InputArgs a, int pie
 #pragma unroll
     for (int e = 0; e < 4; ++e) at[e] = first + lane + 64 * e, in[e] = at[e] < end;
   }
-  const bool whole = LANES > 0 && in[3] && (a.channels & 3) == 0;       // four neighbours, 16 bytes aligned
+  const bool whole = LANES > 0 && in[3] && ((a.channels | a.u_ld) & 3) == 0;       // four neighbours, 16 bytes aligned
   constexpr int BACK = TAPS > 1 ? TAPS - 1 : 1;
   float taps_w[TAPS > 0 ? TAPS : 1][4], bias[4], scale[4], before[BACK][4];
 #pragma unroll
@@ -175,7 +176,7 @@ __global__ void __launch_bounds__(256) memory_inputs_kernel(InputArgs a, int pie
       }
     }
     const float f = unit ? 1.f / sqrtf(sum + 1e-6f) : 1.f;
-    float* out = a.u + (size_t)t * a.channels;
+    float* out = a.u + (size_t)t * a.u_ld;
     if (whole) {
       f32x4 o;
 #pragma unroll
@@ -425,10 +426,14 @@ void launch_walk_sized(const WalkArgs& a, int requests, bool singles, bool align
 // float32 on the matrix unit (16x16x4: float32 operands, float32 sums). The sums c are taken in float64: their
 // differences decide what a token far back in the chunk still weighs.
 //
-// The matrix unit's operands: lane l holds row (or column) l % 16 and k = l / 16; four instructions take k = 16 kk +
-// 4 (l / 16) + j for j = 0 .. 3, so that a lane reads 16 bytes for four of them. The accumulator: column l % 16, rows
-// 4 (l / 16) + i.
+// The matrix unit's operands: lane l holds row (or column) l % 16 and k = l / 16; four instructions take k = 16 s +
+// 4 (l / 16) + e for e = 0 .. 3, so that a lane holds four neighbours for four of them. The accumulator: column l % 16,
+// rows 4 (l / 16) + e. What the first kernel leaves for the second lies in the order of those lanes (tiles of 64 lanes by
+// four elements): 16 lanes that read 16 bytes each of 16 rows would ask the cache for 16 lines, four times an
+// instruction. Rows are filled up with zeros to 16 NB elements on the way, and tokens beyond a run's last (in its last
+// chunk) have zeros for write weights, so that what else is made of them meets zeros.
 constexpr int CHUNK = 64;
+constexpr int TILE = 256;                 // elements of 64 lanes by four
 
 struct ChunkArgs {
   const float* u;           // [T, ld]
@@ -446,57 +451,89 @@ struct ChunkArgs {
   int num_long;
   float* memory;            // [slots, 2, H, v, n]
   float* out;               // [T, H v]
-  float* ahead;             // [T, H]: e^c_i
-  float* behind;            // [T, H]: e^(c_64 - c_i)
-  float* pairs;             // [chunks, H, 64, 64]: e^(c_i - c_j) (q_i . k_j), j <= i; blocks above the diagonal unwritten
-  float* w;                 // [T, H, n]
-  float* u0;                // [T, H, v]
+  float* gates;             // [chunks, H, 3, 64]: e^c_i, e^(c_64 - c_i), write_i
+  float* qx;                // [chunks, G, 4, NB, tile]: queries, token 16 w + l % 16, elements 16 s + 4 (l / 16) ..
+  float* kx;                // [chunks, G, NB, 4, tile]: keys, element 16 x + l % 16, tokens 16 s + 4 (l / 16) ..
+  float* pairs;             // [chunks, H, 4, 4, tile]: e^(c_i - c_j) (q_i . k_j), i = 16 w + l % 16, j = 16 s + 4 (l / 16) ..;
+                            //   zero for j > i, unwritten for s > w
+  float* wx;                // [chunks, H, 4, NB, tile]: w, as the queries
+  float* ux;                // [chunks, H, blocks of 16 columns, 4, tile]: u0, column l % 16, tokens 16 w + 4 (l / 16) ..
   int heads, groups, n, v;
 };
 
-// grid: chunks * groups * parts of a group's heads, `per` heads a block. Wave w makes rows 16 w .. 16 w + 15 of q . k
-// (and k . k) once for the group, then every head's weights; with DELTA a thread then solves the system for a column.
+// A chunk's queries or keys to LDS, a token's row by row, zeros behind n.
+template <int NB, int THREADS, bool ALIGNED>
+__device__ __forceinline__ void stage_rows(const float* src, int ld, int len, int n, float* dst) {
+  constexpr int LD = 16 * NB + 4, PT = 4 * NB;        // 16-byte pieces of a token
+#pragma unroll 4
+  for (int f = threadIdx.x; f < CHUNK * PT; f += THREADS) {
+    const int t = f / PT, d = 4 * (f - t * PT);
+    *(f32x4*)(dst + t * LD + d) = load4<ALIGNED>(src + (unsigned)(min(t, len - 1) * ld) + d, n - d);
+  }
+}
+
+// grid: chunks * groups * parts of a group's heads, `per` heads a block. Wave w of the first four makes the products
+// q . k of tokens 16 w .. 16 w + 15 once for the group (with DELTA wave 4 + w the products k . k), then every head's weights.
+// With DELTA the system (I + M) x = b, M strictly lower triangular, is solved by blocks of 16 rows: the diagonal blocks
+// are inverted (a lane a column), and x_i = T_ii (b_i - sum_{k<i} M_ik x_k) follows on the matrix unit, two blocks of 16
+// columns of b a wave at a time: an accumulator's rows are just what a lane hands to the next product as its second
+// operand. Dynamic LDS: queries (later w), keys, with DELTA -M and the inverted blocks.
 template <int NB, bool DELTA, bool ALIGNED>
-__global__ void __launch_bounds__(256) memory_pairs_kernel(ChunkArgs a, int parts, int per) {
-  constexpr int MLD = CHUNK + 4;
+__global__ void __launch_bounds__(DELTA ? 512 : 256) memory_pairs_kernel(ChunkArgs a, int parts, int per) {
+  constexpr int THREADS = DELTA ? 512 : 256, WAVES = THREADS / 64;
+  constexpr int LD = 16 * NB + 4, MLD = CHUNK + 4, TLD = 20;
+  extern __shared__ __attribute__((aligned(16))) float room[];
   __shared__ double cs[CHUNK];
-  __shared__ float beta[CHUNK], up[CHUNK];
-  __shared__ __attribute__((aligned(16))) float mt[DELTA ? CHUNK * MLD : 4];      // the system, column by column
+  __shared__ __attribute__((aligned(16))) float beta[CHUNK], up[CHUNK];
+  float* q_l = room;                            // [64][LD]
+  float* k_l = q_l + CHUNK * LD;                // [64][LD]
+  float* mn = k_l + CHUNK * LD;                 // [64][MLD]: -M, row by row
+  float* td = mn + CHUNK * MLD;                 // [64][TLD]: the inverted diagonal blocks
   const int part = blockIdx.x % parts, rest = blockIdx.x / parts;
   const int group = rest % a.groups, chunk = rest / a.groups;
   const int run = a.chunk_run[chunk], begin = a.chunk_begin[chunk];
   const int t0 = a.run_start[run] + begin, len = min(CHUNK, a.run_start[run + 1] - t0);
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
-  const float* q = a.u + a.q_at + group * a.n;
-  const float* k = a.u + a.k_at + group * a.n;
-  f32x4 qk[4], kk[4];
+  const int w4 = wave & 3;
+  const bool keys_side = wave >= 4;             // (DELTA: the waves that make k . k)
+  const float* base = a.u + (size_t)t0 * a.ld;
+  stage_rows<NB, THREADS, ALIGNED>(base + a.q_at + group * a.n, a.ld, len, a.n, q_l);
+  stage_rows<NB, THREADS, ALIGNED>(base + a.k_at + group * a.n, a.ld, len, a.n, k_l);
+  __syncthreads();
+  // prod[cb][e]: token j = 16 cb + 4 g + e (key) with token i = 16 w4 + r
+  f32x4 prod[4];
 #pragma unroll
-  for (int cb = 0; cb < 4; ++cb) qk[cb] = kk[cb] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  for (int cb = 0; cb < 4; ++cb) prod[cb] = (f32x4){0.f, 0.f, 0.f, 0.f};
   {
-    const int i = 16 * wave + r;
-    const size_t row = (size_t)(t0 + min(i, len - 1)) * a.ld;
+    const float* mine = (keys_side ? k_l : q_l) + (16 * w4 + r) * LD + 4 * g;
+    float* qx = a.qx + ((size_t)(chunk * a.groups + group) * 4 + w4) * NB * TILE + 4 * lane;
 #pragma unroll 2
     for (int s = 0; s < NB; ++s) {
-      const int d = 16 * s + 4 * g, valid = i < len ? a.n - d : 0;
-      const f32x4 qa = load4<ALIGNED>(q + row + d, valid);
-      f32x4 ka = {0.f, 0.f, 0.f, 0.f};
-      if (DELTA) ka = load4<ALIGNED>(k + row + d, valid);
+      const f32x4 x = *(const f32x4*)(mine + 16 * s);
+      if (!keys_side && part == 0) *(f32x4*)(qx + s * TILE) = x;
 #pragma unroll
       for (int cb = 0; cb < 4; ++cb) {
-        if (cb > wave) continue;
-        const int j = 16 * cb + r;
-        const f32x4 kb = load4<ALIGNED>(k + (size_t)(t0 + min(j, len - 1)) * a.ld + d, j < len ? a.n - d : 0);
+        if (cb > w4) continue;
+        const f32x4 kb = *(const f32x4*)(k_l + (16 * cb + r) * LD + 16 * s + 4 * g);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          qk[cb] = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[e], kb[e], qk[cb], 0, 0, 0);
-          if (DELTA) kk[cb] = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[e], kb[e], kk[cb], 0, 0, 0);
-        }
+        for (int e = 0; e < 4; ++e) prod[cb] = __builtin_amdgcn_mfma_f32_16x16x4f32(kb[e], x[e], prod[cb], 0, 0, 0);
       }
+    }
+  }
+  if (part == 0) {
+    float* kx = a.kx + (size_t)(chunk * a.groups + group) * NB * 4 * TILE + 4 * lane;
+    for (int f = wave; f < 4 * NB; f += WAVES) {
+      const int x = f >> 2, s = f & 3;
+      f32x4 v;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = k_l[(16 * s + 4 * g + e) * LD + 16 * x + r];
+      *(f32x4*)(kx + f * TILE) = v;
     }
   }
   const int per_group = a.heads / a.groups;
   for (int hh = part * per; hh < min(per_group, (part + 1) * per); ++hh) {
     const int head = group * per_group + hh;
+    const size_t place = (size_t)chunk * a.heads + head;
     if (wave == 0) {
       const size_t at = (size_t)(t0 + min(lane, len - 1)) * a.heads + head;
       double c = lane < len ? (double)a.log_decay[at] : 0.0;
@@ -506,57 +543,126 @@ __global__ void __launch_bounds__(256) memory_pairs_kernel(ChunkArgs a, int part
         if (lane >= d) c += before;
       }
       const double all = __shfl(c, 63, 64);
-      const float e = expf((float)c);
+      const float e = expf((float)c), b = lane < len ? a.write[at] : 0.f;
       cs[lane] = c;
       up[lane] = e;
-      beta[lane] = lane < len ? a.write[at] : 0.f;
-      if (lane < len) {
-        a.ahead[at] = e;
-        a.behind[at] = expf((float)(all - c));
-      }
+      beta[lane] = b;
+      float* gates = a.gates + place * 3 * CHUNK + lane;
+      gates[0] = e;
+      gates[CHUNK] = expf((float)(all - c));
+      gates[2 * CHUNK] = b;
     }
     __syncthreads();
-    float* pairs = a.pairs + ((size_t)chunk * a.heads + head) * CHUNK * CHUNK;
+    {
+      const int i = 16 * w4 + r;
+      const double ci = cs[i];
+      const float bi = beta[i];
+      float* pairs = a.pairs + (place * 4 + w4) * 4 * TILE + 4 * lane;
 #pragma unroll
-    for (int cb = 0; cb < 4; ++cb) {
-      if (cb > wave) continue;
-      const int j = 16 * cb + r;
-      f32x4 m;
+      for (int cb = 0; cb < 4; ++cb) {
+        if (cb > w4) continue;
+        f32x4 v;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int i = 16 * wave + 4 * g + e;
-        const float d = j <= i ? expf((float)(cs[i] - cs[j])) : 0.f;
-        pairs[i * CHUNK + j] = qk[cb][e] * d;
-        if (DELTA) m[e] = j < i ? beta[i] * d * kk[cb][e] : 0.f;
+        for (int e = 0; e < 4; ++e) {
+          const int j = 16 * cb + 4 * g + e;
+          const float x = prod[cb][e] * expf((float)fmin(ci - cs[j], 0.0));
+          if (keys_side)
+            v[e] = j < i ? -bi * x : 0.f;
+          else
+            v[e] = j <= i ? x : 0.f;
+        }
+        if (keys_side)
+          *(f32x4*)(mn + i * MLD + 16 * cb + 4 * g) = v;
+        else
+          *(f32x4*)(pairs + cb * TILE) = v;
       }
-      if (DELTA) *(f32x4*)(mt + j * MLD + 16 * wave + 4 * g) = m;
     }
     if (DELTA) {
       __syncthreads();
-      for (int c = threadIdx.x; c < a.v + a.n; c += 256) {
-        const bool value = c < a.v;
-        const float* src = a.u + (size_t)t0 * a.ld + (value ? a.v_at + head * a.v + c : a.k_at + group * a.n + c - a.v);
-        float x[CHUNK];
+      if (wave < 4) {
+        // the inverse of I + M_ww: column r, x_i = [i = r] - sum_{j<i} M[i, j] x_j
+        const float* m = mn + 16 * wave * MLD + 16 * wave;
+        float x[16];
 #pragma unroll
-        for (int i = 0; i < CHUNK; ++i) x[i] = i < len ? src[(size_t)i * a.ld] : 0.f;
+        for (int i = 0; i < 16; ++i) {
+          float acc = i == r ? 1.f : 0.f;
 #pragma unroll
-        for (int i = 0; i < CHUNK; ++i) x[i] *= value ? beta[i] : beta[i] * up[i];
-#pragma unroll
-        for (int j = 0; j < CHUNK - 1; ++j) {
-#pragma unroll
-          for (int i4 = j / 4; i4 < CHUNK / 4; ++i4) {
-            const f32x4 m = *(const f32x4*)(mt + j * MLD + 4 * i4);
+          for (int j4 = 0; j4 < (i + 3) / 4; ++j4) {
+            const f32x4 row = *(const f32x4*)(m + i * MLD + 4 * j4);
 #pragma unroll
             for (int e = 0; e < 4; ++e)
-              if (4 * i4 + e > j) x[4 * i4 + e] -= m[e] * x[j];
+              if (4 * j4 + e < i) acc += row[e] * x[4 * j4 + e];
+          }
+          x[i] = acc;
+        }
+        if (g == 0) {
+#pragma unroll
+          for (int i = 0; i < 16; ++i) td[(16 * wave + i) * TLD + r] = x[i];
+        }
+      }
+      __syncthreads();
+      const float* vals = base + a.v_at + head * a.v;
+      const int vb = (a.v + 15) / 16;
+      for (int b0 = 2 * wave; b0 < vb + NB; b0 += 2 * WAVES) {      // blocks of 16 columns: the values', then the keys'
+        f32x4 x[2][4];                                              // [block of columns][block of rows]
+#pragma unroll
+        for (int cc = 0; cc < 2; ++cc) {
+          const bool value = b0 + cc < vb;
+          const int c = 16 * (b0 + cc) + r, d = min(16 * (b0 + cc - vb) + r, 16 * NB - 1);
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              const int t = 16 * i + 4 * g + e;
+              if (value)
+                x[cc][i][e] = vals[(unsigned)(min(t, len - 1) * a.ld) + min(c, a.v - 1)];
+              else
+                x[cc][i][e] = k_l[t * LD + d] * up[t];
+            }
+#pragma unroll
+          for (int i = 0; i < 4; ++i) x[cc][i] = x[cc][i] * *(const f32x4*)(beta + 16 * i + 4 * g);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+#pragma unroll
+          for (int kb = 0; kb < i; ++kb) {
+            const f32x4 m = *(const f32x4*)(mn + (16 * i + r) * MLD + 16 * kb + 4 * g);
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+#pragma unroll
+              for (int cc = 0; cc < 2; ++cc) x[cc][i] = __builtin_amdgcn_mfma_f32_16x16x4f32(m[e], x[cc][kb][e], x[cc][i], 0, 0, 0);
+          }
+          const f32x4 t = *(const f32x4*)(td + (16 * i + r) * TLD + 4 * g);
+          f32x4 y[2];
+#pragma unroll
+          for (int cc = 0; cc < 2; ++cc) y[cc] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int cc = 0; cc < 2; ++cc) y[cc] = __builtin_amdgcn_mfma_f32_16x16x4f32(t[e], x[cc][i][e], y[cc], 0, 0, 0);
+#pragma unroll
+          for (int cc = 0; cc < 2; ++cc) x[cc][i] = y[cc];
+        }
+#pragma unroll
+        for (int cc = 0; cc < 2; ++cc) {
+          if (b0 + cc < vb) {
+            float* ux = a.ux + (place * vb + b0 + cc) * 4 * TILE + 4 * lane;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) *(f32x4*)(ux + i * TILE) = x[cc][i];
+          } else if (b0 + cc < vb + NB) {
+            const int d = 16 * (b0 + cc - vb) + r;
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+              for (int e = 0; e < 4; ++e) q_l[(16 * i + 4 * g + e) * LD + d] = x[cc][i][e];      // (nobody reads the queries any more)
           }
         }
-        float* dst = value ? a.u0 + ((size_t)t0 * a.heads + head) * a.v + c
-                           : a.w + ((size_t)t0 * a.heads + head) * a.n + c - a.v;
-        const size_t step = (size_t)a.heads * (value ? a.v : a.n);
-#pragma unroll
-        for (int i = 0; i < CHUNK; ++i)
-          if (i < len) dst[(size_t)i * step] = x[i];
+      }
+      __syncthreads();
+      float* wx = a.wx + place * 4 * NB * TILE + 4 * lane;
+      for (int f = wave; f < 4 * NB; f += WAVES) {
+        const int w = f / NB, s = f - w * NB;
+        *(f32x4*)(wx + f * TILE) = *(const f32x4*)(q_l + (16 * w + r) * LD + 16 * s + 4 * g);
       }
     }
     __syncthreads();      // before the next head's decays
@@ -566,9 +672,10 @@ __global__ void __launch_bounds__(256) memory_pairs_kernel(ChunkArgs a, int part
 // grid: (run, head) pairs in eights * column blocks: the blocks of a (run, head) come eight apart, so that they share an
 // XCD's cache. A block walks a run's chunks for 16 columns of S; wave w has the chunk's tokens 16 w .. 16 w + 15, and of S
 // the blocks of 16 rows w, w + 4, ..., in the accumulators from chunk to chunk. What a chunk's products read of memory is
-// asked for during the products before them.
+// asked for two chunks ahead, into the registers (one set for even, one for odd chunks) that the chunk before last has
+// just read: a compute unit has one such block, and a load takes as long as a chunk's products do.
 template <int NB, bool DELTA, bool ALIGNED>
-__global__ void __launch_bounds__(256) memory_scan_kernel(ChunkArgs a, int column_blocks) {
+__global__ void __launch_bounds__(256, 1) memory_scan_kernel(ChunkArgs a, int column_blocks) {
   constexpr int RB = (NB + 3) / 4;               // blocks of rows of S a wave
   constexpr int SLD = 16 * NB + 4, ULD = CHUNK + 4;
   __shared__ __attribute__((aligned(16))) float s_l[16 * SLD];        // [column][row]
@@ -583,67 +690,70 @@ __global__ void __launch_bounds__(256) memory_scan_kernel(ChunkArgs a, int colum
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
   const int col = 16 * cb + r;
   const bool col_ok = col < a.v;
+  const int ccol = col_ok ? col : 0;
   const int from = (have - 1) & 1, to = (have + count - 1) & 1;
   const size_t head_at = (size_t)slot * 2 * a.heads + head;
   const f32x4 zero4 = {0.f, 0.f, 0.f, 0.f};
-  f32x4 S[RB];
+  f32x4 S[RB];                                   // (rows from n on stay zero: the keys have zeros there)
+  auto share = [&]() {
+#pragma unroll
+    for (int x = 0; x < RB; ++x)
+      if (wave + 4 * x < NB) *(f32x4*)(s_l + r * SLD + 16 * (wave + 4 * x) + 4 * g) = S[x];
+  };
 #pragma unroll
   for (int x = 0; x < RB; ++x) {
     const int row = 16 * (wave + 4 * x) + 4 * g;
-    const float* p = a.memory + ((head_at + (size_t)from * a.heads) * a.v + (col_ok ? col : 0)) * a.n + row;
+    const float* p = a.memory + ((head_at + (size_t)from * a.heads) * a.v + ccol) * a.n + row;
     S[x] = load4<ALIGNED>(p, have > 0 && col_ok ? a.n - row : 0);
-    if (wave + 4 * x < NB) *(f32x4*)(s_l + r * SLD + row) = S[x];
   }
-  f32x4 wa[DELTA ? NB : 1], qa[NB], pa[4];
-  float kt[RB][4][4], u0[4], up[4], down[4], decay = 0.f;
-  const float* q = a.u + a.q_at + group * a.n;
-  const float* k = a.u + a.k_at + group * a.n;
-  auto fetch_state_side = [&](int c) {          // what meets S: this wave's tokens' queries and rows of w, their u0
+  share();
+  struct Set {
+    f32x4 wa[DELTA ? NB : 1], qa[NB], pa[4], kt[RB][4], u0, up, down, wr;
+    float decay;
+  };
+  Set even, odd;
+  auto fetch_state_side = [&](int c, Set& z) {          // what meets S: this wave's tokens' queries and rows of w, their u0
     const int t0 = start + CHUNK * c, len = min(CHUNK, count - CHUNK * c);
-    const int i = 16 * wave + r;
-    const size_t t = t0 + min(i, len - 1);
+    const size_t of_group = (size_t)(first + c) * a.groups + group, of_head = (size_t)(first + c) * a.heads + head;
+    const float* q = a.qx + (of_group * 4 + wave) * NB * TILE + 4 * lane;
+    const float* w = a.wx + (of_head * 4 + wave) * NB * TILE + 4 * lane;
 #pragma unroll
     for (int s = 0; s < NB; ++s) {
-      const int d = 16 * s + 4 * g, valid = i < len ? a.n - d : 0;
-      qa[s] = load4<ALIGNED>(q + t * a.ld + d, valid);
-      if (DELTA) wa[DELTA ? s : 0] = load4<ALIGNED>(a.w + (t * a.heads + head) * a.n + d, valid);
+      z.qa[s] = *(const f32x4*)(q + s * TILE);
+      if (DELTA) z.wa[DELTA ? s : 0] = *(const f32x4*)(w + s * TILE);
     }
+    if (DELTA) {
+      z.u0 = *(const f32x4*)(a.ux + ((of_head * column_blocks + cb) * 4 + wave) * TILE + 4 * lane);
+    } else {
+      const float* vals = a.u + (size_t)t0 * a.ld + a.v_at + head * a.v + ccol;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int it = 16 * wave + 4 * g + e;
-      const size_t tt = t0 + min(it, len - 1);
-      const bool in = it < len && col_ok;
-      if (DELTA)
-        u0[e] = in ? a.u0[(tt * a.heads + head) * a.v + col] : 0.f;
-      else
-        u0[e] = in ? a.write[tt * a.heads + head] * a.u[tt * a.ld + a.v_at + head * a.v + col] : 0.f;
-      up[e] = a.ahead[tt * a.heads + head];
-      down[e] = a.behind[tt * a.heads + head];
+      for (int e = 0; e < 4; ++e) z.u0[e] = vals[(unsigned)(min(16 * wave + 4 * g + e, len - 1) * a.ld)];
     }
-    decay = a.ahead[(size_t)(t0 + len - 1) * a.heads + head];
+    const float* gates = a.gates + of_head * 3 * CHUNK;
+    z.up = *(const f32x4*)(gates + 16 * wave + 4 * g);
+    z.down = *(const f32x4*)(gates + CHUNK + 16 * wave + 4 * g);
+    if (!DELTA) z.wr = *(const f32x4*)(gates + 2 * CHUNK + 16 * wave + 4 * g);
+    z.decay = gates[CHUNK - 1];
   };
-  auto fetch_token_side = [&](int c) {          // what meets the writes: the weights among the tokens, the keys
-    const int t0 = start + CHUNK * c, len = min(CHUNK, count - CHUNK * c);
-    const float* pairs = a.pairs + ((size_t)(first + c) * a.heads + head) * CHUNK * CHUNK + (16 * wave + r) * CHUNK;
+  auto fetch_token_side = [&](int c, Set& z) {          // what meets the writes: the weights among the tokens, the keys
+    const float* pairs = a.pairs + (((size_t)(first + c) * a.heads + head) * 4 + wave) * 4 * TILE + 4 * lane;
+    const float* k = a.kx + ((size_t)(first + c) * a.groups + group) * NB * 4 * TILE + 4 * lane;
 #pragma unroll
-    for (int s = 0; s < 4; ++s) pa[s] = s <= wave ? *(const f32x4*)(pairs + 16 * s + 4 * g) : zero4;
+    for (int s = 0; s < 4; ++s) z.pa[s] = *(const f32x4*)(pairs + min(s, wave) * TILE);
 #pragma unroll
-    for (int x = 0; x < RB; ++x) {
-      const int row = 16 * (wave + 4 * x) + r;
+    for (int x = 0; x < RB; ++x)
 #pragma unroll
-      for (int s = 0; s < 4; ++s)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const int j = 16 * s + 4 * g + e;
-          kt[x][s][e] = j < len && row < a.n ? k[(size_t)(t0 + j) * a.ld + row] : 0.f;
-        }
-    }
+      for (int s = 0; s < 4; ++s) z.kt[x][s] = *(const f32x4*)(k + (4 * min(wave + 4 * x, NB - 1) + s) * TILE);
   };
-  fetch_state_side(0);
-  fetch_token_side(0);
-  __syncthreads();
   const int chunks = (count + CHUNK - 1) / CHUNK;
-  for (int c = 0; c < chunks; ++c) {
+  fetch_state_side(0, even);
+  fetch_token_side(0, even);
+  if (chunks > 1) {
+    fetch_state_side(1, odd);
+    fetch_token_side(1, odd);
+  }
+  __syncthreads();
+  auto chunk = [&](int c, Set& z) {
     const int t0 = start + CHUNK * c, len = min(CHUNK, count - CHUNK * c);
     f32x4 o = zero4, m = zero4;
 #pragma unroll
@@ -651,21 +761,16 @@ __global__ void __launch_bounds__(256) memory_scan_kernel(ChunkArgs a, int colum
       const f32x4 s4 = *(const f32x4*)(s_l + r * SLD + 16 * s + 4 * g);
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        o = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[s][e], s4[e], o, 0, 0, 0);
-        if (DELTA) m = __builtin_amdgcn_mfma_f32_16x16x4f32(wa[DELTA ? s : 0][e], s4[e], m, 0, 0, 0);
+        o = __builtin_amdgcn_mfma_f32_16x16x4f32(z.qa[s][e], s4[e], o, 0, 0, 0);
+        if (DELTA) m = __builtin_amdgcn_mfma_f32_16x16x4f32(z.wa[DELTA ? s : 0][e], s4[e], m, 0, 0, 0);
       }
     }
-    f32x4 u4, b4;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      u4[e] = u0[e] - m[e];
-      b4[e] = u4[e] * down[e];
-      o[e] *= up[e];
-    }
+    const f32x4 u4 = DELTA ? z.u0 - m : z.wr * z.u0;
     *(f32x4*)(u_l + r * ULD + 16 * wave + 4 * g) = u4;
-    *(f32x4*)(b_l + r * ULD + 16 * wave + 4 * g) = b4;
-    const float keep = decay;
-    if (c + 1 < chunks) fetch_state_side(c + 1);
+    *(f32x4*)(b_l + r * ULD + 16 * wave + 4 * g) = u4 * z.down;
+    o = o * z.up;
+    const float keep = z.decay;
+    if (c + 2 < chunks) fetch_state_side(c + 2, z);
     __syncthreads();
 #pragma unroll
     for (int x = 0; x < RB; ++x) S[x] = S[x] * keep;
@@ -674,22 +779,27 @@ __global__ void __launch_bounds__(256) memory_scan_kernel(ChunkArgs a, int colum
       const f32x4 us = *(const f32x4*)(u_l + r * ULD + 16 * s + 4 * g);
       const f32x4 bs = *(const f32x4*)(b_l + r * ULD + 16 * s + 4 * g);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        if (s <= wave) o = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[s][e], us[e], o, 0, 0, 0);
+      for (int e = 0; e < 4; ++e)
 #pragma unroll
-        for (int x = 0; x < RB; ++x) S[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[x][s][e], bs[e], S[x], 0, 0, 0);
+        for (int x = 0; x < RB; ++x) S[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(z.kt[x][s][e], bs[e], S[x], 0, 0, 0);
+      if (s <= wave) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o = __builtin_amdgcn_mfma_f32_16x16x4f32(z.pa[s][e], us[e], o, 0, 0, 0);
       }
     }
-    if (c + 1 < chunks) fetch_token_side(c + 1);
-#pragma unroll
-    for (int x = 0; x < RB; ++x)
-      if (wave + 4 * x < NB) *(f32x4*)(s_l + r * SLD + 16 * (wave + 4 * x) + 4 * g) = S[x];
+    if (c + 2 < chunks) fetch_token_side(c + 2, z);
+    share();
+    float* out = a.out + ((size_t)t0 * a.heads + head) * a.v + ccol;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int i = 16 * wave + 4 * g + e;
-      if (i < len && col_ok) a.out[((size_t)(t0 + i) * a.heads + head) * a.v + col] = o[e];
+      if (i < len && col_ok) out[(unsigned)(i * a.heads * a.v)] = o[e];
     }
     __syncthreads();
+  };
+  for (int c = 0; c < chunks; c += 2) {
+    chunk(c, even);
+    if (c + 1 < chunks) chunk(c + 1, odd);
   }
   if (!col_ok) return;
 #pragma unroll
@@ -706,35 +816,39 @@ __global__ void __launch_bounds__(256) memory_scan_kernel(ChunkArgs a, int colum
   }
 }
 
-template <int NB, bool DELTA>
-void launch_chunks(const ChunkArgs& a, bool aligned, hipStream_t stream) {
+template <int NB, bool DELTA, bool ALIGNED>
+int launch_chunks(const ChunkArgs& a, hipStream_t stream) {
   const int per_group = a.heads / a.groups;
   int per = 1;                                   // heads of a group a block of the first kernel
   while (!DELTA && per < per_group && (long long)a.chunks * a.groups * ((per_group + 2 * per - 1) / (2 * per)) >= 2 * tnx_compute_units())
     per *= 2;
   const int parts = (per_group + per - 1) / per;
-  const dim3 pair_grid((unsigned)((size_t)a.chunks * a.groups * parts));
   const int column_blocks = (a.v + 15) / 16;
-  const dim3 scan_grid((unsigned)((a.num_long * a.heads + 7) / 8 * 8 * column_blocks));
-  if (aligned) {
-    memory_pairs_kernel<NB, DELTA, true><<<pair_grid, 256, 0, stream>>>(a, parts, per);
-    memory_scan_kernel<NB, DELTA, true><<<scan_grid, 256, 0, stream>>>(a, column_blocks);
-  } else {
-    memory_pairs_kernel<NB, DELTA, false><<<pair_grid, 256, 0, stream>>>(a, parts, per);
-    memory_scan_kernel<NB, DELTA, false><<<scan_grid, 256, 0, stream>>>(a, column_blocks);
+  const int lds = (2 * CHUNK * (16 * NB + 4) + (DELTA ? CHUNK * (CHUNK + 4) + CHUNK * 20 : 0)) * (int)sizeof(float);
+  static bool configured = false;
+  if (!configured) {
+    const hipError_t e = hipFuncSetAttribute((const void*)memory_pairs_kernel<NB, DELTA, ALIGNED>,
+                                             hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    TNX_REQUIRE(e == hipSuccess, "memory_chunks: cannot reserve %d bytes of LDS: %s", lds, hipGetErrorString(e));
+    configured = true;
   }
+  memory_pairs_kernel<NB, DELTA, ALIGNED>
+      <<<(unsigned)((size_t)a.chunks * a.groups * parts), DELTA ? 512 : 256, lds, stream>>>(a, parts, per);
+  TNX_CHECK_LAUNCH("memory_pairs");
+  memory_scan_kernel<NB, DELTA, ALIGNED>
+      <<<(unsigned)((a.num_long * a.heads + 7) / 8 * 8 * column_blocks), 256, 0, stream>>>(a, column_blocks);
+  TNX_CHECK_LAUNCH("memory_scan");
+  return 0;
 }
 
-template <bool DELTA>
-void launch_chunks_sized(const ChunkArgs& a, bool aligned, hipStream_t stream) {
-  if (a.n <= 32)
-    launch_chunks<2, DELTA>(a, aligned, stream);
-  else if (a.n <= 64)
-    launch_chunks<4, DELTA>(a, aligned, stream);
-  else if (a.n <= 128)
-    launch_chunks<8, DELTA>(a, aligned, stream);
-  else
-    launch_chunks<16, DELTA>(a, aligned, stream);
+template <bool DELTA, bool ALIGNED>
+int launch_chunks_sized(const ChunkArgs& a, int nb, hipStream_t stream) {
+  switch (nb) {
+    case 2: return launch_chunks<2, DELTA, ALIGNED>(a, stream);
+    case 4: return launch_chunks<4, DELTA, ALIGNED>(a, stream);
+    case 8: return launch_chunks<8, DELTA, ALIGNED>(a, stream);
+    default: return launch_chunks<16, DELTA, ALIGNED>(a, stream);
+  }
 }
 
 // ------------------------------------------------------------------------------------------ after the memory
@@ -755,77 +869,115 @@ struct FinishArgs {
 };
 
 // A row's `parts` equal parts at unit root mean square, times weight; (o + skip x) silu(gate) before the norm or
-// silu(gate) after it. A part is THREADS threads' work, element by element or (VEC) four neighbours a thread.
-template <typename T, int THREADS, int VEC>
+// silu(gate) after it. A part is THREADS threads' work, four neighbours a thread at a time (ALIGNED: 16-byte loads; parts,
+// rows and heads begin at multiples of four elements). HELD pieces of a part stay in registers between the two passes.
+template <typename T, int THREADS, bool ALIGNED>
 __global__ void __launch_bounds__(256) gated_norm_kernel(FinishArgs a) {
   __shared__ float scratch[4];
   constexpr int PER_BLOCK = 256 / THREADS;
-  const long long idx = (long long)blockIdx.x * PER_BLOCK + (THREADS == 256 ? 0 : threadIdx.x >> 6);
+  const long long idx = (long long)blockIdx.x * PER_BLOCK + (THREADS == 256 ? 0 : threadIdx.x / THREADS);
   const bool active = idx < (long long)a.tokens * a.parts;
-  if (THREADS < 256 && !active) return;
+  if (THREADS == 64 && !active) return;
   const size_t t = active ? idx / a.parts : 0;
   const int part = active ? (int)(idx - (long long)t * a.parts) : 0;
   const int size = a.width / a.parts, first = part * size;
-  const int me = THREADS == 256 ? threadIdx.x : threadIdx.x & 63;
+  const int me = threadIdx.x % THREADS;
   const float* o = a.o + t * a.width + first;
   const float* gate = a.gate + t * a.gate_ld + first;
   const float* x = a.skip ? a.x + t * a.x_ld + first : nullptr;
-  auto value = [&](int i) {
-    float y = o[i];
-    if (x) y += a.skip[(first + i) / a.per_head] * x[i];
-    if (a.gate_first) y *= silu(gate[i]);
+  auto value = [&](int i) {            // elements i .. i + 3, zeros from the part's end on
+    f32x4 y = load4<ALIGNED>(o + i, size - i);
+    if (x) {
+      const f32x4 xs = load4<ALIGNED>(x + i, size - i);
+      if (ALIGNED) {
+        y = y + a.skip[(first + i) / a.per_head] * xs;
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (i + e < size) y[e] += a.skip[(first + i + e) / a.per_head] * xs[e];
+      }
+    }
+    if (a.gate_first) {
+      const f32x4 gs = load4<ALIGNED>(gate + i, size - i);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[e] *= silu(gs[e]);
+    }
     return y;
   };
-  constexpr int HELD = 4;              // so many pieces of a part stay in registers between the two passes
-  float held[HELD][VEC];
+  constexpr int HELD = 2;
+  f32x4 held[HELD];
   float s = 0.f;
 #pragma unroll
   for (int c = 0; c < HELD; ++c) {
-    const int i = VEC * (me + THREADS * c);
+    const int i = 4 * (me + THREADS * c);
+    held[c] = i < size ? value(i) : (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) {
-      held[c][e] = i + e < size ? value(i + e) : 0.f;
-      s += held[c][e] * held[c][e];
+    for (int e = 0; e < 4; ++e) s += held[c][e] * held[c][e];
+  }
+  for (int i = 4 * (me + THREADS * HELD); i < size; i += 4 * THREADS) {
+    const f32x4 y = value(i);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) s += y[e] * y[e];
+  }
+  if (THREADS == 256) {
+    s = block_sum<4>(s, scratch);
+  } else {
+    s = sum16(s);
+    if (THREADS >= 32) {
+      unsigned lo, hi;
+      swap_rows(__float_as_uint(s), lo, hi);
+      s = __uint_as_float(lo) + __uint_as_float(hi);
+    }
+    if (THREADS >= 64) {
+      unsigned lo, hi;
+      swap_halves(__float_as_uint(s), lo, hi);
+      s = __uint_as_float(lo) + __uint_as_float(hi);
     }
   }
-  for (int i = VEC * (me + THREADS * HELD); i < size; i += VEC * THREADS)
-#pragma unroll
-    for (int e = 0; e < VEC; ++e) {
-      const float y = i + e < size ? value(i + e) : 0.f;
-      s += y * y;
-    }
-  s = THREADS == 256 ? block_sum<4>(s, scratch) : wave_sum(s);
+  if (!active) return;
   const float r = 1.f / sqrtf(s / (float)size + a.eps);
   T* out = (T*)a.out + t * a.width + first;
   const float* w = a.weight + first;
-  auto put = [&](int i, float y) {
-    y *= r * w[i];
-    if (!a.gate_first) y *= silu(gate[i]);
-    out[i] = from_f32<T>(y);
+  auto put = [&](int i, f32x4 y) {
+    const f32x4 ws = load4<ALIGNED>(w + i, size - i);
+    y = y * r * ws;
+    if (!a.gate_first) {
+      const f32x4 gs = load4<ALIGNED>(gate + i, size - i);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[e] *= silu(gs[e]);
+    }
+    typedef T four __attribute__((ext_vector_type(4)));
+    four v;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = from_f32<T>(y[e]);
+    if (ALIGNED) {
+      *(four*)(out + i) = v;
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (i + e < size) out[i + e] = v[e];
+    }
   };
 #pragma unroll
   for (int c = 0; c < HELD; ++c) {
-    const int i = VEC * (me + THREADS * c);
-#pragma unroll
-    for (int e = 0; e < VEC; ++e)
-      if (i + e < size) put(i + e, held[c][e]);
+    const int i = 4 * (me + THREADS * c);
+    if (i < size) put(i, held[c]);
   }
-  for (int i = VEC * (me + THREADS * HELD); i < size; i += VEC * THREADS)
-#pragma unroll
-    for (int e = 0; e < VEC; ++e)
-      if (i + e < size) put(i + e, value(i + e));
+  for (int i = 4 * (me + THREADS * HELD); i < size; i += 4 * THREADS) put(i, value(i));
 }
 
-template <typename T>
+template <typename T, bool ALIGNED>
 void launch_gated_norm(const FinishArgs& a, hipStream_t stream) {
   const int size = a.width / a.parts;
   const long long rows = (long long)a.tokens * a.parts;
   if (size <= 64)
-    gated_norm_kernel<T, 64, 1><<<(unsigned)((rows + 3) / 4), 256, 0, stream>>>(a);
-  else if (size <= 256)
-    gated_norm_kernel<T, 64, 4><<<(unsigned)((rows + 3) / 4), 256, 0, stream>>>(a);
+    gated_norm_kernel<T, 16, ALIGNED><<<(unsigned)((rows + 15) / 16), 256, 0, stream>>>(a);
+  else if (size <= 128)
+    gated_norm_kernel<T, 32, ALIGNED><<<(unsigned)((rows + 7) / 8), 256, 0, stream>>>(a);
+  else if (size <= 512)
+    gated_norm_kernel<T, 64, ALIGNED><<<(unsigned)((rows + 3) / 4), 256, 0, stream>>>(a);
   else
-    gated_norm_kernel<T, 256, 4><<<(unsigned)rows, 256, 0, stream>>>(a);
+    gated_norm_kernel<T, 256, ALIGNED><<<(unsigned)rows, 256, 0, stream>>>(a);
 }
 
 }  // namespace
@@ -833,12 +985,13 @@ void launch_gated_norm(const FinishArgs& a, hipStream_t stream) {
 extern "C" int tnx_memory_inputs(const float* proj, int ld, int conv_at, int channels, const float* w, const float* bias,
                                  float* state, int taps, const int* positions, const int* token_request,
                                  const int* run_start, const int* slots, int unit_size, int unit_count, int scaled,
-                                 float scale, float* u, int heads, int dt_at, int write_at, const float* rate,
+                                 float scale, float* u, int u_ld, int heads, int dt_at, int write_at, const float* rate,
                                  const float* dt_bias, float* log_decay, float* write, int tokens, int runs,
                                  hipStream_t stream) {
   TNX_REQUIRE(tokens >= 0 && runs >= 0 && channels > 0 && taps >= 1 && heads > 0, "memory_inputs: bad sizes");
   TNX_REQUIRE(conv_at >= 0 && ld >= conv_at + channels && dt_at >= 0 && ld >= dt_at + heads && ld >= write_at + heads,
               "memory_inputs: rows of %d elements do not hold what is read", ld);
+  TNX_REQUIRE(u_ld >= channels, "memory_inputs: result rows of %d elements, %d needed", u_ld, channels);
   TNX_REQUIRE(taps == 1 || state, "memory_inputs: %d taps need the requests' state", taps);
   TNX_REQUIRE(unit_count >= 0 && unit_count <= channels && scaled <= channels &&
                   (unit_count == 0 || (unit_size > 0 && unit_size <= 256 && unit_count % unit_size == 0)),
@@ -847,7 +1000,7 @@ extern "C" int tnx_memory_inputs(const float* proj, int ld, int conv_at, int cha
   if (tokens == 0 || runs == 0) return 0;
   const bool singles = tokens == runs;
   InputArgs a{proj, ld, conv_at, channels, w, bias, taps > 1 ? state : nullptr, taps, positions, token_request, run_start, slots,
-              unit_count ? unit_size : 0, unit_count, scaled, scale, u, heads, dt_at, write_at, rate, dt_bias, log_decay, write,
+              unit_count ? unit_size : 0, unit_count, scaled, scale, u, u_ld, heads, dt_at, write_at, rate, dt_bias, log_decay, write,
               tokens, singles};
   int lanes = 0;
   if (unit_count == 0 || unit_size == 64)
@@ -913,31 +1066,40 @@ extern "C" int tnx_memory_walk(const float* u, int ld, int q_at, int k_at, int v
 }
 
 // The runs of several tokens that `long_run` names, chunk by chunk: `chunk_run` and `chunk_begin` name the chunks of 64
-// tokens, a run's chunks one behind the other from `long_first` on. `ahead`, `behind` [T, H], `pairs` [chunks, H, 64, 64],
-// and with `delta` `w` [T, H, n] and `u0` [T, H, v] are room for what the first kernel leaves for the second.
+// tokens, a run's chunks one behind the other from `long_first` on. `room`: what the first kernel leaves for the second,
+// `room_size` floats: with nb = 2, 4, 8 or 16, the least with n <= 16 nb, for every chunk 2 G 1024 nb + H (3 * 64 + 4096),
+// and with `delta` H (1024 nb + 1024 ceil(v / 16)) more.
 extern "C" int tnx_memory_chunks(const float* u, int ld, int q_at, int k_at, int v_at, const float* log_decay,
                                  const float* write, const int* run_start, const int* cached, const int* slots,
                                  const int* chunk_run, const int* chunk_begin, int chunks, int chunk_size, const int* long_run,
-                                 const int* long_first, int num_long, float* memory, float* out, float* ahead, float* behind,
-                                 float* pairs, float* w, float* u0, int heads, int groups, int n, int v, int delta,
-                                 hipStream_t stream) {
+                                 const int* long_first, int num_long, float* memory, float* out, float* room,
+                                 long long room_size, int heads, int groups, int n, int v, int delta, hipStream_t stream) {
   TNX_REQUIRE(heads > 0 && groups > 0 && heads % groups == 0 && n > 0 && v > 0 && n <= 256, "memory_chunks: bad sizes");
   TNX_REQUIRE(chunk_size == CHUNK, "memory_chunks: chunks of %d tokens, the kernels take %d", chunk_size, CHUNK);
   TNX_REQUIRE(q_at >= 0 && k_at >= 0 && v_at >= 0 && ld >= q_at + groups * n && ld >= k_at + groups * n && ld >= v_at + heads * v,
               "memory_chunks: rows of %d elements do not hold what is read", ld);
-  TNX_REQUIRE(ahead && behind && pairs && (!delta || (w && u0)), "memory_chunks: no room for what is made ahead");
   if (chunks <= 0 || num_long <= 0) return 0;
   TNX_REQUIRE((long long)chunks * heads < (1ll << 30) && ((long long)num_long * heads + 7) * ((v + 15) / 16) < (1ll << 31),
               "memory_chunks: too many blocks");
+  TNX_REQUIRE((long long)CHUNK * ld < (1ll << 31) && (long long)CHUNK * heads * v < (1ll << 31), "memory_chunks: rows too long");
+  const int nb = n <= 32 ? 2 : n <= 64 ? 4 : n <= 128 ? 8 : 16, vb = (v + 15) / 16;
   ChunkArgs a{u, ld, q_at, k_at, v_at, log_decay, write, run_start, cached, slots, chunk_run, chunk_begin, chunks, long_run,
-              long_first, num_long, memory, out, ahead, behind, pairs, w, u0, heads, groups, n, v};
+              long_first, num_long, memory, out, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, heads, groups, n, v};
+  const size_t of_group = (size_t)chunks * groups, of_head = (size_t)chunks * heads;
+  float* at = room;
+  a.qx = at, at += of_group * 4 * nb * TILE;
+  a.kx = at, at += of_group * 4 * nb * TILE;
+  a.pairs = at, at += of_head * 16 * TILE;
+  a.gates = at, at += of_head * 3 * CHUNK;
+  if (delta) {
+    a.wx = at, at += of_head * 4 * nb * TILE;
+    a.ux = at, at += of_head * vb * 4 * TILE;
+  }
+  TNX_REQUIRE(room && (uintptr_t)room % 16 == 0 && at - room <= room_size, "memory_chunks: %lld floats of room, %lld needed",
+              room_size, (long long)(at - room));
   const bool aligned = n % 4 == 0 && ((ld | q_at | k_at) & 3) == 0 && (uintptr_t)u % 16 == 0;
-  if (delta)
-    launch_chunks_sized<true>(a, aligned, stream);
-  else
-    launch_chunks_sized<false>(a, aligned, stream);
-  TNX_CHECK_LAUNCH("memory_chunks");
-  return 0;
+  if (delta) return aligned ? launch_chunks_sized<true, true>(a, nb, stream) : launch_chunks_sized<true, false>(a, nb, stream);
+  return aligned ? launch_chunks_sized<false, true>(a, nb, stream) : launch_chunks_sized<false, false>(a, nb, stream);
 }
 
 extern "C" int tnx_gated_norm(const float* o, const float* gate, long long gate_ld, const float* weight, float eps, int parts,
@@ -949,10 +1111,19 @@ extern "C" int tnx_gated_norm(const float* o, const float* gate, long long gate_
   TNX_REQUIRE((long long)tokens * parts < (1ll << 31), "gated_norm: too many rows");
   if (tokens == 0) return 0;
   FinishArgs a{o, gate, gate_ld, weight, eps, parts, gate_first, skip, x, x_ld, skip ? width / skip_heads : 1, out, tokens, width};
-  if (dtype == TNX_F32)
-    launch_gated_norm<float>(a, stream);
-  else
-    launch_gated_norm<bf16_t>(a, stream);
+  const bool aligned = (width / parts) % 4 == 0 && gate_ld % 4 == 0 && (uintptr_t)gate % 16 == 0 && (uintptr_t)o % 16 == 0 &&
+                       (uintptr_t)weight % 16 == 0 && (uintptr_t)out % 16 == 0 &&
+                       (!skip || (x_ld % 4 == 0 && a.per_head % 4 == 0 && (uintptr_t)x % 16 == 0));
+  if (dtype == TNX_F32) {
+    if (aligned)
+      launch_gated_norm<float, true>(a, stream);
+    else
+      launch_gated_norm<float, false>(a, stream);
+  } else if (aligned) {
+    launch_gated_norm<bf16_t, true>(a, stream);
+  } else {
+    launch_gated_norm<bf16_t, false>(a, stream);
+  }
   TNX_CHECK_LAUNCH("gated_norm");
   return 0;
 }

@@ -13,7 +13,7 @@ import torch
 
 from . import build
 from .attention_plan import QUERY_TILE
-from .memory_plan import MEMORY_CHUNK, MEMORY_LONG
+from .memory_plan import MEMORY_CHUNK
 from .. import debug
 
 _F32, _BF16 = 0, 1
@@ -138,7 +138,7 @@ _SIGNATURES = {
                               _c_int, _c_float, _c_void_p],
     },
     "experts": {
-        "tnx_route": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_float,
+        "tnx_route": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_float,
                       _c_int, _c_int, _c_void_p],
         "tnx_expert_mixture": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                                _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
@@ -177,13 +177,12 @@ _SIGNATURES = {
     "linear_memory": {
         "tnx_memory_inputs": [_c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p,
                               _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_float, _c_void_p, _c_int, _c_int,
-                              _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p],
+                              _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p],
         "tnx_memory_walk": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                             _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
         "tnx_memory_chunks": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                               _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_int, _c_void_p,
-                              _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int,
-                              _c_int, _c_void_p],
+                              _c_void_p, _c_void_p, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
         "tnx_gated_norm": [_c_void_p, _c_void_p, _c_ll, _c_void_p, _c_float, _c_int, _c_int, _c_void_p, _c_int, _c_void_p,
                            _c_ll, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
     },
@@ -1752,12 +1751,14 @@ class HipOps:
         _want(rate, "rates", torch.float32, (heads,))
         _want(dt_bias, "dt bias", torch.float32, (heads,))
         size, count, scaled, scale = unit if unit is not None else (0, 0, 0, 1.0)
-        u = torch.empty(t, channels, dtype=torch.float32, device=proj.device)
+        # rows a power of two of bytes apart would put a head's queries (or keys) of all tokens onto the same few memory
+        # channels: 256 bytes more between them
+        u = torch.empty(t, channels + 64, dtype=torch.float32, device=proj.device)[:, :channels]
         gates = torch.empty(2, t, heads, dtype=torch.float32, device=proj.device)
         self._call("linear_memory", "tnx_memory_inputs", _ptr(proj), proj.shape[1], int(conv_at), channels,
                    _ptr(self._taps_first(weight)), _ptr(bias), _ptr(state) if taps > 1 else None, taps, _ptr(ctx.positions),
                    _ptr(ctx.token_request), _ptr(ctx.run_start), _ptr(ctx.slots), int(size), int(count), int(scaled),
-                   float(scale), _ptr(u), heads, int(dt_at), -1 if write_at is None else int(write_at), _ptr(rate),
+                   float(scale), _ptr(u), channels + 64, heads, int(dt_at), -1 if write_at is None else int(write_at), _ptr(rate),
                    _ptr(dt_bias), _ptr(gates[0]), _ptr(gates[1]), t, ctx.num_requests, _stream(),
                    work=(f"{t}x{channels}", t * channels * 8.0 + ctx.num_requests * (taps - 1) * channels * 8.0, 0.0))
         return u, gates[0], gates[1]
@@ -1765,9 +1766,9 @@ class HipOps:
     def linear_memory(self, u, q_at, k_at, v_at, heads, groups, n, v, log_decay, write, ctx, memory, delta):
         """See `ReferenceOps.linear_memory`."""
         t = ctx.num_tokens
-        _want(u, "queries, keys and values", torch.float32)
-        if u.dim() != 2 or u.shape[0] != t:
-            raise ValueError(f"queries, keys and values must be [{t}, columns], got {tuple(u.shape)}")
+        u_ld = self._rows_apart(u, "queries, keys and values", torch.float32, t, 2 * groups * n + heads * v)
+        if min(q_at, k_at, v_at) < 0 or max(q_at + groups * n, k_at + groups * n, v_at + heads * v) > u.shape[1]:
+            raise ValueError(f"queries, keys and values at columns {q_at}, {k_at}, {v_at} of {u.shape[1]}")
         _want(log_decay, "decays", torch.float32, (t, heads))
         _want(write, "write weights", torch.float32, (t, heads))
         _want(memory, "memory", torch.float32, (memory.shape[0], 2, heads, v, n))
@@ -1779,22 +1780,20 @@ class HipOps:
         longest = 0
         if by_chunks is not None and by_chunks.numel() and self.memory_by_chunks:
             # the long runs, chunk by chunk
-            longest = MEMORY_LONG - 1
+            longest = ctx.plan_host["memory_walk_most"]
             chunk_run, first = ctx.plan["memory_chunk_run"], ctx.plan["memory_long_first"]
             chunks = chunk_run.numel()
-            ahead, behind, w, u0, pairs = (
-                torch.empty(size, dtype=torch.float32, device=u.device)
-                for size in (t * heads, t * heads, t * heads * n if delta else 0, t * heads * v if delta else 0,
-                             chunks * heads * MEMORY_CHUNK * MEMORY_CHUNK))
-            self._call("linear_memory", "tnx_memory_chunks", _ptr(u), u.shape[1], int(q_at), int(k_at), int(v_at),
+            nb, vb = next(x for x in (2, 4, 8, 16) if n <= 16 * x), -(-v // 16)
+            size = chunks * (2 * groups * 1024 * nb + heads * (3 * 64 + 4096) + (heads * 1024 * (nb + vb) if delta else 0))
+            room = torch.empty(size, dtype=torch.float32, device=u.device)
+            self._call("linear_memory", "tnx_memory_chunks", _ptr(u), u_ld, int(q_at), int(k_at), int(v_at),
                        _ptr(log_decay), _ptr(write), _ptr(ctx.run_start), _ptr(ctx.cached_lens), _ptr(ctx.slots),
                        _ptr(chunk_run), _ptr(ctx.plan["memory_chunk_begin"]), chunks, MEMORY_CHUNK, _ptr(by_chunks), _ptr(first),
-                       by_chunks.numel(), _ptr(memory), _ptr(out), _ptr(ahead), _ptr(behind), _ptr(pairs),
-                       _ptr(w) if delta else None, _ptr(u0) if delta else None, heads, groups, n, v, int(bool(delta)), _stream(),
+                       by_chunks.numel(), _ptr(memory), _ptr(out), _ptr(room), size, heads, groups, n, v, int(bool(delta)), _stream(),
                        work=work)
             if by_chunks.numel() == ctx.num_requests:
                 return out
-        self._call("linear_memory", "tnx_memory_walk", _ptr(u), u.shape[1], int(q_at), int(k_at), int(v_at), _ptr(log_decay),
+        self._call("linear_memory", "tnx_memory_walk", _ptr(u), u_ld, int(q_at), int(k_at), int(v_at), _ptr(log_decay),
                    _ptr(write), _ptr(ctx.run_start), _ptr(ctx.cached_lens), _ptr(ctx.slots), _ptr(memory), _ptr(out), t,
                    ctx.num_requests, heads, groups, n, v, int(bool(delta)), longest, _stream(), work=None if longest else work)
         return out
@@ -1823,8 +1822,8 @@ class HipOps:
 
     def route(self, z, top, score="sigmoid", renormalize=False, correction=None, scale=1.0, groups=None):
         """See `ReferenceOps.route`."""
-        _want(z, "router logits", torch.float32)
         t, experts = z.shape
+        ld = self._rows_apart(z, "router logits", torch.float32, t, experts)
         if score not in ("sigmoid", "softmax"):
             raise ValueError(f"unknown router score {score!r}")
         chosen = torch.empty(t, top, dtype=torch.int32, device=z.device)
@@ -1832,7 +1831,7 @@ class HipOps:
         if correction is not None:
             _want(correction, "the choice's correction", torch.float32, (experts,))
         count, keep = groups if groups is not None else (1, 1)
-        self._call("experts", "tnx_route", _ptr(z), t, experts, top, int(score == "softmax"), int(bool(renormalize)),
+        self._call("experts", "tnx_route", _ptr(z), ld, t, experts, top, int(score == "softmax"), int(bool(renormalize)),
                    _ptr(chosen), _ptr(weights), _ptr(correction), float(scale), int(count), int(keep), _stream())
         return chosen, weights
 

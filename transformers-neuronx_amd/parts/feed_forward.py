@@ -193,7 +193,11 @@ class ExpertMixture(FeedForward):
         # an expert's gate rows, then its up rows: `[experts, 2 inner, width]`; the down matrices `[experts, width, inner]`
         self.w_gate_up = torch.stack([torch.cat([tensors[f"{p}{g}{s}"], tensors[f"{p}{u}{s}"]], dim=0) for p in each]).contiguous()
         self.w_down = torch.stack([tensors[f"{p}{d}{s}"] for p in each]).contiguous()
-        self.w_router = ops.prepare_weight(tensors[f"{prefix}{self.router_name}{s}"])
+        # with experts that have no tensors the router's rows are rarely a multiple of eight: zero rows behind them let the
+        # product of many rows go to the vendor library all the same
+        router = tensors[f"{prefix}{self.router_name}{s}"]
+        fill = -self.routed % 8 if self.identity else 0
+        self.w_router = ops.prepare_weight(torch.nn.functional.pad(router, (0, 0, 0, fill)).contiguous() if fill else router)
         self.correction = tensors[f"{prefix}{self.correction_name}"] if self.correction_name else None
         if self.shared_inner:
             p = prefix + self.shared_name
@@ -205,7 +209,7 @@ class ExpertMixture(FeedForward):
 
     def forward(self, h, ctx, residual):
         ops = self.ops
-        z = ops.linear(h, self.w_router, None, out_f32=True, f32_by_library=True)
+        z = ops.linear(h, self.w_router, None, out_f32=True, f32_by_library=True)[:, :self.routed]
         more = {}
         if self.correction is not None or self.route_scale != 1.0:
             more = dict(correction=self.correction, scale=self.route_scale)
