@@ -64,7 +64,7 @@ def short_conv(x, weight, bias=None):
 
 def delta_rule(q, k, v, log_decay, beta):
     """q, k `[T, H, n]`, v `[T, H, v]`, log_decay and beta `[T, H]`: with S `[n, v]` a head, from zero,
-    S <- e^log_decay S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q."""
+    S_t = S' + k_t w_t^T where S' = e^log_decay_t S_(t-1) and w_t = beta_t (v_t - S'^T k_t); o_t = S_t^T q_t."""
     t, heads, n = q.shape
     s = torch.zeros(heads, n, v.shape[2], dtype=q.dtype)
     out = torch.zeros_like(v)
@@ -171,7 +171,7 @@ def parallel(m, w, p, h, eps):
 # ---------------------------------------------------------------- feed-forward
 
 def dense(mlp, w, p, h):
-    """g = min(W_gate h, limit), u = clamp(W_up h, +-limit): W_down (g sigmoid(1.702 g) (u + 1))."""
+    """With a = W_gate h kept below `limit` and b = W_up h kept inside +-`limit`: W_down (a sigmoid(1.702 a) (b + 1))."""
     g = torch.clamp(h @ w[p + "gate"].T, max=mlp["limit"])
     u = torch.clamp(h @ w[p + "up"].T, min=-mlp["limit"], max=mlp["limit"])
     return (g * sigmoid(1.702 * g) * (u + 1.0)) @ w[p + "down"].T

@@ -1,5 +1,5 @@
 // Linear memories: a matrix S [n, v] a head that is carried from token to token,
-//     S <- e^g S,   S <- S + k w^T,   o = S^T q,      w = write * val,  or with DELTA  w = write * (val - S^T k),
+//     S_t = S' + k w^T,  S' = e^g S_(t-1),  o = S_t^T q,    w = write * val,  or with DELTA  w = write * (val - S'^T k),
 // and what stands before and after them in a mixer:
 //   memory_inputs   a short causal convolution over time with silu, unit vectors a head, decays and write weights
 //   memory_walk     the recurrence token by token (decoded tokens, short runs)
@@ -376,6 +376,16 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
   }
   if (!col_ok) return;
   float* Sw = a.memory + ((head_at + (size_t)to * a.heads) * a.v + col) * a.n;
+  if (ALIGNED && NR % 4 == 0) {
+#pragma unroll
+    for (int j = 0; j < NR; j += 4) {
+      f32x4 out;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) out[e] = S[j + (NR % 4 == 0 ? e : 0)];
+      if (grp * NR + j < a.n) *(f32x4*)(Sw + grp * NR + j) = out;
+    }
+    return;
+  }
 #pragma unroll
   for (int j = 0; j < NR; ++j)
     if (grp * NR + j < a.n) Sw[grp * NR + j] = S[j];

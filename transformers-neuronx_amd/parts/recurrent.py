@@ -163,7 +163,7 @@ class GatedLinearRecurrence(_BesideAnother, Mixer):
 class _LinearMemory(Mixer):
     """What the mixers around a linear memory share: a matrix S `[n, v]` a head that is carried from token to token,
 
-        S <- e^g S,   S <- S + k w^T,   o = S^T q,        w = write * val   or   w = write * (val - S^T k)  (`delta`),
+        S_t = S' + k w^T,  S' = e^g S_(t-1),  o = S_t^T q,      w = write * val   or   w = write * (val - S'^T k)  (`delta`),
 
     whose queries, keys and values come out of a short causal convolution over time (`taps` a channel) and silu. Queries
     and keys have `groups` heads, head h takes number floor(h / (heads / groups)). One product makes everything that is
@@ -216,7 +216,7 @@ class GatedDeltaRule(_LinearMemory):
     each through a convolution over time and silu, q and k made unit vectors a head and q times n^(-1/2):
 
         beta = sigmoid(W_b h),   g = -exp(A_log) softplus(W_a h + dt_bias)                     (a number a head each)
-        S <- e^g S;   u = beta (val - S^T k);   S <- S + k u^T;   o = S^T q
+        S_t = S' + k_t w_t^T,   S' = e^g S_(t-1),   w_t = beta_t (val_t - S'^T k_t),   o_t = S_t^T q_t
 
     A head's o at unit root mean square, times `norm` (v elements, the same for all heads), times silu(W_g h);
     W_o on the heads side by side."""
