@@ -42,7 +42,8 @@ _ARCHITECTURES: Dict[str, Architecture] = {}
 # by commas, that are importable from where it runs.
 ARCHITECTURE_PACKAGES: List[str] = ["transformers_neuronx_amd.opt", "transformers_neuronx_amd.ratesun",
                                     "transformers_neuronx_amd.sunatar", "transformers_neuronx_amd.tadolix",
-                                    "transformers_neuronx_amd.zotunex", "transformers_neuronx_amd.gubulorn"]
+                                    "transformers_neuronx_amd.zotunex", "transformers_neuronx_amd.gubulorn",
+                                    "transformers_neuronx_amd.zudusun"]
 PACKAGES_VARIABLE = "TNX_ARCHITECTURE_PACKAGES"
 
 

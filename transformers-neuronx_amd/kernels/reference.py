@@ -737,11 +737,31 @@ class ReferenceOps:
         write = dt if write_at is None else torch.sigmoid(proj[:, write_at:write_at + heads].float())
         return u, dt * rate.float(), write
 
+    def channel_decays(self, low, weight, bias, tau):
+        """The decay's logarithm for every key channel: log_sigmoid(low weight^T + bias) / tau, `low` float32 `[T, rank]`
+        (rows may lie apart), `weight` `[channels, rank]`, `bias` `[channels]`; float32 `[T, channels]`, sums float32."""
+        z = low.float() @ weight.float().t() + bias.float()
+        return torch.nn.functional.logsigmoid(z) / float(tau)
+
+    def turn_heads(self, x, at, heads, n, freqs, interleaved, ctx):
+        """In place: the first `2 len(freqs)` elements of the `heads` heads of `n` that begin at column `at` of `x` (float32
+        `[T, columns]`) turned by position * freqs, in neighbouring pairs (`interleaved`) or pairs (i, i + len(freqs))."""
+        part = x[:, at:at + heads * n].reshape(x.shape[0], heads, n)
+        angle = ctx.positions.float()[:, None, None] * freqs.float()[None, None, :]
+        cos, sin, half = torch.cos(angle), torch.sin(angle), freqs.numel()
+        a, b = (part[..., 0:2 * half:2], part[..., 1:2 * half:2]) if interleaved else (part[..., :half], part[..., half:2 * half])
+        u, v = a * cos - b * sin, b * cos + a * sin
+        turned = torch.stack([u, v], dim=-1).flatten(-2) if interleaved else torch.cat([u, v], dim=-1)
+        x[:, at:at + heads * n] = torch.cat([turned, part[..., 2 * half:]], dim=-1).reshape(x.shape[0], heads * n)
+        return x
+
     def linear_memory(self, u, q_at, k_at, v_at, heads, groups, n, v, log_decay, write, ctx, memory, delta):
         """A matrix S `[n, v]` a head that is carried from token to token: S <- e^log_decay S, S <- S + k w^T with
         w = write * val, or, with `delta`, w = write * (val - S^T k), and o = S^T q. Queries, keys and values are
         columns of `u` float32 `[T, columns]` from `q_at`, `k_at`, `v_at` on; queries and keys come in `groups` heads,
-        head h takes number h // (heads / groups). `memory` float32 `[slots, 2, heads, v, n]` (a column's rows side by
+        head h takes number h // (heads / groups). `log_decay` float32 `[T, heads]`, `[heads]` (the same for every token)
+        or, with groups = heads and without `delta`, `[T, heads * n]`: a decay for every row of S. `write` float32
+        `[T, heads]` or None: 1. `memory` float32 `[slots, 2, heads, v, n]` (a column's rows side by
         side): the token at position p reads place (p - 1) & 1 (zeros at p = 0) and writes place p & 1. Returns
         float32 `[T, heads * v]`."""
         t = u.shape[0]
@@ -749,29 +769,34 @@ class ReferenceOps:
         q = u[:, q_at:q_at + groups * n].reshape(t, groups, n)[:, share]
         k = u[:, k_at:k_at + groups * n].reshape(t, groups, n)[:, share]
         val = u[:, v_at:v_at + heads * v].reshape(t, heads, v)
-        decay = torch.exp(log_decay)
+        if log_decay.dim() == 1:
+            log_decay = log_decay[None, :].expand(t, heads)
+        decay = torch.exp(log_decay).reshape(t, heads, 1, -1)          # [.., 1, n] or [.., 1, 1]
         out = torch.empty(t, heads, v, dtype=torch.float32, device=u.device)
         start = 0
         for r in range(ctx.num_requests):
             count, slot, have = int(ctx.run_lens_host[r]), int(ctx.slots_host[r]), int(ctx.cached_lens_host[r])
             s = memory[slot, (have - 1) & 1].clone() if have > 0 else torch.zeros_like(memory[slot, 0])       # [H, v, n]
             for i in range(start, start + count):
-                s = s * decay[i][:, None, None]
+                s = s * decay[i]
                 w = val[i]
                 if delta:
                     w = w - torch.einsum("hvn,hn->hv", s, k[i])
-                s = s + (write[i][:, None] * w)[:, :, None] * k[i][:, None, :]
+                if write is not None:
+                    w = write[i][:, None] * w
+                s = s + w[:, :, None] * k[i][:, None, :]
                 out[i] = torch.einsum("hvn,hn->hv", s, q[i])
             if count:
                 memory[slot, (have + count - 1) & 1] = s
             start += count
         return out.reshape(t, heads * v)
 
-    def gated_norm(self, o, gate, weight, eps, parts, gate_first, skip=None):
+    def gated_norm(self, o, gate, weight, eps, parts, gate_first, skip=None, out=None, out_scale=1.0):
         """What follows a memory up to the output product: rows `o` float32 `[T, width]` in `parts` equal parts, each
-        scaled to unit root mean square, times `weight` `[width]`; times silu(`gate`) (float32 `[T, width]`, rows may lie
-        apart) after the norm, or before it with `gate_first`. `skip` = (factors `[heads]`, x float32 `[T, width]`, rows
-        may lie apart): o + factor x first, head by head. In the compute dtype."""
+        scaled to unit root mean square, times `weight` `[width]` (None: 1); times silu(`gate`) (float32 `[T, width]`, rows
+        may lie apart) after the norm, or before it with `gate_first`. `skip` = (factors `[heads]`, x float32 `[T, width]`,
+        rows may lie apart): o + factor x first, head by head. The result times `out_scale`, in the compute dtype (into
+        `out`, whose rows may lie apart, or a new tensor)."""
         t, width = o.shape
         o = o.float()
         if skip is not None:
@@ -781,8 +806,14 @@ class ReferenceOps:
         if gate_first:
             o = o * g
         p = o.reshape(t, parts, width // parts)
-        o = (p * torch.rsqrt((p * p).mean(-1, keepdim=True) + eps)).reshape(t, width) * weight.float()
-        return (o if gate_first else o * g).to(self.dtype)
+        o = (p * torch.rsqrt((p * p).mean(-1, keepdim=True) + eps)).reshape(t, width)
+        if weight is not None:
+            o = o * weight.float()
+        o = (o if gate_first else o * g) * out_scale
+        if out is None:
+            return o.to(self.dtype)
+        out.copy_(o)
+        return out
 
     # ---------------------------------------------------------------- experts
 
@@ -829,11 +860,20 @@ class ReferenceOps:
             g, u = g * row_weights.float()[:, None], u * row_weights.float()[:, None]
         return self._gated(g, u, activation, limit).to(self.dtype)
 
+    def row_activation(self, x, activation, row_gate=None):
+        """`act(x)` from float32 `[T, F]`, times sigmoid(`row_gate`) of its row (float32 `[T, 1]`, rows may lie apart), in
+        the compute dtype."""
+        y = self.activation(x.float(), activation)
+        if row_gate is not None:
+            y = y * torch.sigmoid(row_gate.float())
+        return y.to(self.dtype)
+
     def expert_mixture(self, h, chosen, weights, w_gate_up, w_down, activation, weight_on, residual=None, may_wait=False,
                        limit=None, identity=0):
         """float32 `residual + sum_c expert_(chosen[t, c])(h[t])` with the weights `weights[t, c]` on the expert's
         input (`weight_on="input"`: act(w g) * (w u), the float32 sums of the first product times w) or on its
-        output. `w_gate_up` `[E, 2 F, D]` (gate rows, then up rows), `w_down` `[E, D, F]`. A number of E or more in
+        output. `w_gate_up` `[E, 2 F, D]` (gate rows, then up rows), `w_down` `[E, D, F]`. `w_gate_up` `[E, F, D]`:
+        experts without a gate, act(w_up h) (activation "relu2", weight_on "output"). A number of E or more in
         `chosen` is an expert without tensors, whose output is its input (weight_on "output")."""
         t, top = chosen.shape
         f = w_down.shape[2]
@@ -849,7 +889,8 @@ class ReferenceOps:
             w = weights[:, c].float()[:, None]
             if weight_on == "input":
                 gu = gu * w
-            inner = self._gated(gu[:, :f], gu[:, f:], activation, limit).to(self.dtype)
+            inner = (self._gated(gu[:, :f], gu[:, f:], activation, limit) if gu.shape[1] == 2 * f
+                     else self.activation(gu, activation)).to(self.dtype)
             y = torch.einsum("tf,tdf->td", inner.to(w_down.dtype).float(), w_down[e].float())
             y = torch.where(same[:, None], h.float(), y)
             out = out + (y if weight_on == "input" else y * w)

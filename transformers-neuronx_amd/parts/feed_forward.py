@@ -111,7 +111,7 @@ class NoFeedForward(FeedForward):
 
 @register_feed_forward("mixture")
 class ExpertMixture(FeedForward):
-    """A mixture of gated experts, of which a token takes `top`, and optionally one more that every token takes.
+    """A mixture of experts, of which a token takes `top`, and optionally one more that every token takes.
 
     Router: z = W_r h in float32, scores s = sigmoid(z) (`score="sigmoid"`) or softmax(z) (`"softmax"`); a token's
     experts are the `top` with the largest scores (the lower number where two are equal), their weights the
@@ -128,7 +128,12 @@ class ExpertMixture(FeedForward):
     `identity`: so many router outputs behind the experts' stand for experts that have no tensors: their output is
     their input. They are scored, corrected, grouped and chosen like the others. `groups` = {count, keep}: experts and
     identity experts together form `count` equal groups of neighbours, a group's score is the largest score (with
-    the correction) in it, and only experts of the `keep` best groups can be chosen."""
+    the correction) in it, and only experts of the `keep` best groups can be chosen.
+
+    `gated=False` with `activation="relu2"`: experts (and the shared one) without a gate, W_down (act(W_up x)), the weight
+    on the output; `names` are then two. `router_bias_name`: a bias of the router's logits. `shared_gate_name`: a matrix of
+    one row w_s under the shared expert's prefix, whose output is multiplied by sigmoid(w_s h); its row rides in the
+    router's product, and the factor enters where the shared expert's inner values are rounded."""
 
     recordable = True
 
@@ -136,9 +141,12 @@ class ExpertMixture(FeedForward):
                  shared_inner: int = 0, shared_name: str = "shared.", score: str = "sigmoid", renormalize: bool = False,
                  weight_on: str = "output", activation: str = "silu", weight_suffix: str = "",
                  correction_name: str = None, route_scale: float = 1.0, limit: float = None, shared_limit: float = None,
-                 identity: int = 0, groups=None):
+                 identity: int = 0, groups=None, gated: bool = True, router_bias_name: str = None,
+                 shared_gate_name: str = None):
         """`expert_name`: a format string that takes the expert's number ("e{}."); `names`: the names of an
-        expert's gate, up and down matrices."""
+        expert's gate, up and down matrices (not `gated`: of its up and down matrices)."""
+        self.gated, self.router_bias_name = bool(gated), router_bias_name
+        self.shared_gate_name = shared_gate_name if shared_inner else None
         self.routed, self.identity = experts + identity, identity
         self.groups = (int(groups["count"]), int(groups["keep"])) if groups else None
         if not 1 <= top <= self.routed or experts < 1 or identity < 0:
@@ -150,13 +158,19 @@ class ExpertMixture(FeedForward):
         if identity and (weight_on != "output" or renormalize):
             raise ValueError("mixture: experts without tensors take their weight on the output, not renormalized")
         if score not in ("sigmoid", "softmax") or weight_on not in ("input", "output") \
-                or activation not in ("silu", "gelu_new", "clamped_swiglu"):
+                or activation not in (("silu", "gelu_new", "clamped_swiglu") if gated else ("relu2",)):
             raise ValueError(f"mixture: score {score!r}, weight_on {weight_on!r}, activation {activation!r}")
         if activation == "clamped_swiglu":
             if limit is None or not float(limit) > 0 or (shared_inner and not float(shared_limit or 0) > 0):
                 raise ValueError("mixture: activation 'clamped_swiglu' needs a positive `limit` (and `shared_limit`)")
             if weight_on != "output":
                 raise ValueError("mixture: a clamped expert takes its weight on the output")
+        if not gated and weight_on != "output":
+            raise ValueError("mixture: experts without a gate take their weight on the output")
+        if gated and self.shared_gate_name:
+            raise ValueError("mixture: a shared expert with a gate number a token is one without a gate matrix")
+        if len(names) != (3 if gated else 2):
+            raise ValueError("mixture: names of an expert's gate, up and down matrices (without a gate: up and down)")
         if correction_name and renormalize:
             raise ValueError("mixture: a correction of the choice goes with scores that are not renormalized")
         self.correction_name, self.route_scale = correction_name, float(route_scale)
@@ -168,48 +182,64 @@ class ExpertMixture(FeedForward):
         self.score, self.renormalize, self.weight_on, self.activation = score, bool(renormalize), weight_on, activation
 
     def _expert_decls(self, prefix: str, inner: int) -> List[ParamDecl]:
-        g, u, d = self.names
+        *ins, d = self.names
         s = self.weight_suffix
-        return [ParamDecl(f"{prefix}{g}{s}", (inner, self.width)), ParamDecl(f"{prefix}{u}{s}", (inner, self.width)),
-                ParamDecl(f"{prefix}{d}{s}", (self.width, inner))]
+        return [ParamDecl(f"{prefix}{n}{s}", (inner, self.width)) for n in ins] + [ParamDecl(f"{prefix}{d}{s}", (self.width, inner))]
 
     def param_decls(self, prefix: str) -> List[ParamDecl]:
         d = []
         for e in range(self.experts):
             d += self._expert_decls(prefix + self.expert_name.format(e), self.inner)
         d.append(ParamDecl(f"{prefix}{self.router_name}{self.weight_suffix}", (self.routed, self.width)))
+        if self.router_bias_name:
+            d.append(ParamDecl(f"{prefix}{self.router_bias_name}", (self.routed,), "vector"))
         if self.correction_name:
             d.append(ParamDecl(f"{prefix}{self.correction_name}", (self.routed,), "vector"))
         if self.shared_inner:
             d += self._expert_decls(prefix + self.shared_name, self.shared_inner)
+        if self.shared_gate_name:
+            d.append(ParamDecl(f"{prefix}{self.shared_name}{self.shared_gate_name}{self.weight_suffix}", (1, self.width)))
         return d
 
     def load(self, tensors: Dict, prefix: str, ops, dtype) -> None:
         import torch
         super().load(tensors, prefix, ops, dtype)
-        g, u, d = self.names
+        *ins, d = self.names
         s = self.weight_suffix
         each = [prefix + self.expert_name.format(e) for e in range(self.experts)]
         # an expert's gate rows, then its up rows: `[experts, 2 inner, width]`; the down matrices `[experts, width, inner]`
-        self.w_gate_up = torch.stack([torch.cat([tensors[f"{p}{g}{s}"], tensors[f"{p}{u}{s}"]], dim=0) for p in each]).contiguous()
+        self.w_gate_up = torch.stack([torch.cat([tensors[f"{p}{n}{s}"] for n in ins], dim=0) for p in each]).contiguous()
         self.w_down = torch.stack([tensors[f"{p}{d}{s}"] for p in each]).contiguous()
-        # with experts that have no tensors the router's rows are rarely a multiple of eight: zero rows behind them let the
-        # product of many rows go to the vendor library all the same
+        # one product for the router's rows and, behind them, the row of the shared expert's gate. Such rows (and those of a
+        # router with experts that have no tensors) are rarely a multiple of eight: zero rows behind them let the product
+        # of many rows go to the vendor library all the same
         router = tensors[f"{prefix}{self.router_name}{s}"]
-        fill = -self.routed % 8 if self.identity else 0
-        self.w_router = ops.prepare_weight(torch.nn.functional.pad(router, (0, 0, 0, fill)).contiguous() if fill else router)
+        rows = self.routed
+        if self.shared_gate_name:
+            router = torch.cat([router, tensors[f"{prefix}{self.shared_name}{self.shared_gate_name}{s}"].to(router.dtype)], dim=0)
+            rows += 1
+        fill = (-rows % 16 if self.shared_gate_name else -rows % 8) if self.identity or self.shared_gate_name else 0
+        router = torch.nn.functional.pad(router, (0, 0, 0, fill)).contiguous() if fill else router.contiguous()
+        self.w_router = ops.prepare_weight(router)
+        self.b_router = None
+        if self.router_bias_name:
+            bias = tensors[f"{prefix}{self.router_bias_name}"]
+            self.b_router = torch.nn.functional.pad(bias, (0, router.shape[0] - bias.numel())).contiguous()
         self.correction = tensors[f"{prefix}{self.correction_name}"] if self.correction_name else None
         if self.shared_inner:
             p = prefix + self.shared_name
-            self.w_shared_in = ops.prepare_weight(torch.cat([tensors[f"{p}{g}{s}"], tensors[f"{p}{u}{s}"]], dim=0).contiguous())
+            self.w_shared_in = ops.prepare_weight(torch.cat([tensors[f"{p}{n}{s}"] for n in ins], dim=0).contiguous())
             self.w_shared_down = ops.prepare_weight(tensors[f"{p}{d}{s}"])
 
     def flops_per_token(self, keys: float = 0.0) -> float:
-        return 2.0 * self.width * (self.routed + 3 * self.top * self.inner * self.experts / self.routed + 3 * self.shared_inner)
+        each = len(self.names)
+        return 2.0 * self.width * (self.routed + each * self.top * self.inner * self.experts / self.routed
+                                   + each * self.shared_inner + (1 if self.shared_gate_name else 0))
 
     def forward(self, h, ctx, residual):
         ops = self.ops
-        z = ops.linear(h, self.w_router, None, out_f32=True, f32_by_library=True)[:, :self.routed]
+        rows = ops.linear(h, self.w_router, self.b_router, out_f32=True, f32_by_library=True)
+        z = rows[:, :self.routed]
         more = {}
         if self.correction is not None or self.route_scale != 1.0:
             more = dict(correction=self.correction, scale=self.route_scale)
@@ -225,6 +255,10 @@ class ExpertMixture(FeedForward):
         if not self.shared_inner:
             return x
         limit = dict(limit=self.shared_limit) if self.shared_limit is not None else {}
-        inner = ops.gated_activation(ops.linear(h, self.w_shared_in, None, out_f32=True, f32_by_library=True),
-                                     self.activation, **limit)
+        up = ops.linear(h, self.w_shared_in, None, out_f32=True, f32_by_library=True)
+        if self.gated:
+            inner = ops.gated_activation(up, self.activation, **limit)
+        else:
+            inner = ops.row_activation(up, self.activation,
+                                       rows[:, self.routed:self.routed + 1] if self.shared_gate_name else None)
         return ops.linear(inner, self.w_shared_down, None, residual=x, out_f32=True)

@@ -58,7 +58,8 @@ class Attention(Mixer):
                  qk_norm=None, value_mix=None, weight_suffix: str = ".weight", bias_suffix: str = ".bias",
                  softcap: Optional[float] = None, distance_bias=None, chunk: Optional[int] = None,
                  out_gate: Optional[str] = None, out_gate_per_head: bool = False, values_from_keys: bool = False,
-                 head_scale: Optional[str] = None, temperature=None, sink: Optional[str] = None):
+                 head_scale: Optional[str] = None, temperature=None, sink: Optional[str] = None,
+                 sink_score: Optional[float] = None, float32_route: bool = False):
         """`names`: the checkpoint's names of the query, key, value and output projections, relative to
         the mixer's prefix (the architecture's spec gives them); a matrix's name adds `weight_suffix`, a bias's
         `bias_suffix`. `out_bias`: whether the output projection has a bias (as the others, if not said).
@@ -93,7 +94,10 @@ class Attention(Mixer):
         its keys as projected, before their norm and turn. `head_scale`: the name of a tensor of one number a query
         head that multiplies the head's scores (beside `scale`). `temperature` = {coef, every}: the queries of the token
         at position p are multiplied by 1 + coef ln(floor((p + 1) / every) + 1). `sink`: the name of a tensor of one
-        number a query head; the softmax's denominator also holds exp(sink), once, a term that stands for no token. With `shared` in `qk_norm` (which implies
+        number a query head; the softmax's denominator also holds exp(sink), once, a term that stands for no token;
+        `sink_score`: the same with one number for all heads in the place of a tensor (0: a one in the denominator).
+        `float32_route`: a mixer that could do without takes the float32 route all the same (one that runs beside another
+        must). With `shared` in `qk_norm` (which implies
         `per_head`) the two weight tensors hold one head's `head_size` elements, the same for every head."""
         self.width, self.num_heads, self.head_size = width, num_heads, head_size
         self.num_kv_heads = num_kv_heads if num_kv_heads is not None else num_heads
@@ -112,7 +116,9 @@ class Attention(Mixer):
         self.temperature = (float(temperature["coef"]), int(temperature["every"])) if temperature else None
         if self.temperature and self.temperature[1] < 1:
             raise ValueError(f"a temperature that grows every {self.temperature[1]} tokens")
-        self.sink = sink
+        self.sink, self.sink_score = sink, None if sink_score is None else float(sink_score)
+        if sink and sink_score is not None:
+            raise ValueError("an attention mixer's sink is a tensor or a number, not both")
         if self.qk_norm and self.qk_norm.get("shared"):
             self.qk_norm["per_head"] = True
         if self.values_from_keys and self.value_size != head_size:
@@ -121,9 +127,9 @@ class Attention(Mixer):
             raise ValueError("values that are the keys are not blended")
         if self.chunk is not None and window is not None:
             raise ValueError("an attention mixer masks by a window or by chunks, not both")
-        self.scored = bool(self.softcap or self.distance_bias or self.chunk or out_gate or sink)
+        self.scored = bool(self.softcap or self.distance_bias or self.chunk or out_gate or sink or sink_score is not None)
         self.prepared = bool(self.qk_norm or self.value_mix or halves or self.value_size != head_size or self.scored
-                             or self.values_from_keys or head_scale or self.temperature)
+                             or self.values_from_keys or head_scale or self.temperature or float32_route)
         self.defer_out = False      # set by a mixer that runs this one beside another and owns the output product
         if self.prepared:
             if not own_kv:
@@ -225,6 +231,8 @@ class Attention(Mixer):
                 self.k_norm = self.k_norm.repeat(self.num_kv_heads).contiguous()
         self.head_scales = tensors[f"{prefix}{self.head_scale}"] if self.head_scale else None
         self.sinks = tensors[f"{prefix}{self.sink}"] if self.sink else None
+        if self.sink_score is not None:
+            self.sinks = torch.full((self.num_heads,), self.sink_score, dtype=torch.float32, device=w_out.device)
         if self.value_mix and not self.value_mix["first"]:
             self.mix_weight = tensors[f"{prefix}{self.value_mix['name']}"].reshape(1)
 

@@ -9,7 +9,7 @@ from typing import Dict, List, Optional
 
 import torch
 
-from .base import MIXERS, CacheNeed, Mixer, register_mixer
+from .base import MIXERS, POSITIONS, CacheNeed, Mixer, register_mixer
 from .spec import ParamDecl, PartSpec
 
 
@@ -312,6 +312,162 @@ class StateSpace(_LinearMemory):
         o = ops.linear_memory(u, i + gn, i, 0, self.heads, self.groups, self.n, self.v, decay, write, ctx, state["memory"],
                               False)
         return ops.gated_norm(o, proj[:, :i], self.norm_weight, self.eps, self.norm_groups, True, skip=(self.skip, u[:, :i]))
+
+
+class _PlainMemory(_BesideAnother, Mixer):
+    """What the mixers around a linear memory without convolutions share: per head a matrix S `[n, v]` that is carried
+    from token to token,
+
+        S_t = diag(e^(g_t)) S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t,   g_t a number a head or one a row of S,
+
+    read straight off the float32 rows of one input product (queries, keys, values, gates, and what a mixer adds); each
+    head's o at unit root mean square, times a weight or not, times silu(W_g h); W_o. The factor n^(-1/2) that the
+    designs put on queries or keys scales every o of a head alike, and the norm takes it off again up to eps: it is not
+    multiplied in anywhere, the norm's eps is n times as large instead. Everything between the two products is float32."""
+
+    recordable = True
+
+    def _sizes(self, width, heads, head_size, value_size, eps):
+        if head_size > 256:
+            raise ValueError(f"a linear memory's queries and keys have up to 256 elements a head, got {head_size}")
+        self.width, self.heads, self.n, self.v, self.eps = width, heads, head_size, value_size, float(eps)
+        self.qk, self.inner = heads * head_size, heads * value_size
+
+    def cache_need(self) -> Optional[CacheNeed]:
+        # (a column's rows side by side: what a lane of the kernel holds are neighbours in memory)
+        return CacheNeed("state", state_shapes=(("memory", (2, self.heads, self.v, self.n)),))
+
+    def step_planners(self):
+        from ..kernels.memory_plan import memory_plan
+        return {"memory": memory_plan}
+
+    def _load_in(self, tensors, names, ops):
+        """The rows of the input matrices one under the other, filled up with zero rows to a multiple of 16, and by 64
+        more where the product's rows would lie a power of two of bytes apart: the queries of all tokens of a prompt
+        would then share few memory channels."""
+        w = torch.cat([tensors[n] for n in names], dim=0)
+        rows = w.shape[0] + -w.shape[0] % 16
+        rows += 64 if rows % 1024 == 0 else 0
+        return ops.prepare_weight(torch.nn.functional.pad(w, (0, 0, 0, rows - w.shape[0])).contiguous())
+
+    def inner_width(self) -> int:
+        return self.inner
+
+    def _decays(self, proj, ctx):
+        """The decays' logarithms as `ops.linear_memory` takes them, after anything else that is done to `proj`."""
+        raise NotImplementedError
+
+    def inner_into(self, h, ctx, cache, out, scale: float):
+        ops, qk = self.ops, self.qk
+        proj = ops.linear(h, self.w_in, None, out_f32=True, f32_by_library=True)
+        decay = self._decays(proj, ctx)
+        at = 2 * qk + self.inner                                # the columns: q | k | v | gate | ...
+        o = ops.linear_memory(proj[:, :at], 0, qk, 2 * qk, self.heads, self.heads, self.n, self.v, decay, None, ctx,
+                              cache.state["memory"], False)
+        return ops.gated_norm(o, proj[:, at:at + self.inner], self.norm_weight, self.eps * self.n, self.heads, False,
+                              out=out, out_scale=scale)
+
+    def forward(self, h, ctx, cache, residual):
+        y = self.inner_into(h, ctx, cache, None, 1.0)
+        return self.ops.linear(y, self.w_out, None, residual=residual, out_f32=True, f32_by_library=residual is None)
+
+
+@register_mixer("gated_linear_attention")
+class GatedLinearAttention(_PlainMemory):
+    """Gated linear attention: queries W_q h n^(-1/2), keys W_k h and values W_v h of `heads` heads, and a decay for every
+    row of S, e^g = sigmoid(z)^(1/tau) with z = W_a2 (W_a1 h) + b. Each head's o is normed with a weight of v elements
+    that all heads share. The inner size of the two small matrices (`rank`) is the checkpoint's if not given."""
+
+    def __init__(self, width: int, heads: int, head_size: int, value_size: int, tau: float, eps: float, names,
+                 rank: Optional[int] = None, weight_suffix: str = "", bias_suffix: str = ".b"):
+        """`names`: the checkpoint's names of W_q, W_k, W_v, W_g, W_o, W_a1, W_a2 (its bias: with `bias_suffix`) and the
+        norm's weight."""
+        self._sizes(width, heads, head_size, value_size, eps)
+        self.tau, self.rank = float(tau), rank
+        if not self.tau > 0:
+            raise ValueError(f"gated linear attention: tau must be positive, got {tau}")
+        self.names, self.weight_suffix, self.bias_suffix = tuple(names), weight_suffix, bias_suffix
+        if len(self.names) != 8:
+            raise ValueError("names: W_q, W_k, W_v, W_g, W_o, W_a1, W_a2 and the norm, eight names")
+
+    def param_decls(self, prefix: str) -> List[ParamDecl]:
+        q, k, v, g, o, a1, a2, norm = (prefix + n for n in self.names)
+        ws = self.weight_suffix
+        return [ParamDecl(q + ws, (self.qk, self.width)), ParamDecl(k + ws, (self.qk, self.width)),
+                ParamDecl(v + ws, (self.inner, self.width)), ParamDecl(g + ws, (self.inner, self.width)),
+                ParamDecl(o + ws, (self.width, self.inner)), ParamDecl(a1 + ws, (self.rank, self.width)),
+                ParamDecl(a2 + ws, (self.qk, self.rank)), ParamDecl(a2 + self.bias_suffix, (self.qk,), "vector"),
+                ParamDecl(norm, (self.v,), "vector", "around_one")]
+
+    def load(self, tensors: Dict, prefix: str, ops, dtype) -> None:
+        super().load(tensors, prefix, ops, dtype)
+        q, k, v, g, o, a1, a2, norm = (prefix + n for n in self.names)
+        ws = self.weight_suffix
+        self.rank = tensors[a1 + ws].shape[0]
+        if tuple(tensors[a2 + ws].shape) != (self.qk, self.rank):
+            raise ValueError(f"{a2}{ws} is {tuple(tensors[a2 + ws].shape)}, behind a matrix of {self.rank} rows it must be "
+                             f"{(self.qk, self.rank)}")
+        self.w_in = self._load_in(tensors, [n + ws for n in (q, k, v, g, a1)], ops)
+        self.w_decay, self.b_decay = tensors[a2 + ws].contiguous(), tensors[a2 + self.bias_suffix]
+        self.norm_weight = tensors[norm].repeat(self.heads).contiguous()
+        self._keep_out(ops, tensors[o + ws])
+
+    def flops_per_token(self, keys: float = 0.0) -> float:
+        rank = self.rank or 0
+        return (2.0 * self.width * (2 * self.qk + 3 * self.inner + rank) + 2.0 * self.qk * rank
+                + 4.0 * self.heads * self.n * self.v)
+
+    def _decays(self, proj, ctx):
+        at = 2 * (self.qk + self.inner)
+        return self.ops.channel_decays(proj[:, at:at + self.rank], self.w_decay, self.b_decay, self.tau)
+
+
+@register_mixer("retention")
+class Retention(_PlainMemory):
+    """Retention: queries and keys turned by the position, keys times n^(-1/2), a decay a head that does not depend on the
+    token, no weight behind the norm."""
+
+    def __init__(self, width: int, heads: int, head_size: int, value_size: int, decay, eps: float, names, rotation=None,
+                 weight_suffix: str = ""):
+        """`decay`: a number a head, the factor itself. `names`: the checkpoint's names of W_q, W_k, W_v, W_g and W_o;
+        `rotation`: a position encoding that gives `frequencies()`, or None."""
+        self._sizes(width, heads, head_size, value_size, eps)
+        self.decay = tuple(float(x) for x in decay)
+        if len(self.decay) != heads or not all(0 < x <= 1 for x in self.decay):
+            raise ValueError(f"retention: {heads} decays in (0, 1], got {self.decay}")
+        self.rotation = POSITIONS.build(rotation) if rotation is not None else None
+        if self.rotation is not None and (not hasattr(self.rotation, "frequencies") or self.rotation.dims > head_size):
+            raise ValueError("retention turns its heads by a rotation that gives `frequencies()` for no more than their elements")
+        self.names, self.weight_suffix = tuple(names), weight_suffix
+        if len(self.names) != 5:
+            raise ValueError("names: W_q, W_k, W_v, W_g and W_o, five names")
+
+    def param_decls(self, prefix: str) -> List[ParamDecl]:
+        q, k, v, g, o = (prefix + n + self.weight_suffix for n in self.names)
+        return [ParamDecl(q, (self.qk, self.width)), ParamDecl(k, (self.qk, self.width)),
+                ParamDecl(v, (self.inner, self.width)), ParamDecl(g, (self.inner, self.width)),
+                ParamDecl(o, (self.width, self.inner))]
+
+    def load(self, tensors: Dict, prefix: str, ops, dtype) -> None:
+        super().load(tensors, prefix, ops, dtype)
+        q, k, v, g, o = (prefix + n + self.weight_suffix for n in self.names)
+        self.w_in = self._load_in(tensors, [q, k, v, g], ops)
+        # (logarithms made in float64 and rounded once)
+        self.log_decay = torch.log(torch.tensor(self.decay, dtype=torch.float64)).float().to(tensors[q].device)
+        self.freqs = None
+        if self.rotation is not None and self.rotation.dims > 0:
+            self.rotation.load(tensors, prefix + "rotation", ops, dtype)
+            self.freqs = self.rotation.frequencies()
+        self.norm_weight = None
+        self._keep_out(ops, tensors[o])
+
+    def flops_per_token(self, keys: float = 0.0) -> float:
+        return super().flops_per_token(keys) + 4.0 * self.heads * self.n * self.v
+
+    def _decays(self, proj, ctx):
+        if self.freqs is not None:
+            self.ops.turn_heads(proj, 0, 2 * self.heads, self.n, self.freqs, self.rotation.interleaved, ctx)
+        return self.log_decay
 
 
 class _SubCache:
