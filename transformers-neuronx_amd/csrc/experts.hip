@@ -1,7 +1,8 @@
-// A mixture of gated experts: the router's choice, the step's (token, choice) pairs put in the order of their
+// A mixture of experts: the router's choice, the step's (token, choice) pairs put in the order of their
 // experts, and the two products of every expert over its own pairs,
 //     inner = act(w g) * (w u)  with [g | u] = W_gate_up[e] h      (the weight w on the expert's input; on its
 //     y = W_down[e] inner                                           output it multiplies y instead)
+// or, for experts without a gate, inner = act(W_up[e] h),
 // summed over a token's choices onto the residual in float32. Nothing is read back by the host: the launches are
 // sized by the most tiles the pairs can make, and a block that finds no tile ends at once.
 #include "common.h"
@@ -158,25 +159,27 @@ __global__ void __launch_bounds__(1024) order_kernel(const int* __restrict__ cho
 
 // ---------------------------------------------------------------- an expert's product over its pairs
 // out[pair, j] = sum_k A[row(pair), k] W[e][j][k] for the pairs of expert e, a tile of 16 pairs by 64 columns a
-// block, float32 sums from tiles staged in LDS. GATED: W holds F gate rows and then F up rows, column j of the
-// result is act(w g_j) * (w u_j) and the A row of a pair is its token's (pair / top). Otherwise the A row is the
-// pair's own, and the result goes to `out` (pair rows, float32) or, where a token has one choice, straight onto
-// the residual into the token's row.
+// block, float32 sums from tiles staged in LDS. UP_GATED: W holds F gate rows and then F up rows, column j of the
+// result is act(w g_j) * (w u_j) and the A row of a pair is its token's (pair / top); UP_PLAIN: W holds F rows, the
+// result is act(u_j). DOWN: the A row is the pair's own, and the result goes to `out` (pair rows, float32) or, where a
+// token has one choice, straight onto the residual into the token's row.
+constexpr int DOWN = 0, UP_GATED = 1, UP_PLAIN = 2;
 struct ProductArgs {
-  const void* a;            // GATED: h [T, K]; else inner [pairs, K]
+  const void* a;            // UP: h [T, K]; DOWN: inner [pairs, K]
   const void* w;            // [E, N(, 2), K]
   const int* first;         // [E + 1]
   const int* order;         // [pairs]
   const float* weights;     // [pairs]
-  const float* residual;    // [T, N] or null (not GATED, one choice a token)
+  const float* residual;    // [T, N] or null (DOWN, one choice a token)
   void* out;
   int experts, top, n, k, act, weight_on_input, pairs;
   float limit;              // of the clamped activation
-  int direct;               // not GATED: pair rows are the tokens' rows of the result, and take the residual
+  int direct;               // DOWN: pair rows are the tokens' rows of the result, and take the residual
 };
 
-template <typename T, bool GATED>
+template <typename T, int KIND>
 __global__ void __launch_bounds__(256) expert_product_kernel(ProductArgs p) {
+  constexpr bool GATED = KIND == UP_GATED, UP = KIND != DOWN;
   constexpr int TM = 16, TN = 64, TK = 32;
   __shared__ float As[TM][TK + 1];
   __shared__ float Ws[GATED ? 2 : 1][TN][TK + 1];
@@ -206,7 +209,7 @@ __global__ void __launch_bounds__(256) expert_product_kernel(ProductArgs p) {
       const int r = i / TK, c = i - r * TK;
       const int pair = rows[r];
       float v = 0.f;
-      if (pair >= 0 && k0 + c < p.k) v = to_f32(A[(size_t)(GATED ? pair / p.top : pair) * p.k + k0 + c]);
+      if (pair >= 0 && k0 + c < p.k) v = to_f32(A[(size_t)(UP ? pair / p.top : pair) * p.k + k0 + c]);
       As[r][c] = v;
     }
     // the tile of W: 64 (or twice 64) rows of 32
@@ -241,6 +244,8 @@ __global__ void __launch_bounds__(256) expert_product_kernel(ProductArgs p) {
       float g = acc[0][r], u = acc[GATED ? 1 : 0][r];
       if (p.weight_on_input) g *= w, u *= w;
       ((T*)p.out)[(size_t)pair * p.n + col] = from_f32<T>(gated(g, u, p.act, p.limit));
+    } else if (UP) {
+      ((T*)p.out)[(size_t)pair * p.n + col] = from_f32<T>(apply_act(acc[0][r], p.act));
     } else {
       float y = acc[0][r];
       if (!p.weight_on_input) y *= w;
@@ -259,8 +264,9 @@ __global__ void __launch_bounds__(256) expert_product_kernel(ProductArgs p) {
 // by side (512 bytes or more a row and instruction, marked as read once), all of a chunk's loads under way
 // together, and takes the operands from there; the pairs' rows come from the caches. The waves of a block never
 // wait for one another.
-template <bool GATED>
+template <int KIND>
 __global__ void __launch_bounds__(256) expert_product_mfma_kernel(ProductArgs p) {
+  constexpr bool GATED = KIND == UP_GATED, UP = KIND != DOWN;
   constexpr int TM = 16;
   constexpr int ROWS = GATED ? 32 : 16;                   // rows of the matrix a wave holds
   constexpr int KC = 256;                                 // elements of a row a chunk
@@ -283,7 +289,7 @@ __global__ void __launch_bounds__(256) expert_product_mfma_kernel(ProductArgs p)
   const int col0 = (blockIdx.x * 4 + wave) * 16;
   if (col0 >= p.n) return;
   const int pair = r < count ? p.order[begin + r] : -1;
-  const bf16_t* xrow = (const bf16_t*)p.a + (size_t)(pair < 0 ? 0 : (GATED ? pair / p.top : pair)) * p.k;
+  const bf16_t* xrow = (const bf16_t*)p.a + (size_t)(pair < 0 ? 0 : (UP ? pair / p.top : pair)) * p.k;
   const bf16_t* W = (const bf16_t*)p.w + (size_t)e * (GATED ? 2 : 1) * p.n * p.k;
   bf16_t* mine = staged[wave];
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
@@ -326,6 +332,8 @@ __global__ void __launch_bounds__(256) expert_product_mfma_kernel(ProductArgs p)
       float gt = acc[i], up = acc_up[i];
       if (p.weight_on_input) gt *= w, up *= w;
       ((bf16_t*)p.out)[(size_t)pair * p.n + col] = (bf16_t)gated(gt, up, p.act, p.limit);
+    } else if (UP) {
+      ((bf16_t*)p.out)[(size_t)pair * p.n + col] = (bf16_t)apply_act(acc[i], p.act);
     } else {
       float y = acc[i];
       if (!p.weight_on_input) y *= w;
@@ -375,6 +383,36 @@ __global__ void gated_activation_kernel(const float* __restrict__ gu, T* __restr
   }
 }
 
+// act(x) from rows of float32, times sigmoid(row_gate) of the row
+template <typename T>
+__global__ void row_activation_kernel(const float* __restrict__ x, T* __restrict__ out, int f, int act, size_t total,
+                                      const float* __restrict__ row_gate, long long gate_ld) {
+  size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  const size_t stride = (size_t)gridDim.x * blockDim.x;
+  for (; i < total; i += stride) {
+    float y = apply_act(x[i], act);
+    if (row_gate) y *= 1.f / (1.f + expf(-row_gate[i / f * gate_ld]));
+    out[i] = from_f32<T>(y);
+  }
+}
+
+// the same, four neighbours a thread (rows of a multiple of four elements)
+template <typename T>
+__global__ void row_activation_four_kernel(const f32x4* __restrict__ x, T* __restrict__ out, int f4, int act, size_t total,
+                                           const float* __restrict__ row_gate, long long gate_ld) {
+  typedef T four __attribute__((ext_vector_type(4)));
+  size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  const size_t stride = (size_t)gridDim.x * blockDim.x;
+  for (; i < total; i += stride) {
+    const f32x4 v = x[i];
+    const float w = row_gate ? 1.f / (1.f + expf(-row_gate[i / f4 * gate_ld])) : 1.f;
+    four o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] = from_f32<T>(apply_act(v[e], act) * w);
+    ((four*)out)[i] = o;
+  }
+}
+
 int blocks_for(size_t total) {
   size_t b = (total + 255) / 256;
   return (int)(b > 16384 ? 16384 : (b ? b : 1));
@@ -401,7 +439,8 @@ extern "C" int tnx_expert_mixture(const void* h, const int* chosen, const float*
                                   const void* w_down, int* first, int* order, void* inner, float* pair_rows,
                                   const float* residual, float* out, int dtype, int tokens, int experts, int top,
                                   int width, int f, int act, int weight_on_input, int plain, float limit,
-                                  int identity, hipStream_t stream) {
+                                  int identity, int ungated, hipStream_t stream) {
+  TNX_REQUIRE(!ungated || !weight_on_input, "expert_mixture: experts without a gate take their weight on the output");
   TNX_REQUIRE(tokens >= 0 && experts > 0 && top > 0 && width > 0 && f > 0, "expert_mixture: bad sizes");
   TNX_REQUIRE(experts <= 4096, "expert_mixture: up to 4096 experts, got %d", experts);
   TNX_REQUIRE(dtype == TNX_F32 || dtype == TNX_BF16, "expert_mixture: dtype %d", dtype);
@@ -420,14 +459,23 @@ extern "C" int tnx_expert_mixture(const void* h, const int* chosen, const float*
                    act, weight_on_input, pairs, limit, direct ? 1 : 0};
   const dim3 grid_up((f + 63) / 64, tiles), grid_down((width + 63) / 64, tiles);
   if (dtype == TNX_F32) {
-    expert_product_kernel<float, true><<<grid_up, 256, 0, stream>>>(up);
-    expert_product_kernel<float, false><<<grid_down, 256, 0, stream>>>(down);
+    if (ungated)
+      expert_product_kernel<float, UP_PLAIN><<<grid_up, 256, 0, stream>>>(up);
+    else
+      expert_product_kernel<float, UP_GATED><<<grid_up, 256, 0, stream>>>(up);
+    expert_product_kernel<float, DOWN><<<grid_down, 256, 0, stream>>>(down);
   } else if (width % 8 == 0 && f % 8 == 0 && !plain) {
-    expert_product_mfma_kernel<true><<<grid_up, 256, 0, stream>>>(up);
-    expert_product_mfma_kernel<false><<<grid_down, 256, 0, stream>>>(down);
+    if (ungated)
+      expert_product_mfma_kernel<UP_PLAIN><<<grid_up, 256, 0, stream>>>(up);
+    else
+      expert_product_mfma_kernel<UP_GATED><<<grid_up, 256, 0, stream>>>(up);
+    expert_product_mfma_kernel<DOWN><<<grid_down, 256, 0, stream>>>(down);
   } else {
-    expert_product_kernel<bf16_t, true><<<grid_up, 256, 0, stream>>>(up);
-    expert_product_kernel<bf16_t, false><<<grid_down, 256, 0, stream>>>(down);
+    if (ungated)
+      expert_product_kernel<bf16_t, UP_PLAIN><<<grid_up, 256, 0, stream>>>(up);
+    else
+      expert_product_kernel<bf16_t, UP_GATED><<<grid_up, 256, 0, stream>>>(up);
+    expert_product_kernel<bf16_t, DOWN><<<grid_down, 256, 0, stream>>>(down);
   }
   TNX_CHECK_LAUNCH("expert products");
   if (!direct) {
@@ -457,6 +505,28 @@ extern "C" int tnx_gated_activation(const float* gate_up, void* out, int dtype, 
     gated_activation_kernel<bf16_t><<<blocks_for(total), 256, 0, stream>>>(gate_up, (bf16_t*)out, f, act, total,
                                                                             row_weights, limit);
   TNX_CHECK_LAUNCH("gated_activation");
+  return 0;
+}
+
+// act(x) of float32 rows, times sigmoid(row_gate) of its row (rows `gate_ld` apart) or not
+extern "C" int tnx_row_activation(const float* x, void* out, int dtype, int tokens, int f, int act, const float* row_gate,
+                                  long long gate_ld, hipStream_t stream) {
+  TNX_REQUIRE(tokens >= 0 && f > 0 && gate_ld >= 0, "row_activation: bad sizes");
+  TNX_REQUIRE(dtype == TNX_F32 || dtype == TNX_BF16, "row_activation: dtype %d", dtype);
+  if (tokens == 0) return 0;
+  const size_t total = (size_t)tokens * f;
+  if (f % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)out % (dtype == TNX_F32 ? 16 : 8) == 0) {
+    const size_t fours = total / 4;
+    if (dtype == TNX_F32)
+      row_activation_four_kernel<float><<<blocks_for(fours), 256, 0, stream>>>((const f32x4*)x, (float*)out, f / 4, act, fours, row_gate, gate_ld);
+    else
+      row_activation_four_kernel<bf16_t><<<blocks_for(fours), 256, 0, stream>>>((const f32x4*)x, (bf16_t*)out, f / 4, act, fours, row_gate, gate_ld);
+  } else if (dtype == TNX_F32) {
+    row_activation_kernel<float><<<blocks_for(total), 256, 0, stream>>>(x, (float*)out, f, act, total, row_gate, gate_ld);
+  } else {
+    row_activation_kernel<bf16_t><<<blocks_for(total), 256, 0, stream>>>(x, (bf16_t*)out, f, act, total, row_gate, gate_ld);
+  }
+  TNX_CHECK_LAUNCH("row_activation");
   return 0;
 }
 

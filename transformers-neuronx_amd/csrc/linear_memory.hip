@@ -1,9 +1,11 @@
 // Linear memories: a matrix S [n, v] a head that is carried from token to token,
 //     S_t = S' + k w^T,  S' = e^g S_(t-1),  o = S_t^T q,    w = write * val,  or with DELTA  w = write * (val - S'^T k),
-// and what stands before and after them in a mixer:
+// g a number a head or, with KEYED, one for every row of S (a key channel), and what stands before and after them in a mixer:
 //   memory_inputs   a short causal convolution over time with silu, unit vectors a head, decays and write weights
+//   channel_decays  the decays of every key channel through a bottleneck
+//   turn_heads      queries and keys turned by the position, in place
 //   memory_walk     the recurrence token by token (decoded tokens, short runs)
-//   memory_pairs, memory_scan   the same for long runs, 64 tokens at a time on the matrix unit
+//   memory_pairs (memory_pairs_keyed), memory_scan   the same for long runs, 64 tokens at a time on the matrix unit
 //   gated_norm      skip, gate and norm, up to what the output product reads
 // Everything is float32. State lies by position: the token at position p reads place (p - 1) & 1 of S's two (nothing at
 // p = 0) and writes place p & 1; the convolution's input at position p lies at place p mod taps. A step of single tokens
@@ -200,13 +202,81 @@ __global__ void __launch_bounds__(256) memory_state_kernel(InputArgs a) {
     mine[(size_t)(a.positions[first + i] % a.taps) * a.channels + c] = a.proj[(size_t)(first + i) * a.ld + a.conv_at + c];
 }
 
+// log_sigmoid(low w^T + bias) / tau for every key channel. A block takes 256 channels, one a thread, and TT tokens, whose
+// `low` goes through LDS 16 elements at a time.
+struct DecayArgs {
+  const float* low;         // [T, low_ld]
+  long long low_ld;
+  const void* w;            // [channels, rank]
+  const float* bias;        // [channels]
+  float over_tau;
+  float* out;               // [T, channels]
+  int tokens, channels, rank;
+};
+
+template <typename W, int TT>
+__global__ void __launch_bounds__(256) channel_decays_kernel(DecayArgs a) {
+  __shared__ __attribute__((aligned(16))) float low[TT * 16];
+  const int c = blockIdx.x * 256 + threadIdx.x, t0 = blockIdx.y * TT;
+  const bool in = c < a.channels;
+  const W* row = (const W*)a.w + (size_t)(in ? c : 0) * a.rank;
+  const float b = in ? a.bias[c] : 0.f;
+  float acc[TT];
+#pragma unroll
+  for (int t = 0; t < TT; ++t) acc[t] = 0.f;
+  for (int r0 = 0; r0 < a.rank; r0 += 16) {
+    if (r0 > 0) __syncthreads();
+    if (threadIdx.x < TT * 16) {
+      const int t = threadIdx.x >> 4, e = threadIdx.x & 15;
+      low[threadIdx.x] = t0 + t < a.tokens && r0 + e < a.rank ? a.low[(size_t)(t0 + t) * a.low_ld + r0 + e] : 0.f;
+    }
+    float w[16];
+#pragma unroll
+    for (int e = 0; e < 16; ++e) w[e] = in && r0 + e < a.rank ? to_f32(row[r0 + e]) : 0.f;
+    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < TT; ++t)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) acc[t] = fmaf(w[e], low[16 * t + e], acc[t]);
+  }
+  if (!in) return;
+#pragma unroll
+  for (int t = 0; t < TT; ++t)
+    if (t0 + t < a.tokens) a.out[(size_t)(t0 + t) * a.channels + c] = -softplus(-(acc[t] + b)) * a.over_tau;
+}
+
+// The first 2 half elements of `heads` heads of n, from column `at` of a row on, turned by the token's position, in place:
+// a block a token, a thread a pair; the token's sines and cosines are made once.
+__global__ void __launch_bounds__(256) turn_heads_kernel(float* __restrict__ x, int ld, int at, int heads, int n,
+                                                         const float* __restrict__ freqs, int half, int interleaved,
+                                                         const int* __restrict__ positions) {
+  __shared__ float cosines[128], sines[128];
+  const int t = blockIdx.x;
+  const float pos = (float)positions[t];
+  for (int i = threadIdx.x; i < half; i += 256) sincosf(pos * freqs[i], &sines[i], &cosines[i]);
+  __syncthreads();
+  float* row = x + (size_t)t * ld + at;
+  for (int f = threadIdx.x; f < heads * half; f += 256) {
+    const int head = f / half, i = f - head * half;
+    float* u = row + head * n + (interleaved ? 2 * i : i);
+    float* v = u + (interleaved ? 1 : half);
+    const float a = *u, b = *v, c = cosines[i], s = sines[i];
+    *u = a * c - b * s;
+    *v = b * c + a * s;
+  }
+}
+
 // ------------------------------------------------------------------------------------------ the memory, token by token
+
+// how a memory's S' and w come about
+constexpr int PLAIN = 0, DELTA_RULE = 1, KEYED = 2;
 
 struct WalkArgs {
   const float* u;           // [T, ld]
   int ld, q_at, k_at, v_at;
-  const float* log_decay;   // [T, H]
-  const float* write;       // [T, H]
+  const float* log_decay;   // [T, H]; [H] with decay_ld = 0: the same for every token; KEYED: [T, H n]
+  int decay_ld;             // elements from one token's decays to the next's
+  const float* write;       // [T, H] or null: 1
   const int* run_start;     // [R + 1]
   const int* cached;        // [R]
   const int* slots;         // [R]
@@ -240,13 +310,16 @@ __device__ __forceinline__ float sum16(float x) {
 // lanes share a column (column 16 b + 4 w + lane / 16): lane % 16 holds its rows NR (lane % 16) + j, j < NR. CH tokens a
 // chunk go through LDS, the next chunk's loads under way meanwhile, a token's operands read a token ahead.
 // With DELTA S^T k, S^T q and k . q are summed side by side from the S that came in, and S'^T q = S^T q + w (k . q).
-template <int NR, int CH, bool DELTA, bool ALIGNED>
+// KEYED: a token's decays go through LDS as its keys do.
+template <int NR, int CH, int MODE, bool ALIGNED>
 __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column_blocks) {
+  constexpr bool DELTA = MODE == DELTA_RULE;
   constexpr int np = 16 * NR;                             // a token's queries (and keys) in LDS, zeros behind n
   constexpr int PT = np / 4;                              // 16-byte pieces of a token's queries
   constexpr int QN = (CH * PT + 255) / 256;               // pieces of queries (and keys) a thread and chunk
   __shared__ __attribute__((aligned(16))) float qs[CH * np];
   __shared__ __attribute__((aligned(16))) float ks[CH * np];
+  __shared__ __attribute__((aligned(16))) float ds[MODE == KEYED ? CH * np : 4];      // e^g, row by row of S
   __shared__ __attribute__((aligned(16))) float vs[CH * 16];
   __shared__ float kp[CH], wr[CH];                        // e^g, write
   const int cb = blockIdx.x % column_blocks, rh = blockIdx.x / column_blocks;
@@ -276,7 +349,7 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
 #pragma unroll
     for (int j = 0; j < NR; ++j) S[j] = live && grp * NR + j < a.n ? Sp[grp * NR + j] : 0.f;
   }
-  f32x4 rq[QN], rk[QN], rv = {0.f, 0.f, 0.f, 0.f};
+  f32x4 rq[QN], rk[QN], rd[MODE == KEYED ? QN : 1], rv = {0.f, 0.f, 0.f, 0.f};
   float rkeep = 1.f, rwrite = 0.f;
   auto fetch = [&](int t0) {
     const int len = min(CH, count - t0);
@@ -287,6 +360,9 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
       const float* row = a.u + (size_t)(start + t0 + (in ? t : 0)) * a.ld + group * a.n + d;
       rq[u] = load4<ALIGNED>(row + a.q_at, in ? a.n - d : 0);
       rk[u] = load4<ALIGNED>(row + a.k_at, in ? a.n - d : 0);
+      if (MODE == KEYED)
+        rd[MODE == KEYED ? u : 0] =
+            load4<ALIGNED>(a.log_decay + (size_t)(start + t0 + (in ? t : 0)) * a.decay_ld + head * a.n + d, in ? a.n - d : 0);
     }
     if (threadIdx.x < CH * 4) {                            // a token's 16 values: four pieces
       const int t = threadIdx.x >> 2, c = 16 * cb + 4 * (threadIdx.x & 3);
@@ -295,9 +371,9 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
     }
     if (threadIdx.x < CH) {
       const bool in = threadIdx.x < len;
-      const size_t at = (size_t)(start + t0 + (in ? threadIdx.x : 0)) * a.heads + head;
-      rkeep = in ? expf(a.log_decay[at]) : 1.f;
-      rwrite = in ? a.write[at] : 0.f;
+      const size_t t = start + t0 + (in ? threadIdx.x : 0);
+      if (MODE != KEYED) rkeep = in ? expf(a.log_decay[t * a.decay_ld + head]) : 1.f;
+      rwrite = in ? (a.write ? a.write[t * a.heads + head] : 1.f) : 0.f;
     }
   };
   auto stash = [&]() {
@@ -307,6 +383,12 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
       if (f < CH * PT) {
         *(f32x4*)(qs + 4 * f) = rq[u];
         *(f32x4*)(ks + 4 * f) = rk[u];
+        if (MODE == KEYED) {
+          f32x4 e4;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) e4[e] = expf(rd[MODE == KEYED ? u : 0][e]);
+          *(f32x4*)(ds + 4 * f) = e4;
+        }
       }
     }
     if (threadIdx.x < CH * 4) *(f32x4*)(vs + 4 * threadIdx.x) = rv;
@@ -319,20 +401,26 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
     const int len = min(CH, count - t0);
     const bool more = t0 + CH < count;
     if (more) fetch(t0 + CH);                             // under way while this chunk is worked on
-    float q_n[NR], k_n[NR], val_n, keep_n, write_n;
+    float q_n[NR], k_n[NR], d_n[MODE == KEYED ? NR : 1], val_n, keep_n, write_n;
     auto read = [&](int t) {
       const float* q = qs + t * np + grp * NR;
       const float* k = ks + t * np + grp * NR;
 #pragma unroll
-      for (int j = 0; j < NR; ++j) q_n[j] = q[j], k_n[j] = k[j];
+      for (int j = 0; j < NR; ++j) {
+        q_n[j] = q[j], k_n[j] = k[j];
+        if (MODE == KEYED) d_n[MODE == KEYED ? j : 0] = ds[t * np + grp * NR + j];
+      }
       val_n = vs[t * 16 + 4 * wave + (lane >> 4)];
       keep_n = kp[t];
       write_n = wr[t];
     };
     auto token = [&](int t, bool last) {
-      float q[NR], k[NR];
+      float q[NR], k[NR], d[MODE == KEYED ? NR : 1];
 #pragma unroll
-      for (int j = 0; j < NR; ++j) q[j] = q_n[j], k[j] = k_n[j];
+      for (int j = 0; j < NR; ++j) {
+        q[j] = q_n[j], k[j] = k_n[j];
+        if (MODE == KEYED) d[MODE == KEYED ? j : 0] = d_n[MODE == KEYED ? j : 0];
+      }
       const float val = val_n, keep = keep_n, write = write_n;
       if (!last) read(t + 1);
       float o = 0.f;
@@ -354,7 +442,7 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
         const float w = write * val;
 #pragma unroll
         for (int j = 0; j < NR; ++j) {
-          S[j] = keep * S[j] + k[j] * w;
+          S[j] = (MODE == KEYED ? d[MODE == KEYED ? j : 0] : keep) * S[j] + k[j] * w;
           o += S[j] * q[j];
         }
         o = sum16(o);
@@ -391,35 +479,35 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
     if (grp * NR + j < a.n) Sw[grp * NR + j] = S[j];
 }
 
-template <int NR, bool DELTA>
+template <int NR, int MODE>
 void launch_walk(const WalkArgs& a, int requests, bool singles, bool aligned, hipStream_t stream) {
   constexpr int CH = NR == 16 ? 16 : 32;
   const int column_blocks = (a.v + 15) / 16;
   const dim3 grid(requests * a.heads * column_blocks);
   if (singles) {
     if (aligned)
-      memory_walk_kernel<NR, 1, DELTA, true><<<grid, 256, 0, stream>>>(a, column_blocks);
+      memory_walk_kernel<NR, 1, MODE, true><<<grid, 256, 0, stream>>>(a, column_blocks);
     else
-      memory_walk_kernel<NR, 1, DELTA, false><<<grid, 256, 0, stream>>>(a, column_blocks);
+      memory_walk_kernel<NR, 1, MODE, false><<<grid, 256, 0, stream>>>(a, column_blocks);
   } else {
     if (aligned)
-      memory_walk_kernel<NR, CH, DELTA, true><<<grid, 256, 0, stream>>>(a, column_blocks);
+      memory_walk_kernel<NR, CH, MODE, true><<<grid, 256, 0, stream>>>(a, column_blocks);
     else
-      memory_walk_kernel<NR, CH, DELTA, false><<<grid, 256, 0, stream>>>(a, column_blocks);
+      memory_walk_kernel<NR, CH, MODE, false><<<grid, 256, 0, stream>>>(a, column_blocks);
   }
 }
 
-template <bool DELTA>
+template <int MODE>
 void launch_walk_sized(const WalkArgs& a, int requests, bool singles, bool aligned, hipStream_t stream) {
   const int rows16 = (a.n + 15) / 16;
   if (rows16 <= 2)
-    launch_walk<2, DELTA>(a, requests, singles, aligned, stream);
+    launch_walk<2, MODE>(a, requests, singles, aligned, stream);
   else if (rows16 <= 4)
-    launch_walk<4, DELTA>(a, requests, singles, aligned, stream);
+    launch_walk<4, MODE>(a, requests, singles, aligned, stream);
   else if (rows16 <= 8)
-    launch_walk<8, DELTA>(a, requests, singles, aligned, stream);
+    launch_walk<8, MODE>(a, requests, singles, aligned, stream);
   else
-    launch_walk<16, DELTA>(a, requests, singles, aligned, stream);
+    launch_walk<16, MODE>(a, requests, singles, aligned, stream);
 }
 
 // ------------------------------------------------------------------------------------------ the memory, chunk by chunk
@@ -448,8 +536,9 @@ constexpr int TILE = 256;                 // elements of 64 lanes by four
 struct ChunkArgs {
   const float* u;           // [T, ld]
   int ld, q_at, k_at, v_at;
-  const float* log_decay;   // [T, H]
-  const float* write;       // [T, H]
+  const float* log_decay;   // [T, H]; [H] with decay_ld = 0; KEYED: [T, H n]
+  int decay_ld;
+  const float* write;       // [T, H] or null: 1
   const int* run_start;
   const int* cached;
   const int* slots;
@@ -468,6 +557,7 @@ struct ChunkArgs {
                             //   zero for j > i, unwritten for s > w
   float* wx;                // [chunks, H, 4, NB, tile]: w, as the queries
   float* ux;                // [chunks, H, blocks of 16 columns, 4, tile]: u0, column l % 16, tokens 16 w + 4 (l / 16) ..
+  float* keep;              // KEYED: [chunks, H, 16 NB]: e^c_64 a row of S (and qx and kx, a head's, hold the scaled ones)
   int heads, groups, n, v;
 };
 
@@ -546,14 +636,14 @@ __global__ void __launch_bounds__(DELTA ? 512 : 256) memory_pairs_kernel(ChunkAr
     const size_t place = (size_t)chunk * a.heads + head;
     if (wave == 0) {
       const size_t at = (size_t)(t0 + min(lane, len - 1)) * a.heads + head;
-      double c = lane < len ? (double)a.log_decay[at] : 0.0;
+      double c = lane < len ? (double)a.log_decay[(size_t)(t0 + min(lane, len - 1)) * a.decay_ld + head] : 0.0;
 #pragma unroll
       for (int d = 1; d < 64; d *= 2) {
         const double before = __shfl_up(c, d, 64);
         if (lane >= d) c += before;
       }
       const double all = __shfl(c, 63, 64);
-      const float e = expf((float)c), b = lane < len ? a.write[at] : 0.f;
+      const float e = expf((float)c), b = lane < len ? (a.write ? a.write[at] : 1.f) : 0.f;
       cs[lane] = c;
       up[lane] = e;
       beta[lane] = b;
@@ -679,18 +769,177 @@ __global__ void __launch_bounds__(DELTA ? 512 : 256) memory_pairs_kernel(ChunkAr
   }
 }
 
+// KEYED, a decay for every row d of S: with c_i[d] the chunk's sums,
+//     o_i = sum_d q_i[d] e^(c_i[d]) S[d] + sum_{j<=i} A_ij val_j,   A_ij = sum_d q_i[d] k_j[d] e^(c_i[d] - c_j[d])
+//     the state after the chunk: e^(c_64[d]) S[d] + sum_j k_j[d] e^(c_64[d] - c_j[d]) val_j
+// No single point d of reference serves all of A: e^(-c_j) alone overflows where a channel forgets fast. The chunk goes in
+// four blocks of 16 tokens, l the sums inside a block and L_b a block's whole: a pair of blocks J < I is the product of
+// q_i e^(l_i) e^(L_(J+1) + .. + L_(I-1)) with k_j e^(L_J - l_j), no exponent above zero. Inside a block q_i e^(l_i) meets
+// k_j e^(-l_j) as long as no channel of the block forgets by more than 2^-LEVEL (float32 then still holds both factors to
+// full precision); a block that does makes its weights pair by pair, the exponents' difference first. Sums are taken in
+// float64 and kept in powers of two.
+//
+// grid: chunks * heads; channels in pieces of at most 128; wave w has the tokens 16 w .. 16 w + 15 as queries.
+constexpr double LOG2E = 1.4426950408889634074;
+constexpr float LEVEL = 60.f;
+__device__ __forceinline__ float pow2(float x) { return __builtin_amdgcn_exp2f(x); }
+
+template <int NB, bool ALIGNED>
+__global__ void __launch_bounds__(256) memory_pairs_keyed_kernel(ChunkArgs a) {
+  constexpr int P = NB < 8 ? NB : 8, PIECES = NB / P, PD = 16 * P, LD = PD + 4, PT = 4 * P;
+  extern __shared__ __attribute__((aligned(16))) float room[];
+  __shared__ __attribute__((aligned(16))) float tot[4 * PD];      // L_b, a block of tokens behind the other
+  float* q_l = room;                            // [64][LD]
+  float* k_l = q_l + CHUNK * LD;                // [64][LD]
+  float* c_l = k_l + CHUNK * LD;                // [64][LD]: l
+  const int head = blockIdx.x % a.heads, chunk = blockIdx.x / a.heads;
+  const int run = a.chunk_run[chunk], begin = a.chunk_begin[chunk];
+  const int t0 = a.run_start[run] + begin, len = min(CHUNK, a.run_start[run + 1] - t0);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
+  const size_t place = (size_t)chunk * a.heads + head;
+  const float* base = a.u + (size_t)t0 * a.ld + head * a.n;
+  const float* decay = a.log_decay + (size_t)t0 * a.decay_ld + head * a.n;
+  // prod[cb][e]: token j = 16 cb + 4 g + e (key) with token i = 16 wave + r
+  f32x4 prod[4];
+#pragma unroll
+  for (int cb = 0; cb < 4; ++cb) prod[cb] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  for (int piece = 0; piece < PIECES; ++piece) {
+    const int d0 = PD * piece;
+    if (piece > 0) __syncthreads();             // before the next piece takes the place of what this one read
+#pragma unroll 4
+    for (int f = threadIdx.x; f < CHUNK * PT; f += 256) {        // zeros behind n and from the run's end on
+      const int t = f / PT, d = 4 * (f - t * PT);
+      const float* row = base + (unsigned)(min(t, len - 1) * a.ld) + d0 + d;
+      const int valid = t < len ? a.n - d0 - d : 0;
+      *(f32x4*)(q_l + t * LD + d) = load4<ALIGNED>(row + a.q_at, valid);
+      *(f32x4*)(k_l + t * LD + d) = load4<ALIGNED>(row + a.k_at, valid);
+    }
+    for (int f = threadIdx.x; f < 4 * PD; f += 256) {
+      const int b = f / PD, d = f - b * PD;
+      const bool in = d0 + d < a.n;
+      float got[16];
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int t = 16 * b + i;
+        got[i] = in && t < len ? decay[(unsigned)(t * a.decay_ld) + d0 + d] : 0.f;
+      }
+      double c = 0.0;
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        c += (double)got[i];
+        c_l[(16 * b + i) * LD + d] = (float)(c * LOG2E);
+      }
+      tot[f] = (float)(c * LOG2E);
+    }
+    __syncthreads();
+    // what the second kernel reads: q_i e^(c_i), k_j e^(c_64 - c_j), e^(c_64)
+    float* qx = a.qx + (place * 4 + wave) * NB * TILE + 4 * lane;
+    const float* my_q = q_l + (16 * wave + r) * LD + 4 * g;
+    const float* my_c = c_l + (16 * wave + r) * LD + 4 * g;
+#pragma unroll 2
+    for (int s = 0; s < P; ++s) {
+      const f32x4 q = *(const f32x4*)(my_q + 16 * s), l = *(const f32x4*)(my_c + 16 * s);
+      f32x4 before = {0.f, 0.f, 0.f, 0.f};
+      for (int b = 0; b < wave; ++b) before = before + *(const f32x4*)(tot + b * PD + 16 * s + 4 * g);
+      f32x4 x;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) x[e] = q[e] * pow2(before[e] + l[e]);
+      *(f32x4*)(qx + (P * piece + s) * TILE) = x;
+    }
+    float* kx = a.kx + place * NB * 4 * TILE + 4 * lane;
+    for (int f = wave; f < 4 * P; f += 4) {
+      const int x = f >> 2, s = f & 3, d = 16 * x + r;
+      float after = tot[s * PD + d];
+      for (int b = s + 1; b < 4; ++b) after += tot[b * PD + d];
+      f32x4 v;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int at = (16 * s + 4 * g + e) * LD + d;
+        v[e] = k_l[at] * pow2(after - c_l[at]);
+      }
+      *(f32x4*)(kx + (4 * P * piece + f) * TILE) = v;
+    }
+    for (int d = threadIdx.x; d < PD; d += 256)
+      a.keep[place * 16 * NB + d0 + d] = pow2(tot[d] + tot[PD + d] + tot[2 * PD + d] + tot[3 * PD + d]);
+    // the weights: does a channel of this wave's block forget too fast for one point of reference?
+    float worst = 0.f;
+    for (int d = lane; d < PD; d += 64) worst = fmaxf(worst, -tot[wave * PD + d]);
+    const bool gentle = wave_max(worst) <= LEVEL;
+#pragma unroll 2
+    for (int s = 0; s < P; ++s) {
+      const f32x4 q = *(const f32x4*)(my_q + 16 * s), l = *(const f32x4*)(my_c + 16 * s);
+      f32x4 x;                                   // q_i e^(l_i), times the blocks between as they come in between
+#pragma unroll
+      for (int e = 0; e < 4; ++e) x[e] = q[e] * pow2(l[e]);
+      if (gentle) {
+        f32x4 kb = *(const f32x4*)(k_l + (16 * wave + r) * LD + 16 * s + 4 * g);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) kb[e] *= pow2(-l[e]);
+#pragma unroll
+        for (int cb = 0; cb < 4; ++cb)
+          if (cb == wave) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) prod[cb] = __builtin_amdgcn_mfma_f32_16x16x4f32(kb[e], x[e], prod[cb], 0, 0, 0);
+          }
+      }
+#pragma unroll
+      for (int cb = 2; cb >= 0; --cb) {
+        if (cb >= wave) continue;
+        const f32x4 whole = *(const f32x4*)(tot + cb * PD + 16 * s + 4 * g);
+        f32x4 kb = *(const f32x4*)(k_l + (16 * cb + r) * LD + 16 * s + 4 * g);
+        const f32x4 lk = *(const f32x4*)(c_l + (16 * cb + r) * LD + 16 * s + 4 * g);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) kb[e] *= pow2(whole[e] - lk[e]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) prod[cb] = __builtin_amdgcn_mfma_f32_16x16x4f32(kb[e], x[e], prod[cb], 0, 0, 0);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) x[e] *= pow2(whole[e]);
+      }
+    }
+    if (!gentle) {
+      // pair by pair: the lane's query i = 16 wave + r with the keys 16 wave + 4 g + e
+      f32x4 sum = {0.f, 0.f, 0.f, 0.f};
+      const float* qi = q_l + (16 * wave + r) * LD;
+      const float* ci = c_l + (16 * wave + r) * LD;
+      for (int d = 0; d < PD; d += 4) {
+        const f32x4 q = *(const f32x4*)(qi + d), l = *(const f32x4*)(ci + d);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const f32x4 k = *(const f32x4*)(k_l + (16 * wave + 4 * g + e) * LD + d);
+          const f32x4 lk = *(const f32x4*)(c_l + (16 * wave + 4 * g + e) * LD + d);
+#pragma unroll
+          for (int c = 0; c < 4; ++c) sum[e] += q[c] * k[c] * pow2(fminf(l[c] - lk[c], 0.f));
+        }
+      }
+#pragma unroll
+      for (int cb = 0; cb < 4; ++cb)
+        if (cb == wave) prod[cb] = prod[cb] + sum;
+    }
+  }
+  float* pairs = a.pairs + (place * 4 + wave) * 4 * TILE + 4 * lane;
+#pragma unroll
+  for (int cb = 0; cb < 4; ++cb) {
+    if (cb > wave) continue;
+    f32x4 v;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = 16 * cb + 4 * g + e <= 16 * wave + r ? prod[cb][e] : 0.f;
+    *(f32x4*)(pairs + cb * TILE) = v;
+  }
+}
+
 // grid: (run, head) pairs in eights * column blocks: the blocks of a (run, head) come eight apart, so that they share an
 // XCD's cache. A block walks a run's chunks for 16 columns of S; wave w has the chunk's tokens 16 w .. 16 w + 15, and of S
 // the blocks of 16 rows w, w + 4, ..., in the accumulators from chunk to chunk. What a chunk's products read of memory is
 // asked for two chunks ahead, into the registers (one set for even, one for odd chunks) that the chunk before last has
 // just read: a compute unit has one such block, and a load takes as long as a chunk's products do.
-template <int NB, bool DELTA, bool ALIGNED>
+template <int NB, int MODE, bool ALIGNED>
 __global__ void __launch_bounds__(256, 1) memory_scan_kernel(ChunkArgs a, int column_blocks) {
+  constexpr bool DELTA = MODE == DELTA_RULE;
   constexpr int RB = (NB + 3) / 4;               // blocks of rows of S a wave
   constexpr int SLD = 16 * NB + 4, ULD = CHUNK + 4;
   __shared__ __attribute__((aligned(16))) float s_l[16 * SLD];        // [column][row]
   __shared__ __attribute__((aligned(16))) float u_l[16 * ULD];        // [column][token]: the writes
-  __shared__ __attribute__((aligned(16))) float b_l[16 * ULD];        // the same times e^(c_64 - c_j)
+  __shared__ __attribute__((aligned(16))) float b_l[MODE == KEYED ? 4 : 16 * ULD];        // the same times e^(c_64 - c_j)
   const int rh = (blockIdx.x & 7) + 8 * (blockIdx.x / (8 * column_blocks));
   const int cb = (blockIdx.x >> 3) % column_blocks;
   if (rh >= a.num_long * a.heads) return;
@@ -718,7 +967,7 @@ __global__ void __launch_bounds__(256, 1) memory_scan_kernel(ChunkArgs a, int co
   }
   share();
   struct Set {
-    f32x4 wa[DELTA ? NB : 1], qa[NB], pa[4], kt[RB][4], u0, up, down, wr;
+    f32x4 wa[DELTA ? NB : 1], qa[NB], pa[4], kt[RB][4], keep[MODE == KEYED ? RB : 1], u0, up, down, wr;
     float decay;
   };
   Set even, odd;
@@ -738,6 +987,12 @@ __global__ void __launch_bounds__(256, 1) memory_scan_kernel(ChunkArgs a, int co
       const float* vals = a.u + (size_t)t0 * a.ld + a.v_at + head * a.v + ccol;
 #pragma unroll
       for (int e = 0; e < 4; ++e) z.u0[e] = vals[(unsigned)(min(16 * wave + 4 * g + e, len - 1) * a.ld)];
+    }
+    if (MODE == KEYED) {
+#pragma unroll
+      for (int x = 0; x < RB; ++x)
+        z.keep[MODE == KEYED ? x : 0] = *(const f32x4*)(a.keep + of_head * 16 * NB + 16 * min(wave + 4 * x, NB - 1) + 4 * g);
+      return;
     }
     const float* gates = a.gates + of_head * 3 * CHUNK;
     z.up = *(const f32x4*)(gates + 16 * wave + 4 * g);
@@ -775,19 +1030,26 @@ __global__ void __launch_bounds__(256, 1) memory_scan_kernel(ChunkArgs a, int co
         if (DELTA) m = __builtin_amdgcn_mfma_f32_16x16x4f32(z.wa[DELTA ? s : 0][e], s4[e], m, 0, 0, 0);
       }
     }
-    const f32x4 u4 = DELTA ? z.u0 - m : z.wr * z.u0;
+    // (KEYED: the decays are in the queries, the keys and the weights already)
+    const f32x4 u4 = DELTA ? z.u0 - m : MODE == KEYED ? z.u0 : z.wr * z.u0;
     *(f32x4*)(u_l + r * ULD + 16 * wave + 4 * g) = u4;
-    *(f32x4*)(b_l + r * ULD + 16 * wave + 4 * g) = u4 * z.down;
-    o = o * z.up;
-    const float keep = z.decay;
+    if (MODE != KEYED) {
+      *(f32x4*)(b_l + r * ULD + 16 * wave + 4 * g) = u4 * z.down;
+      o = o * z.up;
+    }
+#pragma unroll
+    for (int x = 0; x < RB; ++x) {
+      if (MODE == KEYED)
+        S[x] = S[x] * z.keep[MODE == KEYED ? x : 0];
+      else
+        S[x] = S[x] * z.decay;
+    }
     if (c + 2 < chunks) fetch_state_side(c + 2, z);
     __syncthreads();
 #pragma unroll
-    for (int x = 0; x < RB; ++x) S[x] = S[x] * keep;
-#pragma unroll
     for (int s = 0; s < 4; ++s) {
       const f32x4 us = *(const f32x4*)(u_l + r * ULD + 16 * s + 4 * g);
-      const f32x4 bs = *(const f32x4*)(b_l + r * ULD + 16 * s + 4 * g);
+      const f32x4 bs = MODE == KEYED ? us : *(const f32x4*)(b_l + r * ULD + 16 * s + 4 * g);
 #pragma unroll
       for (int e = 0; e < 4; ++e)
 #pragma unroll
@@ -826,38 +1088,50 @@ __global__ void __launch_bounds__(256, 1) memory_scan_kernel(ChunkArgs a, int co
   }
 }
 
-template <int NB, bool DELTA, bool ALIGNED>
+template <int NB, int MODE, bool ALIGNED>
 int launch_chunks(const ChunkArgs& a, hipStream_t stream) {
+  constexpr bool DELTA = MODE == DELTA_RULE;
   const int per_group = a.heads / a.groups;
-  int per = 1;                                   // heads of a group a block of the first kernel
-  while (!DELTA && per < per_group && (long long)a.chunks * a.groups * ((per_group + 2 * per - 1) / (2 * per)) >= 2 * tnx_compute_units())
-    per *= 2;
-  const int parts = (per_group + per - 1) / per;
   const int column_blocks = (a.v + 15) / 16;
-  const int lds = (2 * CHUNK * (16 * NB + 4) + (DELTA ? CHUNK * (CHUNK + 4) + CHUNK * 20 : 0)) * (int)sizeof(float);
   static bool configured = false;
-  if (!configured) {
-    const hipError_t e = hipFuncSetAttribute((const void*)memory_pairs_kernel<NB, DELTA, ALIGNED>,
-                                             hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-    TNX_REQUIRE(e == hipSuccess, "memory_chunks: cannot reserve %d bytes of LDS: %s", lds, hipGetErrorString(e));
-    configured = true;
+  if constexpr (MODE == KEYED) {
+    constexpr int lds = 3 * CHUNK * (16 * (NB < 8 ? NB : 8) + 4) * (int)sizeof(float);
+    if (!configured) {
+      const hipError_t e = hipFuncSetAttribute((const void*)memory_pairs_keyed_kernel<NB, ALIGNED>,
+                                               hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+      TNX_REQUIRE(e == hipSuccess, "memory_chunks: cannot reserve %d bytes of LDS: %s", lds, hipGetErrorString(e));
+      configured = true;
+    }
+    memory_pairs_keyed_kernel<NB, ALIGNED><<<(unsigned)((size_t)a.chunks * a.heads), 256, lds, stream>>>(a);
+  } else {
+    int per = 1;                                   // heads of a group a block of the first kernel
+    while (!DELTA && per < per_group && (long long)a.chunks * a.groups * ((per_group + 2 * per - 1) / (2 * per)) >= 2 * tnx_compute_units())
+      per *= 2;
+    const int parts = (per_group + per - 1) / per;
+    const int lds = (2 * CHUNK * (16 * NB + 4) + (DELTA ? CHUNK * (CHUNK + 4) + CHUNK * 20 : 0)) * (int)sizeof(float);
+    if (!configured) {
+      const hipError_t e = hipFuncSetAttribute((const void*)memory_pairs_kernel<NB, DELTA, ALIGNED>,
+                                               hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+      TNX_REQUIRE(e == hipSuccess, "memory_chunks: cannot reserve %d bytes of LDS: %s", lds, hipGetErrorString(e));
+      configured = true;
+    }
+    memory_pairs_kernel<NB, DELTA, ALIGNED>
+        <<<(unsigned)((size_t)a.chunks * a.groups * parts), DELTA ? 512 : 256, lds, stream>>>(a, parts, per);
   }
-  memory_pairs_kernel<NB, DELTA, ALIGNED>
-      <<<(unsigned)((size_t)a.chunks * a.groups * parts), DELTA ? 512 : 256, lds, stream>>>(a, parts, per);
   TNX_CHECK_LAUNCH("memory_pairs");
-  memory_scan_kernel<NB, DELTA, ALIGNED>
+  memory_scan_kernel<NB, MODE, ALIGNED>
       <<<(unsigned)((a.num_long * a.heads + 7) / 8 * 8 * column_blocks), 256, 0, stream>>>(a, column_blocks);
   TNX_CHECK_LAUNCH("memory_scan");
   return 0;
 }
 
-template <bool DELTA, bool ALIGNED>
+template <int MODE, bool ALIGNED>
 int launch_chunks_sized(const ChunkArgs& a, int nb, hipStream_t stream) {
   switch (nb) {
-    case 2: return launch_chunks<2, DELTA, ALIGNED>(a, stream);
-    case 4: return launch_chunks<4, DELTA, ALIGNED>(a, stream);
-    case 8: return launch_chunks<8, DELTA, ALIGNED>(a, stream);
-    default: return launch_chunks<16, DELTA, ALIGNED>(a, stream);
+    case 2: return launch_chunks<2, MODE, ALIGNED>(a, stream);
+    case 4: return launch_chunks<4, MODE, ALIGNED>(a, stream);
+    case 8: return launch_chunks<8, MODE, ALIGNED>(a, stream);
+    default: return launch_chunks<16, MODE, ALIGNED>(a, stream);
   }
 }
 
@@ -867,14 +1141,16 @@ struct FinishArgs {
   const float* o;           // [T, width]
   const float* gate;        // [T, gate_ld]
   long long gate_ld;
-  const float* weight;      // [width]
+  const float* weight;      // [width] or null: 1
   float eps;
   int parts, gate_first;
   const float* skip;        // [heads] or null
   const float* x;           // [T, x_ld]
   long long x_ld;
   int per_head;             // elements a head
-  void* out;                // [T, width]
+  void* out;                // [T, out_ld]
+  long long out_ld;
+  float out_scale;
   int tokens, width;
 };
 
@@ -946,11 +1222,10 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(FinishArgs a) {
   }
   if (!active) return;
   const float r = 1.f / sqrtf(s / (float)size + a.eps);
-  T* out = (T*)a.out + t * a.width + first;
-  const float* w = a.weight + first;
+  T* out = (T*)a.out + t * a.out_ld + first;
   auto put = [&](int i, f32x4 y) {
-    const f32x4 ws = load4<ALIGNED>(w + i, size - i);
-    y = y * r * ws;
+    y = y * r;
+    if (a.weight) y = y * load4<ALIGNED>(a.weight + first + i, size - i);
     if (!a.gate_first) {
       const f32x4 gs = load4<ALIGNED>(gate + i, size - i);
 #pragma unroll
@@ -959,7 +1234,7 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(FinishArgs a) {
     typedef T four __attribute__((ext_vector_type(4)));
     four v;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) v[e] = from_f32<T>(y[e]);
+    for (int e = 0; e < 4; ++e) v[e] = from_f32<T>(y[e] * a.out_scale);
     if (ALIGNED) {
       *(four*)(out + i) = v;
     } else {
@@ -1053,10 +1328,48 @@ extern "C" int tnx_memory_inputs(const float* proj, int ld, int conv_at, int cha
   return 0;
 }
 
-extern "C" int tnx_memory_walk(const float* u, int ld, int q_at, int k_at, int v_at, const float* log_decay,
+extern "C" int tnx_channel_decays(const float* low, long long low_ld, const void* w, int w_dtype, const float* bias, float over_tau,
+                                  float* out, int tokens, int channels, int rank, hipStream_t stream) {
+  TNX_REQUIRE(tokens >= 0 && channels > 0 && rank > 0 && low_ld >= rank, "channel_decays: bad sizes");
+  TNX_REQUIRE(w_dtype == TNX_F32 || w_dtype == TNX_BF16, "channel_decays: dtype %d", w_dtype);
+  TNX_REQUIRE(tokens < 16 * 65535, "channel_decays: too many tokens");
+  if (tokens == 0) return 0;
+  DecayArgs a{low, low_ld, w, bias, over_tau, out, tokens, channels, rank};
+  const int blocks = (channels + 255) / 256;
+  // few tokens: one a block, so that the chip has something to do
+  if ((long long)blocks * tokens <= 4 * tnx_compute_units()) {
+    if (w_dtype == TNX_F32)
+      channel_decays_kernel<float, 1><<<dim3(blocks, tokens), 256, 0, stream>>>(a);
+    else
+      channel_decays_kernel<bf16_t, 1><<<dim3(blocks, tokens), 256, 0, stream>>>(a);
+  } else {
+    if (w_dtype == TNX_F32)
+      channel_decays_kernel<float, 16><<<dim3(blocks, (tokens + 15) / 16), 256, 0, stream>>>(a);
+    else
+      channel_decays_kernel<bf16_t, 16><<<dim3(blocks, (tokens + 15) / 16), 256, 0, stream>>>(a);
+  }
+  TNX_CHECK_LAUNCH("channel_decays");
+  return 0;
+}
+
+extern "C" int tnx_turn_heads(float* x, int ld, int at, int heads, int n, const float* freqs, int half, int interleaved,
+                              const int* positions, int tokens, hipStream_t stream) {
+  TNX_REQUIRE(tokens >= 0 && heads > 0 && n > 0 && at >= 0 && ld >= at + heads * n, "turn_heads: bad sizes");
+  TNX_REQUIRE(half > 0 && half <= 128 && 2 * half <= n, "turn_heads: %d turned elements in heads of %d", 2 * half, n);
+  if (tokens == 0) return 0;
+  turn_heads_kernel<<<tokens, 256, 0, stream>>>(x, ld, at, heads, n, freqs, half, interleaved, positions);
+  TNX_CHECK_LAUNCH("turn_heads");
+  return 0;
+}
+
+// `mode`: 0 plain, 1 with the delta rule, 2 a decay for every row of S (`log_decay` [T, H n]). `decay_ld`: elements from one
+// token's decays to the next's (0: the same for every token).
+extern "C" int tnx_memory_walk(const float* u, int ld, int q_at, int k_at, int v_at, const float* log_decay, int decay_ld,
                                const float* write, const int* run_start, const int* cached, const int* slots, float* memory,
-                               float* out, int tokens, int requests, int heads, int groups, int n, int v, int delta,
+                               float* out, int tokens, int requests, int heads, int groups, int n, int v, int mode,
                                int longest, hipStream_t stream) {
+  TNX_REQUIRE(mode >= PLAIN && mode <= KEYED && (mode != KEYED || (groups == heads && !write)), "memory_walk: bad mode");
+  TNX_REQUIRE(decay_ld == 0 || decay_ld >= (mode == KEYED ? heads * n : heads), "memory_walk: rows of %d decays", decay_ld);
   TNX_REQUIRE(tokens >= 0 && requests >= 0 && heads > 0 && groups > 0 && heads % groups == 0 && n > 0 && v > 0,
               "memory_walk: bad sizes");
   TNX_REQUIRE(n <= 256, "memory_walk: query/key heads of up to 256 elements, got %d", n);
@@ -1064,13 +1377,16 @@ extern "C" int tnx_memory_walk(const float* u, int ld, int q_at, int k_at, int v
               "memory_walk: rows of %d elements do not hold what is read", ld);
   if (tokens == 0 || requests == 0) return 0;
   TNX_REQUIRE((long long)requests * heads * ((v + 15) / 16) < (1ll << 31), "memory_walk: too many blocks");
-  WalkArgs a{u, ld, q_at, k_at, v_at, log_decay, write, run_start, cached, slots, memory, out, heads, groups, n, v, longest};
+  WalkArgs a{u, ld, q_at, k_at, v_at, log_decay, decay_ld, write, run_start, cached, slots, memory, out, heads, groups, n, v, longest};
   // rows and heads that begin at multiples of 16 bytes are loaded 16 bytes at a time
-  const bool aligned = n % 4 == 0 && v % 4 == 0 && ((ld | q_at | k_at | v_at) & 3) == 0 && (uintptr_t)u % 16 == 0;
-  if (delta)
-    launch_walk_sized<true>(a, requests, tokens == requests, aligned, stream);
+  const bool aligned = n % 4 == 0 && v % 4 == 0 && ((ld | q_at | k_at | v_at) & 3) == 0 && (uintptr_t)u % 16 == 0 &&
+                       (mode != KEYED || (decay_ld % 4 == 0 && (uintptr_t)log_decay % 16 == 0));
+  if (mode == DELTA_RULE)
+    launch_walk_sized<DELTA_RULE>(a, requests, tokens == requests, aligned, stream);
+  else if (mode == KEYED)
+    launch_walk_sized<KEYED>(a, requests, tokens == requests, aligned, stream);
   else
-    launch_walk_sized<false>(a, requests, tokens == requests, aligned, stream);
+    launch_walk_sized<PLAIN>(a, requests, tokens == requests, aligned, stream);
   TNX_CHECK_LAUNCH("memory_walk");
   return 0;
 }
@@ -1078,12 +1394,16 @@ extern "C" int tnx_memory_walk(const float* u, int ld, int q_at, int k_at, int v
 // The runs of several tokens that `long_run` names, chunk by chunk: `chunk_run` and `chunk_begin` name the chunks of 64
 // tokens, a run's chunks one behind the other from `long_first` on. `room`: what the first kernel leaves for the second,
 // `room_size` floats: with nb = 2, 4, 8 or 16, the least with n <= 16 nb, for every chunk 2 G 1024 nb + H (3 * 64 + 4096),
-// and with `delta` H (1024 nb + 1024 ceil(v / 16)) more.
-extern "C" int tnx_memory_chunks(const float* u, int ld, int q_at, int k_at, int v_at, const float* log_decay,
+// and with the delta rule H (1024 nb + 1024 ceil(v / 16)) more, with a decay for every row of S H 16 nb more. `mode` and
+// `decay_ld` as above.
+extern "C" int tnx_memory_chunks(const float* u, int ld, int q_at, int k_at, int v_at, const float* log_decay, int decay_ld,
                                  const float* write, const int* run_start, const int* cached, const int* slots,
                                  const int* chunk_run, const int* chunk_begin, int chunks, int chunk_size, const int* long_run,
                                  const int* long_first, int num_long, float* memory, float* out, float* room,
-                                 long long room_size, int heads, int groups, int n, int v, int delta, hipStream_t stream) {
+                                 long long room_size, int heads, int groups, int n, int v, int mode, hipStream_t stream) {
+  TNX_REQUIRE(mode >= PLAIN && mode <= KEYED && (mode != KEYED || (groups == heads && !write)), "memory_chunks: bad mode");
+  TNX_REQUIRE(decay_ld == 0 || decay_ld >= (mode == KEYED ? heads * n : heads), "memory_chunks: rows of %d decays", decay_ld);
+  TNX_REQUIRE((long long)CHUNK * decay_ld < (1ll << 31), "memory_chunks: rows too long");
   TNX_REQUIRE(heads > 0 && groups > 0 && heads % groups == 0 && n > 0 && v > 0 && n <= 256, "memory_chunks: bad sizes");
   TNX_REQUIRE(chunk_size == CHUNK, "memory_chunks: chunks of %d tokens, the kernels take %d", chunk_size, CHUNK);
   TNX_REQUIRE(q_at >= 0 && k_at >= 0 && v_at >= 0 && ld >= q_at + groups * n && ld >= k_at + groups * n && ld >= v_at + heads * v,
@@ -1093,36 +1413,43 @@ extern "C" int tnx_memory_chunks(const float* u, int ld, int q_at, int k_at, int
               "memory_chunks: too many blocks");
   TNX_REQUIRE((long long)CHUNK * ld < (1ll << 31) && (long long)CHUNK * heads * v < (1ll << 31), "memory_chunks: rows too long");
   const int nb = n <= 32 ? 2 : n <= 64 ? 4 : n <= 128 ? 8 : 16, vb = (v + 15) / 16;
-  ChunkArgs a{u, ld, q_at, k_at, v_at, log_decay, write, run_start, cached, slots, chunk_run, chunk_begin, chunks, long_run,
-              long_first, num_long, memory, out, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, heads, groups, n, v};
+  ChunkArgs a{u, ld, q_at, k_at, v_at, log_decay, decay_ld, write, run_start, cached, slots, chunk_run, chunk_begin, chunks,
+              long_run, long_first, num_long, memory, out, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, heads,
+              groups, n, v};
   const size_t of_group = (size_t)chunks * groups, of_head = (size_t)chunks * heads;
   float* at = room;
   a.qx = at, at += of_group * 4 * nb * TILE;
   a.kx = at, at += of_group * 4 * nb * TILE;
   a.pairs = at, at += of_head * 16 * TILE;
   a.gates = at, at += of_head * 3 * CHUNK;
-  if (delta) {
+  if (mode == KEYED) a.keep = at, at += of_head * 16 * nb;
+  if (mode == DELTA_RULE) {
     a.wx = at, at += of_head * 4 * nb * TILE;
     a.ux = at, at += of_head * vb * 4 * TILE;
   }
   TNX_REQUIRE(room && (uintptr_t)room % 16 == 0 && at - room <= room_size, "memory_chunks: %lld floats of room, %lld needed",
               room_size, (long long)(at - room));
   const bool aligned = n % 4 == 0 && ((ld | q_at | k_at) & 3) == 0 && (uintptr_t)u % 16 == 0;
-  if (delta) return aligned ? launch_chunks_sized<true, true>(a, nb, stream) : launch_chunks_sized<true, false>(a, nb, stream);
-  return aligned ? launch_chunks_sized<false, true>(a, nb, stream) : launch_chunks_sized<false, false>(a, nb, stream);
+  if (mode == DELTA_RULE)
+    return aligned ? launch_chunks_sized<DELTA_RULE, true>(a, nb, stream) : launch_chunks_sized<DELTA_RULE, false>(a, nb, stream);
+  if (mode == KEYED)
+    return aligned ? launch_chunks_sized<KEYED, true>(a, nb, stream) : launch_chunks_sized<KEYED, false>(a, nb, stream);
+  return aligned ? launch_chunks_sized<PLAIN, true>(a, nb, stream) : launch_chunks_sized<PLAIN, false>(a, nb, stream);
 }
 
 extern "C" int tnx_gated_norm(const float* o, const float* gate, long long gate_ld, const float* weight, float eps, int parts,
                               int gate_first, const float* skip, int skip_heads, const float* x, long long x_ld, void* out,
-                              int dtype, int tokens, int width, hipStream_t stream) {
-  TNX_REQUIRE(tokens >= 0 && width > 0 && parts > 0 && width % parts == 0 && gate_ld >= width, "gated_norm: bad sizes");
+                              long long out_ld, float out_scale, int dtype, int tokens, int width, hipStream_t stream) {
+  TNX_REQUIRE(tokens >= 0 && width > 0 && parts > 0 && width % parts == 0 && gate_ld >= width && out_ld >= width,
+              "gated_norm: bad sizes");
   TNX_REQUIRE(!skip || (skip_heads > 0 && width % skip_heads == 0 && x && x_ld >= width), "gated_norm: bad skip");
   TNX_REQUIRE(dtype == TNX_F32 || dtype == TNX_BF16, "gated_norm: dtype %d", dtype);
   TNX_REQUIRE((long long)tokens * parts < (1ll << 31), "gated_norm: too many rows");
   if (tokens == 0) return 0;
-  FinishArgs a{o, gate, gate_ld, weight, eps, parts, gate_first, skip, x, x_ld, skip ? width / skip_heads : 1, out, tokens, width};
+  FinishArgs a{o, gate, gate_ld, weight, eps, parts, gate_first, skip, x, x_ld, skip ? width / skip_heads : 1, out, out_ld, out_scale,
+               tokens, width};
   const bool aligned = (width / parts) % 4 == 0 && gate_ld % 4 == 0 && (uintptr_t)gate % 16 == 0 && (uintptr_t)o % 16 == 0 &&
-                       (uintptr_t)weight % 16 == 0 && (uintptr_t)out % 16 == 0 &&
+                       (uintptr_t)weight % 16 == 0 && (uintptr_t)out % (dtype == TNX_F32 ? 16 : 8) == 0 && out_ld % 4 == 0 &&
                        (!skip || (x_ld % 4 == 0 && a.per_head % 4 == 0 && (uintptr_t)x % 16 == 0));
   if (dtype == TNX_F32) {
     if (aligned)

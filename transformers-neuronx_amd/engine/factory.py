@@ -54,7 +54,9 @@ def _room_for_weight_copies(cfg: EngineConfig, model: DecoderModel, bytes_per_pa
         return False
     if cfg.weight_copy_bytes is not None:
         return "later"
-    matrices = sum(2 * int(torch.Size(d.shape).numel()) for d in model.param_decls() if d.role in ("matrix", "table"))
+    # (matrices of which only the checkpoint knows a size are small ones, and are not counted)
+    matrices = sum(2 * int(torch.Size(d.shape).numel()) for d in model.param_decls()
+                   if d.role in ("matrix", "table") and None not in d.shape)
     _, total = torch.cuda.mem_get_info(device)
     return True if 2.2 * matrices + _cache_bytes(cfg, bytes_per_page, total) <= 0.9 * total else "later"
 

@@ -142,7 +142,8 @@ _SIGNATURES = {
                       _c_int, _c_int, _c_void_p],
         "tnx_expert_mixture": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                                _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                               _c_int, _c_int, _c_float, _c_int, _c_void_p],
+                               _c_int, _c_int, _c_float, _c_int, _c_int, _c_void_p],
+        "tnx_row_activation": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_ll, _c_void_p],
         "tnx_gated_activation": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_float, _c_void_p],
         "tnx_expert_order": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                              _c_void_p, _c_void_p],
@@ -178,13 +179,16 @@ _SIGNATURES = {
         "tnx_memory_inputs": [_c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p,
                               _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_float, _c_void_p, _c_int, _c_int,
                               _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p],
-        "tnx_memory_walk": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
+        "tnx_channel_decays": [_c_void_p, _c_ll, _c_void_p, _c_int, _c_void_p, _c_float, _c_void_p, _c_int, _c_int, _c_int,
+                               _c_void_p],
+        "tnx_turn_heads": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_int, _c_int, _c_void_p, _c_int, _c_void_p],
+        "tnx_memory_walk": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                             _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
-        "tnx_memory_chunks": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
+        "tnx_memory_chunks": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p,
                               _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_int, _c_void_p,
                               _c_void_p, _c_void_p, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
         "tnx_gated_norm": [_c_void_p, _c_void_p, _c_ll, _c_void_p, _c_float, _c_int, _c_int, _c_void_p, _c_int, _c_void_p,
-                           _c_ll, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
+                           _c_ll, _c_void_p, _c_ll, _c_float, _c_int, _c_int, _c_int, _c_void_p],
     },
     "probe": {
         "tnx_probe_stream_read": [_c_void_p, ctypes.c_size_t, _c_void_p, _c_int, _c_void_p],
@@ -1763,18 +1767,47 @@ class HipOps:
                    work=(f"{t}x{channels}", t * channels * 8.0 + ctx.num_requests * (taps - 1) * channels * 8.0, 0.0))
         return u, gates[0], gates[1]
 
+    def channel_decays(self, low, weight, bias, tau):
+        """See `ReferenceOps.channel_decays`."""
+        t, rank = low.shape
+        channels = weight.shape[0]
+        low_ld = self._rows_apart(low, "the small projection", torch.float32, t, rank)
+        _want(weight, "decay matrix", None, (channels, rank))
+        _want(bias, "decay bias", torch.float32, (channels,))
+        out = torch.empty(t, channels, dtype=torch.float32, device=low.device)
+        self._call("linear_memory", "tnx_channel_decays", _ptr(low), low_ld, _ptr(weight), _code(weight.dtype), _ptr(bias),
+                   1.0 / float(tau), _ptr(out), t, channels, rank, _stream(),
+                   work=(f"{t}x{channels}", t * channels * 4.0 + channels * rank * weight.element_size(), 2.0 * t * channels * rank))
+        return out
+
+    def turn_heads(self, x, at, heads, n, freqs, interleaved, ctx):
+        """See `ReferenceOps.turn_heads`."""
+        _want(x, "projections", torch.float32)
+        _want(freqs, "frequencies", torch.float32)
+        if x.dim() != 2 or x.shape[0] != ctx.num_tokens or at < 0 or x.shape[1] < at + heads * n:
+            raise ValueError(f"projections must be [{ctx.num_tokens}, {at + heads * n} or more], got {tuple(x.shape)}")
+        self._call("linear_memory", "tnx_turn_heads", _ptr(x), x.shape[1], int(at), int(heads), int(n), _ptr(freqs), freqs.numel(),
+                   int(bool(interleaved)), _ptr(ctx.positions), x.shape[0], _stream(),
+                   work=(f"{x.shape[0]}x{heads}", x.shape[0] * heads * 2.0 * freqs.numel() * 8, 0.0))
+        return x
+
     def linear_memory(self, u, q_at, k_at, v_at, heads, groups, n, v, log_decay, write, ctx, memory, delta):
         """See `ReferenceOps.linear_memory`."""
         t = ctx.num_tokens
         u_ld = self._rows_apart(u, "queries, keys and values", torch.float32, t, 2 * groups * n + heads * v)
         if min(q_at, k_at, v_at) < 0 or max(q_at + groups * n, k_at + groups * n, v_at + heads * v) > u.shape[1]:
             raise ValueError(f"queries, keys and values at columns {q_at}, {k_at}, {v_at} of {u.shape[1]}")
-        _want(log_decay, "decays", torch.float32, (t, heads))
-        _want(write, "write weights", torch.float32, (t, heads))
+        keyed = (log_decay.dim() == 2 and log_decay.shape[1] == heads * n and write is None and not delta
+                 and groups == heads)
+        _want(log_decay, "decays", torch.float32, (heads,) if log_decay.dim() == 1 else (t, heads * n if keyed else heads))
+        decay_ld = 0 if log_decay.dim() == 1 else log_decay.shape[1]
+        mode = 2 if keyed else int(bool(delta))
+        if write is not None:
+            _want(write, "write weights", torch.float32, (t, heads))
         _want(memory, "memory", torch.float32, (memory.shape[0], 2, heads, v, n))
         out = torch.empty(t, heads * v, dtype=torch.float32, device=u.device)
         state = float(ctx.num_requests) * heads * n * v * 8
-        work = (f"{t} tokens {ctx.num_requests} runs", state + t * (u.shape[1] + heads * v) * 4.0,
+        work = (f"{t} tokens {ctx.num_requests} runs", state + t * (u.shape[1] + heads * v + decay_ld) * 4.0,
                 (6.0 if delta else 4.0) * t * heads * n * v)
         by_chunks = ctx.plan.get("memory_long_run")
         longest = 0
@@ -1784,37 +1817,41 @@ class HipOps:
             chunk_run, first = ctx.plan["memory_chunk_run"], ctx.plan["memory_long_first"]
             chunks = chunk_run.numel()
             nb, vb = next(x for x in (2, 4, 8, 16) if n <= 16 * x), -(-v // 16)
-            size = chunks * (2 * groups * 1024 * nb + heads * (3 * 64 + 4096) + (heads * 1024 * (nb + vb) if delta else 0))
+            size = chunks * (2 * groups * 1024 * nb + heads * (3 * 64 + 4096) + (heads * 1024 * (nb + vb) if delta else 0)
+                             + (heads * 16 * nb if keyed else 0))
             room = torch.empty(size, dtype=torch.float32, device=u.device)
             self._call("linear_memory", "tnx_memory_chunks", _ptr(u), u_ld, int(q_at), int(k_at), int(v_at),
-                       _ptr(log_decay), _ptr(write), _ptr(ctx.run_start), _ptr(ctx.cached_lens), _ptr(ctx.slots),
+                       _ptr(log_decay), decay_ld, _ptr(write), _ptr(ctx.run_start), _ptr(ctx.cached_lens), _ptr(ctx.slots),
                        _ptr(chunk_run), _ptr(ctx.plan["memory_chunk_begin"]), chunks, MEMORY_CHUNK, _ptr(by_chunks), _ptr(first),
-                       by_chunks.numel(), _ptr(memory), _ptr(out), _ptr(room), size, heads, groups, n, v, int(bool(delta)), _stream(),
+                       by_chunks.numel(), _ptr(memory), _ptr(out), _ptr(room), size, heads, groups, n, v, mode, _stream(),
                        work=work)
             if by_chunks.numel() == ctx.num_requests:
                 return out
-        self._call("linear_memory", "tnx_memory_walk", _ptr(u), u_ld, int(q_at), int(k_at), int(v_at), _ptr(log_decay),
+        self._call("linear_memory", "tnx_memory_walk", _ptr(u), u_ld, int(q_at), int(k_at), int(v_at), _ptr(log_decay), decay_ld,
                    _ptr(write), _ptr(ctx.run_start), _ptr(ctx.cached_lens), _ptr(ctx.slots), _ptr(memory), _ptr(out), t,
-                   ctx.num_requests, heads, groups, n, v, int(bool(delta)), longest, _stream(), work=None if longest else work)
+                   ctx.num_requests, heads, groups, n, v, mode, longest, _stream(), work=None if longest else work)
         return out
 
     memory_by_chunks = True            # tests clear it: every run token by token
 
-    def gated_norm(self, o, gate, weight, eps, parts, gate_first, skip=None):
+    def gated_norm(self, o, gate, weight, eps, parts, gate_first, skip=None, out=None, out_scale=1.0):
         """See `ReferenceOps.gated_norm`."""
         _want(o, "the memory's result", torch.float32)
         t, width = o.shape
         gate_ld = self._rows_apart(gate, "the gate", torch.float32, t, width)
-        _want(weight, "norm weight", torch.float32, (width,))
+        if weight is not None:
+            _want(weight, "norm weight", torch.float32, (width,))
         factors, x, x_ld = None, None, 0
         if skip is not None:
             factors, x = skip
             _want(factors, "skip factors", torch.float32)
             x_ld = self._rows_apart(x, "the skipped input", torch.float32, t, width)
-        out = torch.empty(t, width, dtype=self.dtype, device=o.device)
+        if out is None:
+            out = torch.empty(t, width, dtype=self.dtype, device=o.device)
+        out_ld = self._rows_apart(out, "the result", self.dtype, t, width)
         self._call("linear_memory", "tnx_gated_norm", _ptr(o), _ptr(gate), gate_ld, _ptr(weight), float(eps), int(parts),
-                   int(bool(gate_first)), _ptr(factors), factors.numel() if factors is not None else 0, _ptr(x), x_ld, _ptr(out),
-                   _code(self.dtype), t, width, _stream(),
+                   int(bool(gate_first)), _ptr(factors), factors.numel() if factors is not None else 0, _ptr(x), x_ld, _ptr(out), out_ld,
+                   float(out_scale), _code(self.dtype), t, width, _stream(),
                    work=(f"{t}x{width}", t * width * (8.0 + (4 if skip is not None else 0) + out.element_size()), 0.0))
         return out
 
@@ -1849,6 +1886,16 @@ class HipOps:
                    work=(f"{t}x{two_f // 2}", t * two_f * 4.0 + out.numel() * out.element_size(), 0.0))
         return out
 
+    def row_activation(self, x, activation, row_gate=None):
+        """See `ReferenceOps.row_activation`."""
+        _want(x, "rows", torch.float32)
+        t, f = x.shape
+        gate_ld = self._rows_apart(row_gate, "the rows' gate", torch.float32, t, 1) if row_gate is not None else 0
+        out = torch.empty(t, f, dtype=self.dtype, device=x.device)
+        self._call("experts", "tnx_row_activation", _ptr(x), _ptr(out), _code(self.dtype), t, f, _ACT[activation], _ptr(row_gate),
+                   gate_ld, _stream(), work=(f"{t}x{f}", t * f * (4.0 + out.element_size()), 0.0))
+        return out
+
     # A step of this many (token, choice) pairs an expert or more, bfloat16, that is not being recorded: the host
     # reads where each expert's pairs begin (one small copy that waits for the device) and every expert's two
     # products go to the vendor library over its own rows, as the many-rows products of the other parts do. Below
@@ -1863,14 +1910,15 @@ class HipOps:
         what the device has made. `identity`: how many experts without tensors the numbers behind the experts' stand
         for."""
         t, top = chosen.shape
-        experts, two_f, width = w_gate_up.shape
-        f = two_f // 2
-        if activation not in _GATE_ACT or weight_on not in ("input", "output") or (identity and weight_on == "input"):
+        experts, rows_in, width = w_gate_up.shape
+        f = w_down.shape[2]
+        ungated = rows_in == f
+        if rows_in not in (f, 2 * f) or activation not in (_ACT if ungated else _GATE_ACT) or (ungated and weight_on == "input") or weight_on not in ("input", "output") or (identity and weight_on == "input"):
             raise ValueError(f"expert_mixture: activation {activation!r}, weight_on {weight_on!r}")
         _want(h, "h", w_gate_up.dtype, (t, width))
         _want(chosen, "chosen experts", torch.int32)
         _want(weights, "weights", torch.float32, (t, top))
-        _want(w_gate_up, "gate and up matrices")
+        _want(w_gate_up, "the experts' input matrices")
         _want(w_down, "down matrices", w_gate_up.dtype, (experts, width, f))
         if residual is not None:
             _want(residual, "residual", torch.float32, (t, width))
@@ -1902,7 +1950,8 @@ class HipOps:
                     continue
                 b = a + -(-(b - a) // step) * step
                 gu = self.linear(rows[a:b], w_gate_up[e], None, out_f32=True, f32_by_library=True)
-                inner = self.gated_activation(gu, activation, scale[a:b] if on_input else None, limit=limit)
+                inner = (self.row_activation(gu, activation) if ungated
+                         else self.gated_activation(gu, activation, scale[a:b] if on_input else None, limit=limit))
                 self.linear(inner, w_down[e], None, out_f32=True, f32_by_library=True, into=y[a:b])
             self._call("experts", "tnx_expert_combine", _ptr(y), _ptr(place), None if on_input else _ptr(weights),
                        _ptr(residual), _ptr(out), t, top, width, _ptr(h) if identity else None, _ptr(chosen), experts, _stream(),
@@ -1915,10 +1964,11 @@ class HipOps:
         used = min(experts, pairs)
         self._call("experts", "tnx_expert_mixture", _ptr(h), _ptr(chosen), _ptr(weights), _ptr(w_gate_up), _ptr(w_down),
                    _ptr(ints[:experts + 1]), _ptr(ints[experts + 1:]), _ptr(inner), _ptr(rows), _ptr(residual), _ptr(out),
-                   _code(h.dtype), t, experts, top, width, f, _GATE_ACT[activation], int(weight_on == "input"),
-                   int(bool(self.expert_plain_products)), float(limit or 0.0), int(identity), _stream(),
-                   work=(f"{t}x{top} of {experts}", used * 3.0 * f * width * item + t * width * (item + 8.0),
-                         6.0 * t * top * f * width))
+                   _code(h.dtype), t, experts, top, width, f, (_ACT if ungated else _GATE_ACT)[activation],
+                   int(weight_on == "input"), int(bool(self.expert_plain_products)), float(limit or 0.0), int(identity),
+                   int(ungated), _stream(),
+                   work=(f"{t}x{top} of {experts}", used * (2.0 if ungated else 3.0) * f * width * item + t * width * (item + 8.0),
+                         (4.0 if ungated else 6.0) * t * top * f * width))
         return out
 
     # ---------------------------------------------------------------- output end
