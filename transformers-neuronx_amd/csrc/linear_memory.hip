@@ -310,7 +310,8 @@ __device__ __forceinline__ float sum16(float x) {
 // lanes share a column (column 16 b + 4 w + lane / 16): lane % 16 holds its rows NR (lane % 16) + j, j < NR. CH tokens a
 // chunk go through LDS, the next chunk's loads under way meanwhile, a token's operands read a token ahead.
 // With DELTA S^T k, S^T q and k . q are summed side by side from the S that came in, and S'^T q = S^T q + w (k . q).
-// KEYED: a token's decays go through LDS as its keys do.
+// KEYED: a token's decays go through LDS as its keys do. Without DELTA S decays by S + S (e^g - 1): a factor just below one,
+// rounded to float32, would be off by the same amount at every token, and a memory of hundreds of tokens with it.
 template <int NR, int CH, int MODE, bool ALIGNED>
 __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column_blocks) {
   constexpr bool DELTA = MODE == DELTA_RULE;
@@ -319,9 +320,9 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
   constexpr int QN = (CH * PT + 255) / 256;               // pieces of queries (and keys) a thread and chunk
   __shared__ __attribute__((aligned(16))) float qs[CH * np];
   __shared__ __attribute__((aligned(16))) float ks[CH * np];
-  __shared__ __attribute__((aligned(16))) float ds[MODE == KEYED ? CH * np : 4];      // e^g, row by row of S
+  __shared__ __attribute__((aligned(16))) float ds[MODE == KEYED ? CH * np : 4];      // e^g - 1, row by row of S
   __shared__ __attribute__((aligned(16))) float vs[CH * 16];
-  __shared__ float kp[CH], wr[CH];                        // e^g, write
+  __shared__ float kp[CH], wr[CH];                        // e^g (DELTA) or e^g - 1, write
   const int cb = blockIdx.x % column_blocks, rh = blockIdx.x / column_blocks;
   const int r = rh / a.heads, head = rh - r * a.heads;
   const int group = head / (a.heads / a.groups);
@@ -372,7 +373,7 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
     if (threadIdx.x < CH) {
       const bool in = threadIdx.x < len;
       const size_t t = start + t0 + (in ? threadIdx.x : 0);
-      if (MODE != KEYED) rkeep = in ? expf(a.log_decay[t * a.decay_ld + head]) : 1.f;
+      if (MODE != KEYED) rkeep = in ? (DELTA ? expf(a.log_decay[t * a.decay_ld + head]) : expm1f(a.log_decay[t * a.decay_ld + head])) : 0.f;
       rwrite = in ? (a.write ? a.write[t * a.heads + head] : 1.f) : 0.f;
     }
   };
@@ -386,7 +387,7 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
         if (MODE == KEYED) {
           f32x4 e4;
 #pragma unroll
-          for (int e = 0; e < 4; ++e) e4[e] = expf(rd[MODE == KEYED ? u : 0][e]);
+          for (int e = 0; e < 4; ++e) e4[e] = expm1f(rd[MODE == KEYED ? u : 0][e]);
           *(f32x4*)(ds + 4 * f) = e4;
         }
       }
@@ -442,7 +443,7 @@ __global__ void __launch_bounds__(256) memory_walk_kernel(WalkArgs a, int column
         const float w = write * val;
 #pragma unroll
         for (int j = 0; j < NR; ++j) {
-          S[j] = (MODE == KEYED ? d[MODE == KEYED ? j : 0] : keep) * S[j] + k[j] * w;
+          S[j] = fmaf(k[j], w, fmaf(MODE == KEYED ? d[MODE == KEYED ? j : 0] : keep, S[j], S[j]));
           o += S[j] * q[j];
         }
         o = sum16(o);
