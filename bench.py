@@ -131,6 +131,22 @@ def gubulorn_config(width, heads, head, ff, vocab, layers):
                              mlp=dense if i % 4 in (0, 3) else moe) for i in range(layers)])
 
 
+def zudusun_config(width, heads, head, ff, vocab, layers, window=1024):
+    """config.json contents of a Zudusun model at the sizes of published layers: in turn attention (a quarter as many
+    key/value heads as query heads) beside gated linear attention (heads of 128 over values of 256, a bottleneck of 16),
+    windowed attention, and retention (heads of 256 over values of 512); eight experts of ff / 4 of which a token takes
+    two, beside a shared one of ff / 2."""
+    grouped = dict(heads=heads, kv_heads=max(1, heads // 4), dim=head, vdim=head, scale=head ** -0.5)
+    kinds = [("parallel", dict(left=grouped, right=dict(heads=width // 256, dim=128, vdim=256, tau=16.0, rank=16),
+                               left_scale=0.5, right_scale=0.5)),
+             ("attention", dict(grouped, mask=dict(size=window), rot=dict(base=10000.0, dims=head))),
+             ("retention", dict(heads=width // 256, dim=256, vdim=512, rot=dict(base=10000.0, dims=256),
+                                decay=[1.0 - 2.0 ** (-5 - 5.0 * i / (width // 256)) for i in range(width // 256)]))]
+    moe = dict(kind="moe", router=dict(experts=8, top=2), expert=dict(ff=ff // 4), shared=dict(ff=ff // 2))
+    return dict(architecture="Zudusun", vocab=vocab, width=width, norm=dict(eps=1e-6), init_std=0.02, max_positions=4096,
+                layers=[dict(type=kinds[i % 3][0], mixer=kinds[i % 3][1], mlp=moe) for i in range(layers)])
+
+
 # a new design beside the closest one the engine had, at equal sizes: {design: {size: (its config, the other's)}};
 # the other's is the name of an OPT preset, or (design, its config)
 BESIDE = {"ratesun": {
@@ -153,6 +169,11 @@ BESIDE = {"ratesun": {
     "2048 wide": (lambda n: gubulorn_config(2048, 32, 64, 8192, 50272, n),
                   ("sunatar", lambda n: sunatar_config(2048, 32, 64, 8192, 50272, n))),
     "4096 wide": (lambda n: gubulorn_config(4096, 32, 128, 16384, 50272, n),
+                  ("sunatar", lambda n: sunatar_config(4096, 32, 128, 16384, 50272, n))),
+}, "zudusun": {
+    "2048 wide": (lambda n: zudusun_config(2048, 32, 64, 8192, 50272, n),
+                  ("sunatar", lambda n: sunatar_config(2048, 32, 64, 8192, 50272, n))),
+    "4096 wide": (lambda n: zudusun_config(4096, 32, 128, 16384, 50272, n),
                   ("sunatar", lambda n: sunatar_config(4096, 32, 128, 16384, 50272, n))),
 }}
 PREFILL_TOKENS = 2048
