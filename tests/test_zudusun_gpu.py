@@ -369,7 +369,8 @@ def test_experts_without_gates_beside_a_shared_one_with_a_number(name, dtype, to
     clear = torch.ones(tokens, dtype=torch.bool) if top == experts else (ranked[:, top - 1] - ranked[:, top]) > 1e-4
     assert int(clear.sum()) >= max(1, tokens // 2)
     assert tokens < 30 or top == experts or P.route(z - wide["p.router.b"], top)[0].tolist() != chosen.tolist()   # the bias matters
-    got_chosen, got_weight = ops.route(ops.linear(h.to(DEV), part.w_router, part.b_router, out_f32=True)[:, :experts], top,
+    at = part.router_at
+    got_chosen, got_weight = ops.route(ops.linear(h.to(DEV), part.w_in, part.b_in, out_f32=True)[:, at:at + experts], top,
                                        "softmax", True)
     if top < experts:
         assert sorted(map(sorted, got_chosen.cpu()[clear].tolist())) == sorted(map(sorted, chosen[clear].tolist()))
@@ -392,6 +393,10 @@ def test_an_activation_with_a_gate_number_a_row(name, dtype, tol, t, f):
     want = P.squared_relu(x.double())
     _close(ops.row_activation(x.to(DEV), "relu2"), want, tol)
     _close(ops.row_activation(x.to(DEV), "relu2", rows.to(DEV)[:, 4:5]), want * P.sigmoid(rows[:, 4:5].double()), tol)
+    for at, more in ((4, 8), (3, 5)):          # rows that lie apart, at places of a multiple of four elements and not
+        wide = torch.full((t, at + f + more), 9.0)
+        wide[:, at:at + f] = x
+        _close(ops.row_activation(wide.to(DEV)[:, at:at + f], "relu2"), want, tol)
 
 
 # ---------------------------------------------------------------- the engine

@@ -383,33 +383,23 @@ __global__ void gated_activation_kernel(const float* __restrict__ gu, T* __restr
   }
 }
 
-// act(x) from rows of float32, times sigmoid(row_gate) of the row
-template <typename T>
-__global__ void row_activation_kernel(const float* __restrict__ x, T* __restrict__ out, int f, int act, size_t total,
-                                      const float* __restrict__ row_gate, long long gate_ld) {
+// act(x) from rows of float32 (`ld` apart), times sigmoid(row_gate) of the row; V neighbours a thread (V = 4: rows and
+// places of a multiple of four elements)
+template <typename T, int V>
+__global__ void row_activation_kernel(const float* __restrict__ x, long long ld, T* __restrict__ out, int pieces, int act,
+                                      size_t total, const float* __restrict__ row_gate, long long gate_ld) {
+  typedef float fv __attribute__((ext_vector_type(V)));
+  typedef T tv __attribute__((ext_vector_type(V)));
   size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   const size_t stride = (size_t)gridDim.x * blockDim.x;
   for (; i < total; i += stride) {
-    float y = apply_act(x[i], act);
-    if (row_gate) y *= 1.f / (1.f + expf(-row_gate[i / f * gate_ld]));
-    out[i] = from_f32<T>(y);
-  }
-}
-
-// the same, four neighbours a thread (rows of a multiple of four elements)
-template <typename T>
-__global__ void row_activation_four_kernel(const f32x4* __restrict__ x, T* __restrict__ out, int f4, int act, size_t total,
-                                           const float* __restrict__ row_gate, long long gate_ld) {
-  typedef T four __attribute__((ext_vector_type(4)));
-  size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
-  const size_t stride = (size_t)gridDim.x * blockDim.x;
-  for (; i < total; i += stride) {
-    const f32x4 v = x[i];
-    const float w = row_gate ? 1.f / (1.f + expf(-row_gate[i / f4 * gate_ld])) : 1.f;
-    four o;
+    const size_t t = i / pieces, c = i - t * pieces;
+    const fv v = *(const fv*)(x + t * ld + V * c);
+    const float w = row_gate ? 1.f / (1.f + expf(-row_gate[t * gate_ld])) : 1.f;
+    tv o;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) o[e] = from_f32<T>(apply_act(v[e], act) * w);
-    ((four*)out)[i] = o;
+    for (int e = 0; e < V; ++e) o[e] = from_f32<T>(apply_act(v[e], act) * w);
+    ((tv*)out)[i] = o;
   }
 }
 
@@ -508,24 +498,24 @@ extern "C" int tnx_gated_activation(const float* gate_up, void* out, int dtype, 
   return 0;
 }
 
-// act(x) of float32 rows, times sigmoid(row_gate) of its row (rows `gate_ld` apart) or not
-extern "C" int tnx_row_activation(const float* x, void* out, int dtype, int tokens, int f, int act, const float* row_gate,
-                                  long long gate_ld, hipStream_t stream) {
-  TNX_REQUIRE(tokens >= 0 && f > 0 && gate_ld >= 0, "row_activation: bad sizes");
+// act(x) of float32 rows (`ld` apart), times sigmoid(row_gate) of its row (numbers `gate_ld` apart) or not
+extern "C" int tnx_row_activation(const float* x, long long ld, void* out, int dtype, int tokens, int f, int act,
+                                  const float* row_gate, long long gate_ld, hipStream_t stream) {
+  TNX_REQUIRE(tokens >= 0 && f > 0 && ld >= f && gate_ld >= 0, "row_activation: bad sizes");
   TNX_REQUIRE(dtype == TNX_F32 || dtype == TNX_BF16, "row_activation: dtype %d", dtype);
   if (tokens == 0) return 0;
   const size_t total = (size_t)tokens * f;
-  if (f % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)out % (dtype == TNX_F32 ? 16 : 8) == 0) {
-    const size_t fours = total / 4;
-    if (dtype == TNX_F32)
-      row_activation_four_kernel<float><<<blocks_for(fours), 256, 0, stream>>>((const f32x4*)x, (float*)out, f / 4, act, fours, row_gate, gate_ld);
-    else
-      row_activation_four_kernel<bf16_t><<<blocks_for(fours), 256, 0, stream>>>((const f32x4*)x, (bf16_t*)out, f / 4, act, fours, row_gate, gate_ld);
-  } else if (dtype == TNX_F32) {
-    row_activation_kernel<float><<<blocks_for(total), 256, 0, stream>>>(x, (float*)out, f, act, total, row_gate, gate_ld);
+  const bool fours = f % 4 == 0 && ld % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)out % (dtype == TNX_F32 ? 16 : 8) == 0;
+#define ROWS_LAUNCH(T, V) \
+  row_activation_kernel<T, V><<<blocks_for(total / V), 256, 0, stream>>>(x, ld, (T*)out, f / V, act, total / V, row_gate, gate_ld)
+  if (dtype == TNX_F32) {
+    if (fours) ROWS_LAUNCH(float, 4);
+    else ROWS_LAUNCH(float, 1);
   } else {
-    row_activation_kernel<bf16_t><<<blocks_for(total), 256, 0, stream>>>(x, (bf16_t*)out, f, act, total, row_gate, gate_ld);
+    if (fours) ROWS_LAUNCH(bf16_t, 4);
+    else ROWS_LAUNCH(bf16_t, 1);
   }
+#undef ROWS_LAUNCH
   TNX_CHECK_LAUNCH("row_activation");
   return 0;
 }

@@ -143,7 +143,7 @@ _SIGNATURES = {
         "tnx_expert_mixture": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                                _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
                                _c_int, _c_int, _c_float, _c_int, _c_int, _c_void_p],
-        "tnx_row_activation": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_ll, _c_void_p],
+        "tnx_row_activation": [_c_void_p, _c_ll, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_ll, _c_void_p],
         "tnx_gated_activation": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_float, _c_void_p],
         "tnx_expert_order": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                              _c_void_p, _c_void_p],
@@ -1476,10 +1476,9 @@ class HipOps:
         need = max(need, (need if values_at is None else int(values_at)) + num_kv * value_size)
         if head_scale is not None:
             _want(head_scale, "head scales", torch.float32, (num_heads,))
-        _want(proj, "projections", torch.float32)
         if proj.dim() != 2 or proj.shape[0] != t or proj.shape[1] < need:
             raise ValueError(f"projections must be [{t}, {need} or more], got {tuple(proj.shape)}")
-        total = proj.shape[1]
+        total = self._rows_apart(proj, "projections", torch.float32, t, proj.shape[1])
         if q_weight is not None:
             _want(q_weight, "query norm", torch.float32, (num_heads * head_size,))
             _want(k_weight, "key norm", torch.float32, (num_kv * head_size,))
@@ -1505,7 +1504,7 @@ class HipOps:
                    value_size, cache_head, int(bool(per_head)), -1 if values_at is None else int(values_at),
                    _ptr(head_scale), float(temperature[0]) if temperature else 0.0, int(temperature[1]) if temperature else 0,
                    _stream(),
-                   work=(f"{t}x{total}", t * (total * 4 + (num_heads + 2 * num_kv) * cache_head * q.element_size()), 0.0))
+                   work=(f"{t}x{need}", t * (need * 4 + (num_heads + 2 * num_kv) * cache_head * q.element_size()), 0.0))
         return q
 
     # ---------------------------------------------------------------- several copies of the stream
@@ -1782,11 +1781,11 @@ class HipOps:
 
     def turn_heads(self, x, at, heads, n, freqs, interleaved, ctx):
         """See `ReferenceOps.turn_heads`."""
-        _want(x, "projections", torch.float32)
         _want(freqs, "frequencies", torch.float32)
         if x.dim() != 2 or x.shape[0] != ctx.num_tokens or at < 0 or x.shape[1] < at + heads * n:
             raise ValueError(f"projections must be [{ctx.num_tokens}, {at + heads * n} or more], got {tuple(x.shape)}")
-        self._call("linear_memory", "tnx_turn_heads", _ptr(x), x.shape[1], int(at), int(heads), int(n), _ptr(freqs), freqs.numel(),
+        ld = self._rows_apart(x, "projections", torch.float32, x.shape[0], x.shape[1])
+        self._call("linear_memory", "tnx_turn_heads", _ptr(x), ld, int(at), int(heads), int(n), _ptr(freqs), freqs.numel(),
                    int(bool(interleaved)), _ptr(ctx.positions), x.shape[0], _stream(),
                    work=(f"{x.shape[0]}x{heads}", x.shape[0] * heads * 2.0 * freqs.numel() * 8, 0.0))
         return x
@@ -1888,11 +1887,11 @@ class HipOps:
 
     def row_activation(self, x, activation, row_gate=None):
         """See `ReferenceOps.row_activation`."""
-        _want(x, "rows", torch.float32)
         t, f = x.shape
+        ld = self._rows_apart(x, "rows", torch.float32, t, f)
         gate_ld = self._rows_apart(row_gate, "the rows' gate", torch.float32, t, 1) if row_gate is not None else 0
         out = torch.empty(t, f, dtype=self.dtype, device=x.device)
-        self._call("experts", "tnx_row_activation", _ptr(x), _ptr(out), _code(self.dtype), t, f, _ACT[activation], _ptr(row_gate),
+        self._call("experts", "tnx_row_activation", _ptr(x), ld, _ptr(out), _code(self.dtype), t, f, _ACT[activation], _ptr(row_gate),
                    gate_ld, _stream(), work=(f"{t}x{f}", t * f * (4.0 + out.element_size()), 0.0))
         return out
 

@@ -95,6 +95,52 @@ class Part:
         return 2.0 * count
 
 
+class OffersRows:
+    """For a part whose products with `h` are one product with a float32 result: an arrangement in which several parts
+    read the same `h` can make theirs one product. Such an arrangement sets `defer_in` before the part loads its tensors,
+    fetches the part's matrix and bias afterwards (`in_matrix`; the part then keeps none of its own) and hands the part
+    its columns of the result (`rows`, float32 `[T, the matrix's rows]`, rows may lie apart)."""
+
+    offers_rows = True
+    defer_in = False
+
+    def _keep_in(self, ops, w, bias=None) -> None:
+        self.in_raw = (w, bias)
+        if not self.defer_in:
+            self.w_in, self.b_in = ops.prepare_weight(w), bias
+            self.in_raw = None
+
+    def in_matrix(self):
+        raw, self.in_raw = self.in_raw, None
+        return raw
+
+    def _rows(self, h, rows):
+        return rows if rows is not None else self.ops.linear(h, self.w_in, self.b_in, out_f32=True, f32_by_library=True)
+
+
+def joined_rows(parts):
+    """The input matrices of `parts` (`OffersRows`) one under the other, each filled up with zero rows to a multiple of 16,
+    and by 64 rows more at the end where the product's rows would lie a power of two of bytes apart (what all tokens of a
+    prompt read at one time would share few memory channels); their biases likewise, or None where no part has one; and a
+    part's first and last row each."""
+    import torch
+    pad = torch.nn.functional.pad
+    raws, places, at = [part.in_matrix() for part in parts], [], 0
+    for w, _ in raws:
+        places.append((at, at + w.shape[0]))
+        at += w.shape[0] + -w.shape[0] % 16
+    total = at + (64 if at % 1024 == 0 else 0)
+    ends = [place[0] for place in places[1:]] + [total]
+    w = torch.cat([pad(w, (0, 0, 0, end - begin - w.shape[0])) for (w, _), (begin, _), end in zip(raws, places, ends)], dim=0)
+    bias = None
+    if any(b is not None for _, b in raws):
+        bias = torch.zeros(total, dtype=torch.float32, device=w.device)
+        for (_, b), (begin, end) in zip(raws, places):
+            if b is not None:
+                bias[begin:end] = b
+    return w.contiguous(), bias, places
+
+
 class Mixer(Part):
     """Mixes information between the tokens of a request.
 

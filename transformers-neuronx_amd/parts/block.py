@@ -1,6 +1,6 @@
 """Arrangements of a layer's parts around the residual stream."""
 from .. import debug
-from .base import Block, Stream, register_block
+from .base import Block, Stream, joined_rows, register_block
 
 
 @register_block("pre_norm")
@@ -78,14 +78,31 @@ class PostNormBlock(Block):
 @register_block("parallel")
 class ParallelBlock(Block):
     """`h = norm(x)`, `x = x + mixer(h) + feed_forward(h)`: one norm, and both parts read its output. The sum
-    is float32: the mixer's last product adds the stream, the feed-forward's adds that."""
+    is float32: the mixer's last product adds the stream, the feed-forward's adds that. With `one_product` the products
+    of both parts with h are one, where both offer their rows (`OffersRows`)."""
 
     recordable = True
 
+    def __init__(self, mixer, feed_forward, mixer_norm, feed_forward_norm, *, one_product: bool = False):
+        super().__init__(mixer, feed_forward, mixer_norm, feed_forward_norm)
+        self.joins = bool(one_product and getattr(mixer, "offers_rows", False) and getattr(feed_forward, "offers_rows", False))
+        if self.joins:
+            mixer.defer_in = feed_forward.defer_in = True
+
+    def load(self, tensors, prefix, ops, dtype) -> None:
+        super().load(tensors, prefix, ops, dtype)
+        if self.joins:
+            w, self.b_in, self.places = joined_rows((self.mixer, self.feed_forward))
+            self.w_in = ops.prepare_weight(w)
+
     def forward(self, stream: Stream, ctx, cache) -> Stream:
         h = self.mixer_norm.forward(stream.x, False, True)[1]
-        x = debug.tap("after_mixer", self.mixer.forward(h, ctx, cache, stream.x))
-        return Stream(self.feed_forward.forward(h, ctx, x), None)
+        mine, theirs = {}, {}
+        if self.joins:
+            both = self.ops.linear(h, self.w_in, self.b_in, out_f32=True, f32_by_library=True)
+            mine, theirs = ({"rows": both[:, a:b]} for a, b in self.places)
+        x = debug.tap("after_mixer", self.mixer.forward(h, ctx, cache, stream.x, **mine))
+        return Stream(self.feed_forward.forward(h, ctx, x, **theirs), None)
 
 
 @register_block("sandwich")

@@ -1,7 +1,7 @@
 """Feed-forward parts."""
 from typing import Dict, List
 
-from .base import FeedForward, register_feed_forward
+from .base import FeedForward, OffersRows, register_feed_forward
 from .spec import ParamDecl
 
 
@@ -110,7 +110,7 @@ class NoFeedForward(FeedForward):
 
 
 @register_feed_forward("mixture")
-class ExpertMixture(FeedForward):
+class ExpertMixture(OffersRows, FeedForward):
     """A mixture of experts, of which a token takes `top`, and optionally one more that every token takes.
 
     Router: z = W_r h in float32, scores s = sigmoid(z) (`score="sigmoid"`) or softmax(z) (`"softmax"`); a token's
@@ -132,8 +132,9 @@ class ExpertMixture(FeedForward):
 
     `gated=False` with `activation="relu2"`: experts (and the shared one) without a gate, W_down (act(W_up x)), the weight
     on the output; `names` are then two. `router_bias_name`: a bias of the router's logits. `shared_gate_name`: a matrix of
-    one row w_s under the shared expert's prefix, whose output is multiplied by sigmoid(w_s h); its row rides in the
-    router's product, and the factor enters where the shared expert's inner values are rounded."""
+    one row w_s under the shared expert's prefix, whose output is multiplied by sigmoid(w_s h); the factor enters where the
+    shared expert's inner values are rounded. The router's rows, w_s and the shared expert's up matrix are then one
+    product."""
 
     recordable = True
 
@@ -210,25 +211,25 @@ class ExpertMixture(FeedForward):
         # an expert's gate rows, then its up rows: `[experts, 2 inner, width]`; the down matrices `[experts, width, inner]`
         self.w_gate_up = torch.stack([torch.cat([tensors[f"{p}{n}{s}"] for n in ins], dim=0) for p in each]).contiguous()
         self.w_down = torch.stack([tensors[f"{p}{d}{s}"] for p in each]).contiguous()
-        # one product for the router's rows and, behind them, the row of the shared expert's gate. Such rows (and those of a
-        # router with experts that have no tensors) are rarely a multiple of eight: zero rows behind them let the product
-        # of many rows go to the vendor library all the same
+        # with experts that have no tensors the router's rows are rarely a multiple of eight: zero rows behind them let the
+        # product of many rows go to the vendor library all the same. Without gates the product holds, one under the other,
+        # the rows of the shared expert's up matrix, of the router, of the shared expert's gate, and zeros to a multiple of 16
         router = tensors[f"{prefix}{self.router_name}{s}"]
-        rows = self.routed
-        if self.shared_gate_name:
-            router = torch.cat([router, tensors[f"{prefix}{self.shared_name}{self.shared_gate_name}{s}"].to(router.dtype)], dim=0)
-            rows += 1
-        fill = (-rows % 16 if self.shared_gate_name else -rows % 8) if self.identity or self.shared_gate_name else 0
-        router = torch.nn.functional.pad(router, (0, 0, 0, fill)).contiguous() if fill else router.contiguous()
-        self.w_router = ops.prepare_weight(router)
-        self.b_router = None
-        if self.router_bias_name:
-            bias = tensors[f"{prefix}{self.router_bias_name}"]
-            self.b_router = torch.nn.functional.pad(bias, (0, router.shape[0] - bias.numel())).contiguous()
+        bias = tensors[f"{prefix}{self.router_bias_name}"] if self.router_bias_name else None
+        p = prefix + self.shared_name
+        before = [] if self.gated or not self.shared_inner else [tensors[f"{p}{ins[0]}{s}"]]
+        behind = [tensors[f"{p}{self.shared_gate_name}{s}"].to(router.dtype)] if self.shared_gate_name else []
+        self.router_at = sum(m.shape[0] for m in before)
+        rows = torch.cat(before + [router] + behind, dim=0)
+        fill = (-rows.shape[0] % 16 if not self.gated else -rows.shape[0] % 8 if self.identity else 0)
+        rows = torch.nn.functional.pad(rows, (0, 0, 0, fill)).contiguous()
+        if bias is not None:
+            bias = torch.nn.functional.pad(bias, (self.router_at, rows.shape[0] - self.router_at - bias.numel())).contiguous()
+        self._keep_in(ops, rows, bias)
         self.correction = tensors[f"{prefix}{self.correction_name}"] if self.correction_name else None
         if self.shared_inner:
-            p = prefix + self.shared_name
-            self.w_shared_in = ops.prepare_weight(torch.cat([tensors[f"{p}{n}{s}"] for n in ins], dim=0).contiguous())
+            if self.gated:
+                self.w_shared_in = ops.prepare_weight(torch.cat([tensors[f"{p}{n}{s}"] for n in ins], dim=0).contiguous())
             self.w_shared_down = ops.prepare_weight(tensors[f"{p}{d}{s}"])
 
     def flops_per_token(self, keys: float = 0.0) -> float:
@@ -236,10 +237,18 @@ class ExpertMixture(FeedForward):
         return 2.0 * self.width * (self.routed + each * self.top * self.inner * self.experts / self.routed
                                    + each * self.shared_inner + (1 if self.shared_gate_name else 0))
 
-    def forward(self, h, ctx, residual):
+    @property
+    def w_router(self):
+        return self.w_in
+
+    @property
+    def offers_rows(self) -> bool:
+        return not self.gated
+
+    def forward(self, h, ctx, residual, rows=None):
         ops = self.ops
-        rows = ops.linear(h, self.w_router, self.b_router, out_f32=True, f32_by_library=True)
-        z = rows[:, :self.routed]
+        rows = self._rows(h, rows)
+        z = rows[:, self.router_at:self.router_at + self.routed]
         more = {}
         if self.correction is not None or self.route_scale != 1.0:
             more = dict(correction=self.correction, scale=self.route_scale)
@@ -255,10 +264,11 @@ class ExpertMixture(FeedForward):
         if not self.shared_inner:
             return x
         limit = dict(limit=self.shared_limit) if self.shared_limit is not None else {}
-        up = ops.linear(h, self.w_shared_in, None, out_f32=True, f32_by_library=True)
         if self.gated:
-            inner = ops.gated_activation(up, self.activation, **limit)
+            inner = ops.gated_activation(ops.linear(h, self.w_shared_in, None, out_f32=True, f32_by_library=True),
+                                         self.activation, **limit)
         else:
-            inner = ops.row_activation(up, self.activation,
-                                       rows[:, self.routed:self.routed + 1] if self.shared_gate_name else None)
+            gate_at = self.router_at + self.routed
+            inner = ops.row_activation(rows[:, :self.shared_inner], self.activation,
+                                       rows[:, gate_at:gate_at + 1] if self.shared_gate_name else None)
         return ops.linear(inner, self.w_shared_down, None, residual=x, out_f32=True)

@@ -4,7 +4,7 @@ from typing import Dict, List, Optional
 
 import torch
 
-from .base import POSITIONS, CacheNeed, Mixer, register_mixer
+from .base import POSITIONS, CacheNeed, Mixer, OffersRows, register_mixer
 from .spec import ParamDecl
 
 
@@ -31,7 +31,7 @@ def bias_by_distance(table: torch.Tensor, max_distance: int) -> torch.Tensor:
 
 
 @register_mixer("attention")
-class Attention(Mixer):
+class Attention(OffersRows, Mixer):
     """Softmax attention over a paged key/value cache.
 
     `Q = (h Wq^T + bq) * scale`, keys and values of the step's tokens are stored
@@ -197,9 +197,8 @@ class Attention(Mixer):
                + ([self.out_gate] if self.out_gate else []))
         # One fused projection: a plain concatenation of the rows (the reference's
         # fused form interleaves per tensor-parallel shard, utils.py:189-242).
-        self.w_qkv = ops.prepare_weight(torch.cat([tensors[f"{prefix}{n}{ws}"] for n in ins], dim=0).contiguous())
-        self.b_qkv = (torch.cat([tensors[f"{prefix}{n}{bs}"] for n in ins], dim=0).contiguous()
-                      if self.has_bias else None)
+        self._keep_in(ops, torch.cat([tensors[f"{prefix}{n}{ws}"] for n in ins], dim=0).contiguous(),
+                      torch.cat([tensors[f"{prefix}{n}{bs}"] for n in ins], dim=0).contiguous() if self.has_bias else None)
         w_out = tensors[f"{prefix}{on}{ws}"]
         if self.cache_head != self.value_size:
             # the attention's result has heads of the cache's size: the columns that meet the filling are zeros
@@ -237,7 +236,15 @@ class Attention(Mixer):
             self.mix_weight = tensors[f"{prefix}{self.value_mix['name']}"].reshape(1)
 
     def first_weight(self):
-        return None if self.prepared else self.w_qkv
+        return None if self.prepared else self.w_in
+
+    @property
+    def w_qkv(self):
+        return self.w_in
+
+    @property
+    def offers_rows(self) -> bool:
+        return self.prepared            # (the other route's product applies and stores more than a product does)
 
     def step_planners(self):
         from ..kernels.attention_plan import attention_plan
@@ -264,21 +271,21 @@ class Attention(Mixer):
         w, self.w_out_raw = self.w_out_raw, None
         return w
 
-    def inner_into(self, h, ctx, cache, out, scale: float) -> None:
+    def inner_into(self, h, ctx, cache, out, scale: float, rows=None) -> None:
         if not self.prepared or self.has_out_bias:
             raise ValueError("an attention mixer beside another takes the float32 route and has no output bias")
-        self._inner_prepared(h, ctx, cache, ctx.groups[cache.group], out, scale)
+        self._inner_prepared(h, ctx, cache, ctx.groups[cache.group], out, scale, rows)
 
-    def _forward_prepared(self, h, ctx, cache, residual, view):
+    def _forward_prepared(self, h, ctx, cache, residual, view, rows=None):
         """The float32 route: projection with its bias, one kernel that norms, turns, scales, blends and stores,
         attention over heads of the cache's size, the output projection."""
         ops = self.ops
-        c = self._inner_prepared(h, ctx, cache, view, None, 1.0)
+        c = self._inner_prepared(h, ctx, cache, view, None, 1.0, rows)
         return ops.linear(c, self.w_out, self.b_out, residual=residual, out_f32=True, f32_by_library=residual is None)
 
-    def _inner_prepared(self, h, ctx, cache, view, out, out_scale):
+    def _inner_prepared(self, h, ctx, cache, view, out, out_scale, rows=None):
         ops = self.ops
-        proj = ops.linear(h, self.w_qkv, self.b_qkv, out_f32=True, f32_by_library=True)
+        proj = self._rows(h, rows)
         first = None
         if self.value_mix:
             key = ("value mix", self.value_mix["key"])
@@ -319,23 +326,23 @@ class Attention(Mixer):
                                     distance_bias=self.bias_by_distance, gate=gate, value_size=self.value_size,
                                     out=out, out_scale=out_scale, **more)
 
-    def forward(self, h, ctx, cache, residual):
+    def forward(self, h, ctx, cache, residual, rows=None):
         if cache.writes != self.own_kv:
             raise ValueError("an attention mixer with own_kv writes its cache; one without reads another's")
         view = ctx.groups[cache.group]
         if self.prepared:
-            return self._forward_prepared(h, ctx, cache, residual, view)
+            return self._forward_prepared(h, ctx, cache, residual, view, rows)
         kv_write = self.num_kv_heads if self.own_kv else 0
         if self.rotation is not None and self.turn is None:
             # the projections with their bias, turned by the encoding, then scaled and stored
-            qkv = self.ops.linear(h, self.w_qkv, self.b_qkv)
+            qkv = self.ops.linear(h, self.w_in, self.b_in)
             qkv = self.rotation.on_query_key(qkv, ctx, self.num_heads, kv_write, self.head_size)
             q = self.ops.qkv_write(qkv, None, self.num_heads, kv_write, self.head_size, self.scale, ctx, view,
                                    cache.k_pages, cache.v_pages)
             c = self.ops.attention(q, self.num_heads, self.num_kv_heads, self.head_size, ctx, view,
                                    cache.k_pages, cache.v_pages, self.window)
             return self.ops.linear(c, self.w_out, self.b_out, residual=residual, out_f32=True)
-        q = self.ops.qkv_project(h, self.w_qkv, self.b_qkv, self.num_heads,
+        q = self.ops.qkv_project(h, self.w_in, self.b_in, self.num_heads,
                                  self.num_kv_heads if self.own_kv else 0, self.head_size, self.scale, ctx, view,
                                  cache.k_pages, cache.v_pages, **({"turn": self.turn} if self.turn is not None else {}))
         c = self.ops.attention(q, self.num_heads, self.num_kv_heads, self.head_size, ctx, view,

@@ -9,7 +9,7 @@ from typing import Dict, List, Optional
 
 import torch
 
-from .base import MIXERS, POSITIONS, CacheNeed, Mixer, register_mixer
+from .base import MIXERS, POSITIONS, CacheNeed, Mixer, OffersRows, joined_rows, register_mixer
 from .spec import ParamDecl, PartSpec
 
 
@@ -314,7 +314,7 @@ class StateSpace(_LinearMemory):
         return ops.gated_norm(o, proj[:, :i], self.norm_weight, self.eps, self.norm_groups, True, skip=(self.skip, u[:, :i]))
 
 
-class _PlainMemory(_BesideAnother, Mixer):
+class _PlainMemory(OffersRows, _BesideAnother, Mixer):
     """What the mixers around a linear memory without convolutions share: per head a matrix S `[n, v]` that is carried
     from token to token,
 
@@ -342,13 +342,9 @@ class _PlainMemory(_BesideAnother, Mixer):
         return {"memory": memory_plan}
 
     def _load_in(self, tensors, names, ops):
-        """The rows of the input matrices one under the other, filled up with zero rows to a multiple of 16, and by 64
-        more where the product's rows would lie a power of two of bytes apart: the queries of all tokens of a prompt
-        would then share few memory channels."""
+        """The rows of the input matrices one under the other, filled up with zero rows to a multiple of 16."""
         w = torch.cat([tensors[n] for n in names], dim=0)
-        rows = w.shape[0] + -w.shape[0] % 16
-        rows += 64 if rows % 1024 == 0 else 0
-        return ops.prepare_weight(torch.nn.functional.pad(w, (0, 0, 0, rows - w.shape[0])).contiguous())
+        self._keep_in(ops, torch.nn.functional.pad(w, (0, 0, 0, -w.shape[0] % 16)).contiguous())
 
     def inner_width(self) -> int:
         return self.inner
@@ -357,9 +353,9 @@ class _PlainMemory(_BesideAnother, Mixer):
         """The decays' logarithms as `ops.linear_memory` takes them, after anything else that is done to `proj`."""
         raise NotImplementedError
 
-    def inner_into(self, h, ctx, cache, out, scale: float):
+    def inner_into(self, h, ctx, cache, out, scale: float, rows=None):
         ops, qk = self.ops, self.qk
-        proj = ops.linear(h, self.w_in, None, out_f32=True, f32_by_library=True)
+        proj = self._rows(h, rows)
         decay = self._decays(proj, ctx)
         at = 2 * qk + self.inner                                # the columns: q | k | v | gate | ...
         o = ops.linear_memory(proj[:, :at], 0, qk, 2 * qk, self.heads, self.heads, self.n, self.v, decay, None, ctx,
@@ -367,8 +363,8 @@ class _PlainMemory(_BesideAnother, Mixer):
         return ops.gated_norm(o, proj[:, at:at + self.inner], self.norm_weight, self.eps * self.n, self.heads, False,
                               out=out, out_scale=scale)
 
-    def forward(self, h, ctx, cache, residual):
-        y = self.inner_into(h, ctx, cache, None, 1.0)
+    def forward(self, h, ctx, cache, residual, rows=None):
+        y = self.inner_into(h, ctx, cache, None, 1.0, rows)
         return self.ops.linear(y, self.w_out, None, residual=residual, out_f32=True, f32_by_library=residual is None)
 
 
@@ -407,7 +403,7 @@ class GatedLinearAttention(_PlainMemory):
         if tuple(tensors[a2 + ws].shape) != (self.qk, self.rank):
             raise ValueError(f"{a2}{ws} is {tuple(tensors[a2 + ws].shape)}, behind a matrix of {self.rank} rows it must be "
                              f"{(self.qk, self.rank)}")
-        self.w_in = self._load_in(tensors, [n + ws for n in (q, k, v, g, a1)], ops)
+        self._load_in(tensors, [n + ws for n in (q, k, v, g, a1)], ops)
         self.w_decay, self.b_decay = tensors[a2 + ws].contiguous(), tensors[a2 + self.bias_suffix]
         self.norm_weight = tensors[norm].repeat(self.heads).contiguous()
         self._keep_out(ops, tensors[o + ws])
@@ -451,7 +447,7 @@ class Retention(_PlainMemory):
     def load(self, tensors: Dict, prefix: str, ops, dtype) -> None:
         super().load(tensors, prefix, ops, dtype)
         q, k, v, g, o = (prefix + n + self.weight_suffix for n in self.names)
-        self.w_in = self._load_in(tensors, [q, k, v, g], ops)
+        self._load_in(tensors, [q, k, v, g], ops)
         # (logarithms made in float64 and rounded once)
         self.log_decay = torch.log(torch.tensor(self.decay, dtype=torch.float64)).float().to(tensors[q].device)
         self.freqs = None
@@ -483,13 +479,14 @@ class _SubCache:
 
 
 @register_mixer("side_by_side")
-class SideBySide(Mixer):
+class SideBySide(OffersRows, Mixer):
     """Two mixers that read the same input, `left_scale * left(h) + right_scale * right(h)`.
 
     Both end in an output product; the two are made one: each mixer writes what its output matrix reads, times
     its factor, into its own columns of one buffer (`inner_into`), and the product of that buffer with the two
     output matrices side by side is the weighted sum, added up in float32. At most one of the two keeps pages;
-    the state of both lives in the one cache of the call, under the prefixes `left.` and `right.`.
+    the state of both lives in the one cache of the call, under the prefixes `left.` and `right.`. Where both offer the
+    rows of their input product (`OffersRows`), the two input products are one as well.
 
     With `out_norms` = {eps, left, right} each of the two results is first scaled to unit root mean square over the
     width and weighted (the tensors `left` and `right`, names under the mixer's prefix): each mixer then keeps its own
@@ -503,10 +500,16 @@ class SideBySide(Mixer):
             if not hasattr(m, "inner_into"):
                 raise ValueError(f"mixer {m.kind!r} cannot run beside another: it has no `inner_into`")
             m.defer_out = True
+        if self.offers_rows:
+            self.left.defer_in = self.right.defer_in = True
         self.left_name, self.right_name = left_name, right_name
         self.left_scale, self.right_scale = float(left_scale), float(right_scale)
         self.recordable = bool(getattr(self.left, "recordable", False) and getattr(self.right, "recordable", False))
         self._subs = {}
+
+    @property
+    def offers_rows(self) -> bool:
+        return self.out_norms is None and all(getattr(m, "offers_rows", False) for m in (self.left, self.right))
 
     def cache_need(self) -> Optional[CacheNeed]:
         needs = [(m.cache_need(), p) for m, p in ((self.left, "left."), (self.right, "right."))]
@@ -533,6 +536,9 @@ class SideBySide(Mixer):
         if self.out_norms:
             self.norm_weights = [tensors[prefix + self.out_norms[side]] for side in ("left", "right")]
             return
+        if self.offers_rows:
+            w, bias, self.places = joined_rows((self.left, self.right))
+            self._keep_in(ops, w, bias)
         self.split = self.left.inner_width()
         self.w_out = ops.prepare_weight(torch.cat([self.left.out_matrix(), self.right.out_matrix()], dim=1).contiguous())
 
@@ -558,7 +564,7 @@ class SideBySide(Mixer):
         return [(m.forward(h, ctx, sub, None), w, eps, scale) for m, sub, w, scale in
                 zip((self.left, self.right), subs[1:], self.norm_weights, (self.left_scale, self.right_scale))]
 
-    def forward(self, h, ctx, cache, residual):
+    def forward(self, h, ctx, cache, residual, rows=None):
         if self.out_norms:
             x = residual
             for y, w, eps, scale in self.results(h, ctx, cache):
@@ -566,6 +572,10 @@ class SideBySide(Mixer):
             return x
         subs = self._parts(cache)
         both = torch.empty(h.shape[0], self.split + self.right.inner_width(), dtype=self.dtype, device=self.ops.device)
-        self.left.inner_into(h, ctx, subs[1], both[:, :self.split], self.left_scale)
-        self.right.inner_into(h, ctx, subs[2], both[:, self.split:], self.right_scale)
+        left, right = {}, {}
+        if self.offers_rows:
+            rows = self._rows(h, rows)
+            left, right = ({"rows": rows[:, a:b]} for a, b in self.places)
+        self.left.inner_into(h, ctx, subs[1], both[:, :self.split], self.left_scale, **left)
+        self.right.inner_into(h, ctx, subs[2], both[:, self.split:], self.right_scale, **right)
         return self.ops.linear(both, self.w_out, None, residual=residual, out_f32=True, f32_by_library=residual is None)

@@ -62,7 +62,8 @@ def zudusun_spec(cfg: ZudusunConfig) -> ModelSpec:
         if cfg.owner(i) != i:
             continue
         place[i] = len(layers)
-        layers.append(LayerSpec(prefix=f"l{i}.", block="parallel", mixer=_mixer(cfg, layer["type"], layer["mixer"]),
+        layers.append(LayerSpec(prefix=f"l{i}.", block=PartSpec("parallel", dict(one_product=True)),
+                                mixer=_mixer(cfg, layer["type"], layer["mixer"]),
                                 feed_forward=_feed_forward(cfg, layer.get("mlp")), mixer_norm=norm,
                                 feed_forward_norm=no_norm, mixer_name="mix.", feed_forward_name="mlp.",
                                 mixer_norm_name="norm1", feed_forward_norm_name="norm2"))
