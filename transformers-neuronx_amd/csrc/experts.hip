@@ -303,22 +303,35 @@ __global__ void __launch_bounds__(256) expert_product_mfma_kernel(ProductArgs p)
     src[i] = n < p.n ? W + ((size_t)(row >> 4) * p.n + n) * p.k + lcol : nullptr;
   }
   f32x4 acc = {0.f, 0.f, 0.f, 0.f}, acc_up = {0.f, 0.f, 0.f, 0.f};
-  for (int k0 = 0; k0 < p.k; k0 += KC) {
-    bf16x8 got[LOADS];
+  // a chunk's rows and the pair's elements that meet them are asked for while the chunk before is multiplied
+  constexpr int STEPS = KC / 32;
+  bf16x8 got[LOADS], x_next[STEPS];
+  auto ask = [&](int k0) {
+#pragma unroll
+    for (int s = 0; s < STEPS; ++s) {
+      const int d = k0 + 32 * s + 8 * g;
+      x_next[s] = (pair >= 0 && d < p.k) ? *(const bf16x8*)(xrow + d) : zero8;
+    }
 #pragma unroll
     for (int i = 0; i < LOADS; ++i) got[i] = (src[i] != nullptr && k0 + lcol < p.k) ? load_once(src[i] + k0) : zero8;
+  };
+  ask(0);
+  for (int k0 = 0; k0 < p.k; k0 += KC) {
+    bf16x8 x[STEPS];
+#pragma unroll
+    for (int s = 0; s < STEPS; ++s) x[s] = x_next[s];
 #pragma unroll
     for (int i = 0; i < LOADS; ++i) *(bf16x8*)(mine + (RPI * i + lrow) * LD + lcol) = got[i];
-    const int steps = min(KC, p.k - k0);
-    for (int kk = 0; kk < steps; kk += 32) {
-      const int d0 = kk + 8 * g;
-      const bool in = k0 + d0 < p.k;
-      const bf16x8 b = (in && pair >= 0) ? *(const bf16x8*)(xrow + k0 + d0) : zero8;
+    if (k0 + KC < p.k) ask(k0 + KC);
+#pragma unroll
+    for (int s = 0; s < STEPS; ++s) {
+      if (k0 + 32 * s >= p.k) break;
+      const int d0 = 32 * s + 8 * g;
       const bf16x8 a = *(const bf16x8*)(mine + r * LD + d0);
-      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, x[s], acc, 0, 0, 0);
       if (GATED) {
         const bf16x8 u = *(const bf16x8*)(mine + (16 + r) * LD + d0);
-        acc_up = __builtin_amdgcn_mfma_f32_16x16x32_bf16(u, b, acc_up, 0, 0, 0);
+        acc_up = __builtin_amdgcn_mfma_f32_16x16x32_bf16(u, x[s], acc_up, 0, 0, 0);
       }
     }
   }

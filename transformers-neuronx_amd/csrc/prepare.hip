@@ -68,13 +68,13 @@ __device__ __forceinline__ float turned(const float* x, const float* w, float r,
   return first ? own * c - mate * s : own * c + mate * s;
 }
 
-// grid: (tokens, 3): a block takes a token's queries, its keys or its values; each of the three needs nothing of
-// the other two.
+// grid: (tokens, 3, shares): a block takes a share of a token's queries, keys or values; each of the three needs nothing
+// of the other two. (A norm over the whole projection is summed up by every block that shares it.)
 template <typename T>
 __global__ void __launch_bounds__(256) qkv_prepare_kernel(PrepareArgs a) {
   __shared__ float scratch[4];
   __shared__ float cosines[128], sines[128];       // of the token's angles, once for all heads
-  const int t = blockIdx.x, part = blockIdx.y;
+  const int t = blockIdx.x, part = blockIdx.y, share = blockIdx.z, shares = gridDim.z;
   const float* row = a.proj + (size_t)t * a.ld;
   const int nq = a.heads * a.n, nk = a.groups * a.n;
   const int page = a.token_page[t], off = a.token_offset[t];
@@ -84,7 +84,7 @@ __global__ void __launch_bounds__(256) qkv_prepare_kernel(PrepareArgs a) {
     T* vp = (T*)a.v_pages + (size_t)page * a.page_stride;
     const float lam = a.first != nullptr ? a.mix_weight[0] : 0.f;
     const float* first = a.first != nullptr ? a.first + (size_t)t * a.first_ld : nullptr;
-    for (int i = threadIdx.x; i < a.groups * a.d; i += 256) {
+    for (int i = threadIdx.x + 256 * share; i < a.groups * a.d; i += 256 * shares) {
       const int g = i / a.d, e = i - g * a.d;
       float val = 0.f;
       if (e < a.v) {
@@ -110,7 +110,7 @@ __global__ void __launch_bounds__(256) qkv_prepare_kernel(PrepareArgs a) {
     __syncthreads();       // the token's sines and cosines are there
     T* kp = part == 1 ? (T*)a.k_pages + (size_t)page * a.page_stride : nullptr;
     T* q_out = part == 0 ? (T*)a.q_out + (size_t)t * a.heads * a.d : nullptr;
-    for (int head = wave; head < heads; head += 4) {
+    for (int head = wave + 4 * share; head < heads; head += 4 * shares) {
       float s = 0.f;
       for (int e = lane; e < a.n; e += 64) s += x[head * a.n + e] * x[head * a.n + e];
       const float r = 1.f / sqrtf(wave_sum(s) / (float)a.n + a.eps);
@@ -134,7 +134,7 @@ __global__ void __launch_bounds__(256) qkv_prepare_kernel(PrepareArgs a) {
   __syncthreads();
   if (part == 0) {
     T* q_out = (T*)a.q_out + (size_t)t * a.heads * a.d;
-    for (int i = threadIdx.x; i < heads * a.d; i += 256) {
+    for (int i = threadIdx.x + 256 * share; i < heads * a.d; i += 256 * shares) {
       const int head = i / a.d, e = i - head * a.d;
       q_out[i] = from_f32<T>(e < a.n ? turned(x, w, norm, head, e, a, cosines, sines) *
                                            (a.head_scale ? scale * a.head_scale[head] : scale)
@@ -142,7 +142,7 @@ __global__ void __launch_bounds__(256) qkv_prepare_kernel(PrepareArgs a) {
     }
   } else {
     T* kp = (T*)a.k_pages + (size_t)page * a.page_stride;
-    for (int i = threadIdx.x; i < heads * a.d; i += 256) {
+    for (int i = threadIdx.x + 256 * share; i < heads * a.d; i += 256 * shares) {
       const int g = i / a.d, e = i - g * a.d;
       kp[((size_t)g * a.page_size + off) * a.d + e] = from_f32<T>(e < a.n ? turned(x, w, norm, g, e, a, cosines, sines) : 0.f);
     }
@@ -172,10 +172,13 @@ extern "C" int tnx_qkv_prepare(const float* proj, int ld, const float* q_weight,
   PrepareArgs a{proj, ld, q_weight, k_weight, eps, freqs, half, interleaved, positions, scale, mix_weight, first, first_ld,
                 token_page, token_offset, q_out, k_pages, v_pages, page_stride, num_pages, page_size, heads, groups, n, v, d,
                 per_head, values_at, head_scale, temp_coef, temp_every};
+  // few tokens: a token's heads over several blocks
+  int shares = 1;
+  while (shares < 8 && 6ll * tokens * shares <= tnx_compute_units() && heads * d >= 1024 * shares) shares *= 2;
   if (dtype == TNX_F32)
-    qkv_prepare_kernel<float><<<dim3(tokens, 3), 256, 0, stream>>>(a);
+    qkv_prepare_kernel<float><<<dim3(tokens, 3, shares), 256, 0, stream>>>(a);
   else
-    qkv_prepare_kernel<bf16_t><<<dim3(tokens, 3), 256, 0, stream>>>(a);
+    qkv_prepare_kernel<bf16_t><<<dim3(tokens, 3, shares), 256, 0, stream>>>(a);
   TNX_CHECK_LAUNCH("qkv_prepare");
   return 0;
 }
