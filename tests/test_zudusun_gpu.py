@@ -185,9 +185,17 @@ def test_decays_through_the_bottleneck(sizes, dtype):
     want = P.log_sigmoid(rows[:, 5:5 + rank].double() @ w.double().T + bias.double()) / 7.0
     got = ops.channel_decays(rows.to(DEV)[:, 5:5 + rank], w.to(DEV), bias.to(DEV), 7.0)
     _close(got, want, 1e-6)
-    near_zero = want.abs() < 1e-3            # a decay of almost one keeps its digits
+    near_zero = (want.abs() < 1e-3) & (want.abs() > 1e-12)       # a decay of almost one keeps its digits
     if bool(near_zero.any()):
         assert float(((got.double().cpu() - want).abs() / want.abs())[near_zero].max()) < 1e-4
+
+
+def test_the_logarithm_of_a_decay_keeps_its_digits():
+    """From pre-activations of -80 (the decay is almost 0) to 80 (almost 1: the logarithm is tiny)."""
+    z = torch.linspace(-80, 80, 40001)
+    want = P.log_sigmoid(z.double())
+    got = _ops(torch.float32).channel_decays(torch.zeros(1, 1, device=DEV), torch.zeros(z.numel(), 1, device=DEV), z.to(DEV), 1.0)
+    assert float(((got[0].double().cpu() - want) / want).abs().max()) < 1e-6
 
 
 @pytest.mark.parametrize("interleaved", [True, False])

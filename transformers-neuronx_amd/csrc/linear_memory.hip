@@ -202,6 +202,14 @@ __global__ void __launch_bounds__(256) memory_state_kernel(InputArgs a) {
     mine[(size_t)(a.positions[first + i] % a.taps) * a.channels + c] = a.proj[(size_t)(first + i) * a.ld + a.conv_at + c];
 }
 
+// ln(1 + x) for x in [0, 1] (Goldberg, "What Every Computer Scientist Should Know About Floating-Point Arithmetic", theorem
+// 4: the rounding of 1 + x drops out of x ln(u) / (u - 1) with u = 1 + x as rounded)
+__device__ __forceinline__ float log_one_plus(float x) {
+  const float u = 1.f + x;
+  return u == 1.f ? x : __fdividef(x * __logf(u), u - 1.f);
+}
+__device__ __forceinline__ float log_sigmoid(float z) { return fminf(z, 0.f) - log_one_plus(expf(-fabsf(z))); }
+
 // log_sigmoid(low w^T + bias) / tau for every key channel. A block takes 256 channels, one a thread, and TT tokens, whose
 // `low` goes through LDS 16 elements at a time.
 struct DecayArgs {
@@ -231,18 +239,29 @@ __global__ void __launch_bounds__(256) channel_decays_kernel(DecayArgs a) {
       low[threadIdx.x] = t0 + t < a.tokens && r0 + e < a.rank ? a.low[(size_t)(t0 + t) * a.low_ld + r0 + e] : 0.f;
     }
     float w[16];
+    if (a.rank % 16 == 0) {
+      typedef W eight __attribute__((ext_vector_type(8)));
+      const eight w0 = *(const eight*)(row + r0), w1 = *(const eight*)(row + r0 + 8);
 #pragma unroll
-    for (int e = 0; e < 16; ++e) w[e] = in && r0 + e < a.rank ? to_f32(row[r0 + e]) : 0.f;
+      for (int e = 0; e < 8; ++e) w[e] = to_f32(w0[e]), w[8 + e] = to_f32(w1[e]);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 16; ++e) w[e] = in && r0 + e < a.rank ? to_f32(row[r0 + e]) : 0.f;
+    }
     __syncthreads();
 #pragma unroll
     for (int t = 0; t < TT; ++t)
 #pragma unroll
-      for (int e = 0; e < 16; ++e) acc[t] = fmaf(w[e], low[16 * t + e], acc[t]);
+      for (int e = 0; e < 16; e += 4) {
+        const f32x4 l = *(const f32x4*)(low + 16 * t + e);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[t] = fmaf(w[e + i], l[i], acc[t]);
+      }
   }
   if (!in) return;
 #pragma unroll
   for (int t = 0; t < TT; ++t)
-    if (t0 + t < a.tokens) a.out[(size_t)(t0 + t) * a.channels + c] = -softplus(-(acc[t] + b)) * a.over_tau;
+    if (t0 + t < a.tokens) a.out[(size_t)(t0 + t) * a.channels + c] = log_sigmoid(acc[t] + b) * a.over_tau;
 }
 
 // The first 2 half elements of `heads` heads of n, from column `at` of a row on, turned by the token's position, in place:
@@ -1334,6 +1353,7 @@ extern "C" int tnx_channel_decays(const float* low, long long low_ld, const void
   TNX_REQUIRE(tokens >= 0 && channels > 0 && rank > 0 && low_ld >= rank, "channel_decays: bad sizes");
   TNX_REQUIRE(w_dtype == TNX_F32 || w_dtype == TNX_BF16, "channel_decays: dtype %d", w_dtype);
   TNX_REQUIRE(tokens < 16 * 65535, "channel_decays: too many tokens");
+  TNX_REQUIRE((uintptr_t)w % 32 == 0, "channel_decays: the matrix does not begin at a multiple of 32 bytes");
   if (tokens == 0) return 0;
   DecayArgs a{low, low_ld, w, bias, over_tau, out, tokens, channels, rank};
   const int blocks = (channels + 255) / 256;
