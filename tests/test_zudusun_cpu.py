@@ -311,6 +311,49 @@ def test_pages_and_slots_that_are_used_again():
         runner.finish(rid)
 
 
+@pytest.mark.parametrize("name", ["a", "b"])
+def test_one_product_for_all_that_reads_a_norm_is_the_products_of_each(name):
+    """The same model with the parts' input products apart, and the joined matrix's rows as the parts laid them."""
+    from dataclasses import replace
+    from transformers_neuronx_amd.engine.model import DecoderModel
+    from transformers_neuronx_amd.kernels import make_ops
+    from transformers_neuronx_amd.parts.spec import PartSpec
+    from transformers_neuronx_amd.weights.loader import TensorDict
+    cfg = zc.config(name)
+    w = zc.weights(cfg, 7)
+    runner = zc.runner(cfg, w)
+    toks = zc.requests(cfg, [25], 0)["r0"]
+    got = runner.step([StepEntry("r", toks, list(range(25)))])
+    spec = zudusun_spec(cfg)
+    apart = DecoderModel(replace(spec, layers=tuple(replace(l, block=PartSpec("parallel", {})) for l in spec.layers)))
+    ops = make_ops("reference", torch.float32, "cpu")
+    apart.load(TensorDict({k: v.clone() for k, v in w.items()}), ops, torch.float32, torch.device("cpu"))
+    assert any(l.block.joins for l in runner.model.layers) and not any(l.block.joins for l in apart.layers)
+    for layer in runner.model.layers:
+        if layer.block.joins:
+            matrix = layer.block.w_in
+            assert matrix.shape[0] % 16 == 0 and all(a % 16 == 0 for a, _ in layer.block.places)
+            assert not hasattr(layer.mixer, "w_in") and not hasattr(layer.feed_forward, "w_in")
+        else:
+            assert layer.mixer.w_in is not None
+    runner.finish("r")
+    runner.model = apart
+    other = runner.step([StepEntry("r", toks, list(range(25)))])
+    assert float((got - other).abs().max() / got.abs().max()) < 1e-5
+
+
+def test_rows_a_power_of_two_apart_are_moved():
+    from types import SimpleNamespace
+    from transformers_neuronx_amd.parts.base import joined_rows
+    part = lambda rows, bias: SimpleNamespace(in_matrix=lambda: (torch.full((rows, 3), float(rows)), bias))
+    w, bias, places = joined_rows((part(5, None), part(1000, torch.ones(1000))))
+    assert places == [(0, 5), (16, 1016)] and w.shape == (1024 + 64, 3)
+    assert float(w[:5].mean()) == 5.0 and float(w[16:1016].mean()) == 1000.0 and float(w[5:16].abs().sum() + w[1016:].abs().sum()) == 0
+    assert float(bias[16:1016].sum()) == 1000.0 and float(bias.sum()) == 1000.0
+    w, bias, _ = joined_rows((part(5, None), part(7, None)))
+    assert bias is None and w.shape == (32, 3)
+
+
 def test_layers_with_the_same_weights_keep_caches_of_their_own():
     cfg = zc.config("b")
     runner = zc.runner(cfg, zc.weights(cfg, 4))
